@@ -55,6 +55,16 @@ _cfgp = ctypes.POINTER(AwqConfig)
 SIGNATURES = {
     "awq_last_error": (ctypes.c_char_p, []),
     "awq_default_config": (None, [_cfgp]),
+    "awq_open": (ctypes.c_int, [ctypes.c_char_p, _vp, ctypes.POINTER(_vp)]),
+    "awq_architecture": (ctypes.c_char_p, [_vp]),
+    "awq_vocab_size": (_i64, [_vp]),
+    "awq_hidden_size": (_i64, [_vp]),
+    "awq_max_positions": (_i64, [_vp]),
+    "awq_forward": (ctypes.c_int, [_vp, _vp, _i32, _vp, _i32, _vp]),
+    "awq_read_hidden_f32": (ctypes.c_int, [_vp, _vp]),
+    "awq_read_logits_f32": (ctypes.c_int, [_vp, _vp]),
+    "awq_set_layer_tap": (ctypes.c_int, [_vp, ctypes.c_int]),
+    "awq_read_layer_tap": (_i64, [_vp, _vp, _i64]),
     "awq_validate_weight_dir": (ctypes.c_int, [ctypes.c_char_p, _cfgp]),
     "awq_create": (ctypes.c_int, [ctypes.c_char_p, _cfgp, ctypes.POINTER(_vp)]),
     "awq_create_empty": (ctypes.c_int, [_cfgp, ctypes.POINTER(_vp)]),
@@ -185,7 +195,123 @@ def _int32_array(values):
     return arr
 
 
-class QWen3AWQInfer:
+class AwqOpenOptions(ctypes.Structure):
+    """struct awq_open_options"""
+    _fields_ = [("dtype", _i32), ("reserved", _i32), ("max_positions", _i64)]
+
+
+DTYPES = {None: 0, "bfloat16": 1, "float32": 2}
+
+
+def open_model(model_dir, dtype=None, max_positions=0):
+    """An engine of the class that the folder's config.json names ("architecture"); a folder without one is the
+    raw weight directory of the int4 model.  dtype: None (the class's own), "bfloat16" or "float32"."""
+    lib = load_library()
+    h = _vp()
+    opt = AwqOpenOptions(DTYPES[dtype], 0, max_positions)
+    check(lib.awq_open(os.fsencode(model_dir), ctypes.byref(opt), ctypes.byref(h)))
+    return Engine(h)
+
+
+class Engine:
+    """A loaded model of any class: one sequence at a time, greedy generation."""
+
+    def __init__(self, handle):
+        self._lib = load_library()
+        self._h = handle
+
+    @property
+    def architecture(self):
+        return self._lib.awq_architecture(self._h).decode()
+
+    @property
+    def vocab_size(self):
+        return int(self._lib.awq_vocab_size(self._h))
+
+    @property
+    def hidden_size(self):
+        return int(self._lib.awq_hidden_size(self._h))
+
+    @property
+    def max_positions(self):
+        return int(self._lib.awq_max_positions(self._h))
+
+    def generateResponse(self, prompt_ids, max_new_tokens):
+        """Returns only the newly generated token ids (Inference.cu:361-366)."""
+        prompt = _int32_array(prompt_ids)
+        out = (ctypes.c_int32 * max(1, max_new_tokens))()
+        check(self._lib.awq_generate(self._h, prompt, len(prompt_ids), max_new_tokens, out))
+        return [int(out[i]) for i in range(max_new_tokens)]
+
+    # the same loop in pieces (timing)
+    def reset(self):
+        check(self._lib.awq_reset(self._h))
+
+    def prefill(self, prompt_ids, batched=False):
+        """The prompt loop; batched=True sends all positions through each layer together."""
+        fn = self._lib.awq_prefill_batched if batched else self._lib.awq_prefill
+        check(fn(self._h, _int32_array(prompt_ids), len(prompt_ids)))
+
+    def set_prefill_mode(self, batched):
+        """Which prompt loop generateResponse uses (default: token by token)."""
+        check(self._lib.awq_set_prefill_mode(self._h, 1 if batched else 0))
+
+    def decode(self, n_steps):
+        out = (ctypes.c_int32 * max(1, n_steps))()
+        check(self._lib.awq_decode(self._h, n_steps, out))
+        return [int(out[i]) for i in range(n_steps)]
+
+    def set_graph_mode(self, enabled):
+        check(self._lib.awq_set_graph_mode(self._h, 1 if enabled else 0))
+
+    def close(self):
+        if self._h:
+            self._lib.awq_destroy(self._h)
+            self._h = _vp()
+
+    def __del__(self):
+        try:
+            self.close()
+        except Exception:
+            pass
+
+    def forward(self, ids, want=()):
+        """The next tokens of the running sequence (reset() starts one); the logits at the places `want` among
+        them as [len(want)][vocab] binary32."""
+        import numpy as np
+        out = np.zeros((len(want), self.vocab_size), dtype=np.float32)
+        check(self._lib.awq_forward(self._h, _int32_array(ids), len(ids), _int32_array(want), len(want),
+                                    out.ctypes.data_as(_vp)))
+        return out
+
+    def read_hidden_f32(self):
+        import numpy as np
+        out = np.zeros(self.hidden_size, dtype=np.float32)
+        check(self._lib.awq_read_hidden_f32(self._h, out.ctypes.data_as(_vp)))
+        return out
+
+    def read_logits_f32(self):
+        import numpy as np
+        out = np.zeros(self.vocab_size, dtype=np.float32)
+        check(self._lib.awq_read_logits_f32(self._h, out.ctypes.data_as(_vp)))
+        return out
+
+    def set_layer_tap(self, on):
+        """Keep the residual stream behind every layer run of the passes that follow (read_layer_tap)."""
+        check(self._lib.awq_set_layer_tap(self._h, 1 if on else 0))
+
+    def read_layer_tap(self):
+        """[layer runs][tokens of the latest pass][hidden]"""
+        import numpy as np
+        n = int(self._lib.awq_read_layer_tap(self._h, None, 0))
+        if n < 0:
+            check(1)
+        out = np.zeros(n, dtype=np.float32)
+        self._lib.awq_read_layer_tap(self._h, out.ctypes.data_as(_vp), n)
+        return out
+
+
+class QWen3AWQInfer(Engine):
     """The reference's engine class (Inference.cu:356-366) on one MI355X.
 
     ``QWen3AWQInfer(weight_dir)`` loads the reference's .bin directory
@@ -193,6 +319,9 @@ class QWen3AWQInfer:
     Errors raise ``AwqError`` (the C++ class of the same name keeps the
     reference's print-and-exit(1)).
     """
+
+    FUSED_WO_W1 = 1      # Wo + residual and RMSNorm + W1 + GeLU of a layer as one launch
+    FUSED_QKV_ATTN = 2   # RMSNorm + Wqkv + rotary + KV append and the attention of a layer as one launch
 
     def __init__(self, weight_dir=None, config=None, _handle=None):
         self._lib = load_library()
@@ -239,34 +368,6 @@ class QWen3AWQInfer:
     def finalize(self):
         check(self._lib.awq_finalize(self._h))
 
-    def generateResponse(self, prompt_ids, max_new_tokens):
-        """Returns only the newly generated token ids (Inference.cu:361-366)."""
-        prompt = _int32_array(prompt_ids)
-        out = (ctypes.c_int32 * max(1, max_new_tokens))()
-        check(self._lib.awq_generate(self._h, prompt, len(prompt_ids), max_new_tokens, out))
-        return [int(out[i]) for i in range(max_new_tokens)]
-
-    # the same loop in pieces (timing)
-    def reset(self):
-        check(self._lib.awq_reset(self._h))
-
-    def prefill(self, prompt_ids, batched=False):
-        """The prompt loop; batched=True sends all positions through each layer together."""
-        fn = self._lib.awq_prefill_batched if batched else self._lib.awq_prefill
-        check(fn(self._h, _int32_array(prompt_ids), len(prompt_ids)))
-
-    def set_prefill_mode(self, batched):
-        """Which prompt loop generateResponse uses (default: token by token)."""
-        check(self._lib.awq_set_prefill_mode(self._h, 1 if batched else 0))
-
-    def decode(self, n_steps):
-        out = (ctypes.c_int32 * max(1, n_steps))()
-        check(self._lib.awq_decode(self._h, n_steps, out))
-        return [int(out[i]) for i in range(n_steps)]
-
-    FUSED_WO_W1 = 1      # Wo + residual and RMSNorm + W1 + GeLU of a layer as one launch
-    FUSED_QKV_ATTN = 2   # RMSNorm + Wqkv + rotary + KV append and the attention of a layer as one launch
-
     def set_fused_mode(self, mode):
         """Which pairs of a layer's launches run as one (a sum of FUSED_*; True means FUSED_WO_W1, False or 0
         none).  A pair the device cannot run fused stays two launches: fused_mode() tells what is on."""
@@ -274,9 +375,6 @@ class QWen3AWQInfer:
 
     def fused_mode(self):
         return int(self._lib.awq_fused_mode(self._h))
-
-    def set_graph_mode(self, enabled):
-        check(self._lib.awq_set_graph_mode(self._h, 1 if enabled else 0))
 
     def read_hidden(self):
         buf = (ctypes.c_uint16 * self.config.hidden)()
@@ -293,17 +391,6 @@ class QWen3AWQInfer:
         us, nbytes = _f32(0), _i64(0)
         check(self._lib.awq_time_linear(self._h, kind, n_rounds, ctypes.byref(us), ctypes.byref(nbytes)))
         return us.value, nbytes.value
-
-    def close(self):
-        if self._h:
-            self._lib.awq_destroy(self._h)
-            self._h = _vp()
-
-    def __del__(self):
-        try:
-            self.close()
-        except Exception:
-            pass
 
 
 def tensor_list(config):

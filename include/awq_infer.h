@@ -74,6 +74,43 @@ int awq_create_empty(const awq_config* cfg, awq_engine** out);
 int awq_upload(awq_engine* e, int layer, int kind, int part, const void* host_src, int64_t bytes);
 int awq_finalize(awq_engine* e);
 
+/* No counterpart in the reference: a model folder of any class of the registry.
+ * A folder with a config.json is opened by the class of its "architecture"
+ * entry (config.json + model.safetensors); one without is the raw weight
+ * directory of Inference.cu:780-899 with the reference's constants, as
+ * awq_create(dir, NULL, ...) opens it.  All fields 0 means the class's own
+ * defaults: its usual number format and its usual cache capacity. */
+#define AWQ_DTYPE_DEFAULT 0
+#define AWQ_DTYPE_BFLOAT16 1 /* 16-bit products and activations, 32-bit accumulation and residual */
+#define AWQ_DTYPE_FLOAT32 2  /* everything in binary32 */
+typedef struct awq_open_options {
+  int32_t dtype;
+  int32_t reserved;
+  int64_t max_positions; /* positions one sequence may hold, prompt and generated tokens together */
+} awq_open_options;
+int awq_open(const char* model_dir, const awq_open_options* options, awq_engine** out);
+const char* awq_architecture(const awq_engine* e);
+int64_t awq_vocab_size(const awq_engine* e);
+int64_t awq_hidden_size(const awq_engine* e);
+int64_t awq_max_positions(const awq_engine* e);
+
+/* No counterpart in the reference: the next n prompt tokens of the running
+ * sequence (awq_reset starts one), cut from the prompt anywhere; the logits at
+ * `want` (n_want ascending places among these tokens) go to host memory as
+ * [n_want][vocab] binary32.  Same passes and steps as awq_prefill_batched. */
+int awq_forward(awq_engine* e, const int32_t* ids, int32_t n, const int32_t* want, int32_t n_want, float* logits);
+/* awq_read_hidden / awq_read_logits in binary32, on an engine of any class (of
+ * an engine that keeps 16-bit values, those values) */
+int awq_read_hidden_f32(awq_engine* e, float* host_dst);
+int awq_read_logits_f32(awq_engine* e, float* host_dst);
+/* Test hook: with `on` non-zero the residual stream behind every layer run of
+ * the passes that follow is kept; awq_read_layer_tap hands out what the latest
+ * pass left, [layer runs][tokens][hidden] binary32, and returns the number of
+ * values (also with host_dst NULL), -1 when there is none.  Steps run as
+ * separate launches meanwhile. */
+int awq_set_layer_tap(awq_engine* e, int on);
+int64_t awq_read_layer_tap(awq_engine* e, float* host_dst, int64_t capacity);
+
 /* generateResponse, Inference.cu:1297-1408.  Writes max_new_tokens ids to
  * out_ids.  Restarts from an empty sequence on every call.  Fails (instead of
  * the reference's assert / cache overrun) when n_prompt + max_new_tokens >
