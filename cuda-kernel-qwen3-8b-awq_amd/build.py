@@ -1,8 +1,11 @@
-"""Compile the HIP library, the command-line harness and (optionally) the CPU oracle.
+"""Compile the HIP library, the command-line programs and (optionally) the CPU oracle.
 
 Run as a script or call build().  Everything lands in-tree next to this file
-(libawq_infer.so, qwen3_awq_infer) so that a source snapshot carries the
+(libawq_infer.so, qwen3_awq_infer, trace_run) so that a source snapshot carries the
 binaries along.
+
+`build.py --trace-run` compiles only what replaying traces needs: the step driver, the models that are
+described by a config.json and their kernels, linked into trace_run itself.
 """
 import os
 import subprocess
@@ -15,7 +18,15 @@ CSRC = os.path.join(HERE, "csrc")
 LIB = os.path.join(HERE, "libawq_infer.so")
 CLI = os.path.join(HERE, "qwen3_awq_infer")
 
-HIP_SOURCES = ["gemv.hip", "gemm.hip", "ops.hip", "prefill.hip", "attention.hip", "fused.hip", "qkv_attn.hip", "engine.cpp", "checkpoint.cpp", "qwen3.cpp", "kernel_api.cpp", "synth.cpp"]
+TRACE = os.path.join(HERE, "trace_run")
+
+# the step driver with the model registry and the operators every model uses
+CORE_SOURCES = ["engine.cpp", "checkpoint.cpp", "ops.hip"]
+# models described by a config.json
+CONFIG_MODEL_SOURCES = ["kugilix.cpp", "dense.hip", "token_ops.hip", "window_attention.hip", "linear_attention.hip"]
+# the int4 model of the raw weight directory and the kernel-level entry points
+INT4_SOURCES = ["gemv.hip", "gemm.hip", "prefill.hip", "attention.hip", "fused.hip", "qkv_attn.hip", "qwen3.cpp",
+                "kernel_api.cpp", "synth.cpp"]
 
 # -ffp-contract=off: every fma in the sources is written out; a contracted
 #   a*b-c*d would break bit parity with the reference's __hmul/__hsub sequence.
@@ -38,7 +49,8 @@ def _run(cmd):
     return res
 
 
-def build(verbose=False, oracle=True):
+def _compile(sources):
+    """object files of the sources, several compilers at a time"""
     hipcc = os.environ.get("HIPCC", "/opt/rocm/bin/hipcc")
     objdir = os.path.join(HERE, "build")
     os.makedirs(objdir, exist_ok=True)
@@ -48,10 +60,30 @@ def build(verbose=False, oracle=True):
         _run([hipcc] + HIPCC_FLAGS + ["-c", os.path.join(CSRC, src), "-o", obj])
         return obj
 
-    with ThreadPoolExecutor(max_workers=min(8, len(HIP_SOURCES))) as pool:
-        objs = list(pool.map(compile_one, HIP_SOURCES))
-    _run([hipcc, "--offload-arch=gfx950", "-shared", "-fopenmp", "-o", LIB] + objs)
-    # the drop-in C++ class and the reference's command line on top of the C ABI
+    with ThreadPoolExecutor(max_workers=min(8, len(sources))) as pool:
+        return dict(zip(sources, pool.map(compile_one, sources)))
+
+
+def _link_trace_run(objs):
+    hipcc = os.environ.get("HIPCC", "/opt/rocm/bin/hipcc")
+    part = "%s.%d" % (TRACE, os.getpid())
+    _run([hipcc, "--offload-arch=gfx950", "-fopenmp", "-o", part] +
+         [objs[s] for s in ["trace_run.cpp"] + CORE_SOURCES + CONFIG_MODEL_SOURCES])
+    os.replace(part, TRACE)
+
+
+def build_trace_run():
+    _link_trace_run(_compile(["trace_run.cpp"] + CORE_SOURCES + CONFIG_MODEL_SOURCES))
+    return TRACE
+
+
+def build(verbose=False, oracle=True):
+    hipcc = os.environ.get("HIPCC", "/opt/rocm/bin/hipcc")
+    library = CORE_SOURCES + CONFIG_MODEL_SOURCES + INT4_SOURCES
+    objs = _compile(library + ["trace_run.cpp"])
+    _run([hipcc, "--offload-arch=gfx950", "-shared", "-fopenmp", "-o", LIB] + [objs[s] for s in library])
+    _link_trace_run(objs)
+    # the drop-in C++ class and the command line on top of the C ABI
     _run([hipcc, "-O2", "-std=c++17", os.path.join(CSRC, "qwen3_awq_infer.cpp"), os.path.join(CSRC, "main.cpp"),
           "-o", CLI, "-L" + HERE, "-lawq_infer", "-Wl,-rpath,$ORIGIN"])
     if oracle:
@@ -62,4 +94,7 @@ def build(verbose=False, oracle=True):
 
 
 if __name__ == "__main__":
-    build(verbose=True)
+    if sys.argv[1:] == ["--trace-run"]:
+        print("built", build_trace_run())
+    else:
+        build(verbose=True)

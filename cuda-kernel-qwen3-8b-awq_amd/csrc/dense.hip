@@ -1,0 +1,388 @@
+// Dense products of bfloat16 (matrix cores) or binary32 weights with one token or many (layers.hpp).
+#include "layers.hpp"
+
+namespace {
+
+typedef float f32x4_t __attribute__((ext_vector_type(4)));
+typedef float f32x16_t __attribute__((ext_vector_type(16)));
+typedef const __attribute__((address_space(1))) void* gptr_t;
+typedef __attribute__((address_space(3))) void* lptr_t;
+
+__device__ __forceinline__ float sigmoid_f32(float z) { return 1.0f / (1.0f + __expf(-z)); }
+__device__ __forceinline__ float sigmoid_exact(float z) { return 1.0f / (1.0f + expf(-z)); }
+
+// exp(z) - 1 - z for z <= 0.  Near zero the difference cancels: there the series z^2/2 + z^3/6 + ...
+__device__ __forceinline__ float exp_minus_1_minus(float z) {
+  if (z > -0.25f) {
+    const float t = z * (1.0f / 7.0f) + 1.0f;
+    float s = __builtin_fmaf(z * (1.0f / 6.0f), t, 1.0f);
+    s = __builtin_fmaf(z * (1.0f / 5.0f), s, 1.0f);
+    s = __builtin_fmaf(z * (1.0f / 4.0f), s, 1.0f);
+    s = __builtin_fmaf(z * (1.0f / 3.0f), s, 1.0f);
+    return 0.5f * z * z * s;
+  }
+  return (expf(z) - 1.0f) - z;
+}
+
+template <bool F32>
+__device__ __forceinline__ float activate(const DenseSegment& s, int row, float z) {
+  if (s.act == DENSE_SILU) return row < s.act_rows ? z * (F32 ? sigmoid_exact(z) : sigmoid_f32(z)) : z;
+  if (s.act == DENSE_XIELU) {
+    const float h = 0.5f * z;
+    return z > 0.0f ? __builtin_fmaf(s.act_pos * z, z, h) : __builtin_fmaf(s.act_neg, exp_minus_1_minus(z), h);
+  }
+  return z;
+}
+
+__device__ __forceinline__ int32_t f32_key(float v) {
+  if (v != v) return INT32_MIN;  // NaN never wins
+  const uint32_t b = __float_as_uint(v);
+  if ((b & 0x7fffffffu) == 0) return 0;
+  return (b & 0x80000000u) ? -(int32_t)(b & 0x7fffffffu) : (int32_t)b;
+}
+
+__device__ __forceinline__ const DenseSegment& segment_of(const DenseArgs& a, int row) {
+  return a.n_seg > 1 && row >= a.seg[1].row0 ? a.seg[1] : a.seg[0];
+}
+
+// one finished sum of one token
+template <typename T, int OUT>
+__device__ __forceinline__ void finish_one(const DenseArgs& a, const DenseSegment& s, int64_t t, int row, float sum) {
+  const int64_t at = t * s.ldy + row;
+  if constexpr (OUT == DENSE_STORE) {
+    reinterpret_cast<T*>(s.y)[at] = (T)activate<sizeof(T) == 4>(s, row, sum);
+  } else if constexpr (OUT == DENSE_RESIDUAL) {
+    float* y = reinterpret_cast<float*>(s.y);
+    float v = y[at] + sum;
+    if (a.addend) v += a.addend[at];
+    y[at] = v;
+  } else {
+    reinterpret_cast<float*>(s.y)[at] = sum;
+  }
+}
+
+// --- one token, bfloat16 -----------------------------------------------------------------------------------
+// A workgroup owns 16 rows and all of k, its wavefronts a run of k each; a load of a wavefront is four pieces of 256
+// contiguous bytes of the block.  v_mfma_f32_16x16x32_bf16 with the token in every column: the matrix unit does the
+// additions, and nothing but loads stands between the wavefront and memory.
+template <int NW, int OUT>
+__global__ __launch_bounds__(NW * 64) void dense_one_kernel(DenseArgs a) {
+  __shared__ float part[NW][16];
+  const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const int row0 = blockIdx.x * 16;
+  const DenseSegment& s = segment_of(a, row0);
+  const int local = row0 - s.row0;
+  if (local >= s.rows) return;  // padding
+  const int steps = (int)(a.k >> 5);  // even: k is a multiple of 64
+  const int per = (steps + NW - 1) / NW;
+  const int s0 = min(wave * per, steps), s1 = min(s0 + per, steps);
+  const int r = lane & 15, c = lane >> 4;
+  // piece of (row, 8-wide chunk c of step i): block (row / 32, 2 i + c / 2), lane 32 (c % 2) + row % 32
+  const bf16x8_t* w = reinterpret_cast<const bf16x8_t*>(a.w) + ((int64_t)(row0 >> 5) * (a.k >> 4) + (c >> 1)) * 64 +
+                      32 * (c & 1) + (row0 & 16) + r;
+  const bf16x8_t* x = reinterpret_cast<const bf16x8_t*>(s.x) + c;
+  f32x4_t acc = {0.0f, 0.0f, 0.0f, 0.0f};
+  constexpr int U = 8;
+  int i = s0;
+  for (; i + U <= s1; i += U) {
+    bf16x8_t wv[U], xv[U];
+#pragma unroll
+    for (int u = 0; u < U; ++u) wv[u] = __builtin_nontemporal_load(w + (int64_t)(i + u) * 128);
+#pragma unroll
+    for (int u = 0; u < U; ++u) xv[u] = x[(i + u) * 4];
+#pragma unroll
+    for (int u = 0; u < U; ++u) acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wv[u], xv[u], acc, 0, 0, 0);
+  }
+  for (; i < s1; ++i)
+    acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_nontemporal_load(w + (int64_t)i * 128), x[i * 4], acc, 0, 0, 0);
+  if (r == 0) {
+#pragma unroll
+    for (int j = 0; j < 4; ++j) part[wave][4 * c + j] = acc[j];
+  }
+  __syncthreads();
+  if (tid >= 16) return;
+  float sum = 0.0f;
+#pragma unroll
+  for (int v = 0; v < NW; ++v) sum += part[v][tid];
+  const int row = local + tid;
+  if (row < s.rows) finish_one<bf16_t, OUT>(a, s, 0, row, sum);
+  if constexpr (OUT == DENSE_ARGMAX) {
+    unsigned long long b = row < s.rows ? awq_pack_candidate(f32_key(sum), (uint32_t)row) : 0ull;
+#pragma unroll
+    for (int off = 8; off > 0; off >>= 1) {
+      const unsigned long long o = __shfl_xor(b, off, 16);
+      b = o > b ? o : b;
+    }
+    if (tid == 0 && b > __hip_atomic_load(a.best, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT)) atomicMax(a.best, b);
+  }
+}
+
+// --- many tokens, bfloat16 ---------------------------------------------------------------------------------
+// A workgroup of four wavefronts takes 256 rows and 32 TT tokens: 64 rows per wavefront as 2 x TT accumulators of
+// v_mfma_f32_32x32x16_bf16.  The weights go from memory into registers in operand order, every byte once per
+// workgroup; the tokens go through LDS (global_load_lds_dwordx4, 128 bytes per token and step of 64 inputs, the
+// eight 16-byte pieces of row r at positions c ^ (r & 7)).  Both are requested a step ahead.
+template <int TT, int OUT>
+__global__ __launch_bounds__(256, 2) void dense_many_kernel(DenseArgs a, int row_tiles, int tok_tiles) {
+  __shared__ __attribute__((aligned(16))) bf16_t tile0[32 * TT * 64];
+  __shared__ __attribute__((aligned(16))) bf16_t tile1[32 * TT * 64];
+  const int total = row_tiles * tok_tiles;
+  // workgroups whose indices agree modulo 8 share a die: each die walks its own run of row tiles
+  const int per = (total + 7) >> 3;
+  const int work = (blockIdx.x & 7) * per + (blockIdx.x >> 3);
+  if (work >= total) return;
+  const int rt = work / tok_tiles, tt0 = (work - rt * tok_tiles) * 32 * TT;
+  const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const int n = lane & 31, kh = lane >> 5;
+  const DenseSegment& s = segment_of(a, rt * 256);
+  const int steps = (int)(a.k >> 6);
+  const int64_t k16 = a.k >> 4;
+
+  // this lane's pieces of the token tile
+  const bf16_t* src[TT];
+#pragma unroll
+  for (int i = 0; i < TT; ++i) {
+    const int row = (wave * TT + i) * 8 + (lane >> 3);
+    const int64_t tok = min((int64_t)tt0 + row, a.M - 1);
+    src[i] = reinterpret_cast<const bf16_t*>(s.x) + tok * s.ldx + (((lane & 7) ^ (row & 7)) << 3);
+  }
+  auto request = [&](bf16_t* tile, int step) __attribute__((always_inline)) {
+#pragma unroll
+    for (int i = 0; i < TT; ++i)
+      __builtin_amdgcn_global_load_lds((gptr_t)(src[i] + step * 64), (lptr_t)(tile + (wave * TT + i) * 8 * 64), 16, 0, 0);
+  };
+  const bf16x8_t* wp = reinterpret_cast<const bf16x8_t*>(a.w) + (int64_t)(rt * 8 + wave * 2) * k16 * 64 + lane;
+  auto weights = [&](bf16x8_t (&wv)[2][4], int step) __attribute__((always_inline)) {
+#pragma unroll
+    for (int b = 0; b < 2; ++b)
+#pragma unroll
+      for (int j = 0; j < 4; ++j) wv[b][j] = wp[(b * k16 + step * 4 + j) * 64];
+  };
+  f32x16_t acc[2][TT];
+#pragma unroll
+  for (int b = 0; b < 2; ++b)
+#pragma unroll
+    for (int t = 0; t < TT; ++t)
+#pragma unroll
+      for (int i = 0; i < 16; ++i) acc[b][t][i] = 0.0f;
+  auto multiply = [&](const bf16_t* tile, const bf16x8_t (&wv)[2][4]) __attribute__((always_inline)) {
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      bf16x8_t xv[TT];
+#pragma unroll
+      for (int t = 0; t < TT; ++t)
+        xv[t] = *reinterpret_cast<const bf16x8_t*>(tile + (32 * t + n) * 64 + (((2 * j + kh) ^ (n & 7)) << 3));
+#pragma unroll
+      for (int b = 0; b < 2; ++b)
+#pragma unroll
+        for (int t = 0; t < TT; ++t) acc[b][t] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(wv[b][j], xv[t], acc[b][t], 0, 0, 0);
+    }
+  };
+  bf16x8_t w0[2][4], w1[2][4];
+  request(tile0, 0);
+  weights(w0, 0);
+  for (int st = 0; st < steps; st += 2) {
+    __syncthreads();  // tile0 has arrived, tile1's readers are done
+    if (st + 1 < steps) {
+      request(tile1, st + 1);
+      weights(w1, st + 1);
+    }
+    multiply(tile0, w0);
+    if (st + 1 < steps) {
+      __syncthreads();
+      if (st + 2 < steps) {
+        request(tile0, st + 2);
+        weights(w0, st + 2);
+      }
+      multiply(tile1, w1);
+    }
+  }
+  // acc[b][t][i]: row 32 b + 8 (i / 4) + 4 kh + i % 4 of the wavefront's 64, token 32 t + n
+#pragma unroll
+  for (int t = 0; t < TT; ++t) {
+    const int64_t tok = (int64_t)tt0 + 32 * t + n;
+    if (tok >= a.M) continue;
+#pragma unroll
+    for (int b = 0; b < 2; ++b)
+#pragma unroll
+      for (int g = 0; g < 4; ++g) {
+        const int row = rt * 256 + wave * 64 + 32 * b + 8 * g + 4 * kh - s.row0;
+        const int64_t at = tok * s.ldy + row;
+        if (row + 3 < s.rows && (s.ldy & 3) == 0) {
+          if constexpr (OUT == DENSE_STORE) {
+            bf16x4_t v;
+#pragma unroll
+            for (int j = 0; j < 4; ++j) v[j] = (bf16_t)activate<false>(s, row + j, acc[b][t][4 * g + j]);
+            *reinterpret_cast<bf16x4_t*>(reinterpret_cast<bf16_t*>(s.y) + at) = v;
+          } else {
+            f32x4_t v;
+#pragma unroll
+            for (int j = 0; j < 4; ++j) v[j] = acc[b][t][4 * g + j];
+            f32x4_t* y = reinterpret_cast<f32x4_t*>(reinterpret_cast<float*>(s.y) + at);
+            if constexpr (OUT == DENSE_RESIDUAL) {
+              v = *y + v;
+              if (a.addend) v = v + *reinterpret_cast<const f32x4_t*>(a.addend + at);
+            }
+            *y = v;
+          }
+        } else {
+#pragma unroll
+          for (int j = 0; j < 4; ++j)
+            if (row + j < s.rows) finish_one<bf16_t, OUT>(a, s, tok, row + j, acc[b][t][4 * g + j]);
+        }
+      }
+  }
+}
+
+// --- binary32 ----------------------------------------------------------------------------------------------
+// one wavefront per row
+template <int OUT>
+__global__ __launch_bounds__(256) void dense_one_f32_kernel(DenseArgs a) {
+  const int lane = threadIdx.x & 63;
+  const int row = blockIdx.x * 4 + (threadIdx.x >> 6);
+  const DenseSegment& s = segment_of(a, row);
+  const int local = row - s.row0;
+  if (local >= s.rows) return;
+  const f32x4_t* w = reinterpret_cast<const f32x4_t*>(reinterpret_cast<const float*>(a.w) + (int64_t)row * a.k);
+  const f32x4_t* x = reinterpret_cast<const f32x4_t*>(s.x);
+  float acc = 0.0f;
+  for (int i = lane; i < (int)(a.k >> 2); i += 64) {
+    const f32x4_t wv = w[i], xv = x[i];
+#pragma unroll
+    for (int j = 0; j < 4; ++j) acc = __builtin_fmaf(wv[j], xv[j], acc);
+  }
+#pragma unroll
+  for (int off = 32; off > 0; off >>= 1) acc += __shfl_xor(acc, off, 64);
+  if (lane != 0) return;
+  finish_one<float, OUT>(a, s, 0, local, acc);
+  if constexpr (OUT == DENSE_ARGMAX) atomicMax(a.best, awq_pack_candidate(f32_key(acc), (uint32_t)local));
+}
+
+// 64 rows x 64 tokens per workgroup, 4 x 4 per thread, through LDS
+template <int OUT>
+__global__ __launch_bounds__(256) void dense_many_f32_kernel(DenseArgs a) {
+  __shared__ float ws[16][68], xs[16][68];
+  const int tid = threadIdx.x;
+  const int row0 = blockIdx.x * 64;
+  const int64_t tok0 = (int64_t)blockIdx.y * 64;
+  const DenseSegment& s = segment_of(a, row0);
+  if (row0 - s.row0 >= s.rows) return;
+  const int lr = tid >> 2, lk = (tid & 3) * 4;
+  const float* w = reinterpret_cast<const float*>(a.w) + (int64_t)(row0 + lr) * a.k + lk;
+  const float* x = reinterpret_cast<const float*>(s.x) + min(tok0 + lr, a.M - 1) * s.ldx + lk;
+  const int tr = (tid & 15) * 4, tc = (tid >> 4) * 4;
+  float acc[4][4] = {};
+  for (int k0 = 0; k0 < (int)a.k; k0 += 16) {
+    const f32x4_t wv = *reinterpret_cast<const f32x4_t*>(w + k0), xv = *reinterpret_cast<const f32x4_t*>(x + k0);
+    __syncthreads();
+#pragma unroll
+    for (int j = 0; j < 4; ++j) ws[lk + j][lr] = wv[j], xs[lk + j][lr] = xv[j];
+    __syncthreads();
+#pragma unroll
+    for (int k = 0; k < 16; ++k)
+#pragma unroll
+      for (int i = 0; i < 4; ++i)
+#pragma unroll
+        for (int j = 0; j < 4; ++j) acc[i][j] = __builtin_fmaf(ws[k][tr + i], xs[k][tc + j], acc[i][j]);
+  }
+#pragma unroll
+  for (int j = 0; j < 4; ++j)
+    if (tok0 + tc + j < a.M)
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const int row = row0 + tr + i - s.row0;
+        if (row < s.rows) finish_one<float, OUT>(a, s, tok0 + tc + j, row, acc[i][j]);
+      }
+}
+
+template <typename S>
+__global__ __launch_bounds__(256) void dense_pack_kernel(const S* __restrict__ src, int64_t rows, int64_t cols, void* w,
+                                                         int64_t k, int64_t row0, int64_t col0, int f32) {
+  const int64_t n = rows * cols;
+  for (int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x; i < n; i += (int64_t)gridDim.x * 256) {
+    const int64_t r = row0 + i / cols, c = col0 + i % cols;
+    if (f32)
+      reinterpret_cast<float*>(w)[r * k + c] = (float)src[i];
+    else
+      reinterpret_cast<bf16_t*>(w)[(((r >> 5) * (k >> 4) + (c >> 4)) * 64 + ((c >> 3) & 1) * 32 + (r & 31)) * 8 + (c & 7)] =
+          (bf16_t)(float)src[i];
+  }
+}
+
+template <int OUT>
+int launch_one(const DenseArgs& a, bool f32, int64_t rows, hipStream_t st) {
+  if (f32) {
+    hipLaunchKernelGGL(dense_one_f32_kernel<OUT>, dim3((unsigned)(rows / 4)), dim3(256), 0, st, a);
+  } else if (a.k > 8192) {
+    hipLaunchKernelGGL((dense_one_kernel<16, OUT>), dim3((unsigned)(rows / 16)), dim3(1024), 0, st, a);
+  } else if (a.k > 1024) {
+    hipLaunchKernelGGL((dense_one_kernel<8, OUT>), dim3((unsigned)(rows / 16)), dim3(512), 0, st, a);
+  } else {
+    hipLaunchKernelGGL((dense_one_kernel<4, OUT>), dim3((unsigned)(rows / 16)), dim3(256), 0, st, a);
+  }
+  AWQ_HIP_TRY(hipGetLastError());
+  return AWQ_OK;
+}
+
+template <int OUT>
+int launch_many(const DenseArgs& a, bool f32, int64_t rows, hipStream_t st) {
+  if (f32) {
+    hipLaunchKernelGGL(dense_many_f32_kernel<OUT>, dim3((unsigned)(rows / 64), (unsigned)((a.M + 63) / 64)), dim3(256), 0,
+                       st, a);
+  } else {
+    const int row_tiles = (int)(rows / 256);
+    // wide tiles once they fill the device
+    const int64_t wide = (a.M + 127) / 128;
+    if (row_tiles * wide >= 256) {
+      const unsigned grid = (unsigned)((row_tiles * wide + 7) / 8 * 8);
+      hipLaunchKernelGGL((dense_many_kernel<4, OUT>), dim3(grid), dim3(256), 0, st, a, row_tiles, (int)wide);
+    } else {
+      const int64_t narrow = (a.M + 63) / 64;
+      const unsigned grid = (unsigned)((row_tiles * narrow + 7) / 8 * 8);
+      hipLaunchKernelGGL((dense_many_kernel<2, OUT>), dim3(grid), dim3(256), 0, st, a, row_tiles, (int)narrow);
+    }
+  }
+  AWQ_HIP_TRY(hipGetLastError());
+  return AWQ_OK;
+}
+
+}  // namespace
+
+int64_t dense_weight_bytes(int64_t rows_padded, int64_t k_padded, bool f32) { return rows_padded * k_padded * (f32 ? 4 : 2); }
+
+int launch_dense_pack(const void* src, bool src_f32, int64_t rows, int64_t cols, void* w, int64_t k_padded, int64_t row0,
+                      int64_t col0, bool f32, hipStream_t st) {
+  AWQ_REQUIRE(rows > 0 && cols > 0 && k_padded % kDenseKAlign == 0 && col0 % 8 == 0 && col0 + cols <= k_padded, "bad block");
+  const unsigned grid = (unsigned)std::min<int64_t>((rows * cols + 255) / 256, 65536);
+  if (src_f32)
+    hipLaunchKernelGGL(dense_pack_kernel<float>, dim3(grid), dim3(256), 0, st, (const float*)src, rows, cols, w, k_padded,
+                       row0, col0, f32 ? 1 : 0);
+  else
+    hipLaunchKernelGGL(dense_pack_kernel<bf16_t>, dim3(grid), dim3(256), 0, st, (const bf16_t*)src, rows, cols, w, k_padded,
+                       row0, col0, f32 ? 1 : 0);
+  AWQ_HIP_TRY(hipGetLastError());
+  return AWQ_OK;
+}
+
+int launch_dense(const DenseArgs& a, bool f32, hipStream_t st) {
+  AWQ_REQUIRE(a.w && a.M >= 1 && a.k > 0 && a.k % kDenseKAlign == 0, "bad product");
+  AWQ_REQUIRE(a.n_seg == 1 || a.n_seg == 2, "one or two segments");
+  for (int i = 0; i < a.n_seg; ++i)
+    AWQ_REQUIRE(a.seg[i].x && a.seg[i].y && a.seg[i].rows > 0 && a.seg[i].row0 % kDenseRowAlign == 0 && a.seg[i].ldx % 8 == 0,
+                "bad segment");
+  AWQ_REQUIRE(a.n_seg == 1 || a.seg[1].row0 >= a.seg[0].row0 + a.seg[0].rows, "segments overlap");
+  const DenseSegment& last = a.seg[a.n_seg - 1];
+  const int64_t rows = round_up(last.row0 + last.rows, kDenseRowAlign);
+  AWQ_REQUIRE(rows < (1ll << 30) && a.M < (1ll << 30), "too large");
+  switch (a.out) {
+    case DENSE_STORE: return a.M == 1 ? launch_one<DENSE_STORE>(a, f32, rows, st) : launch_many<DENSE_STORE>(a, f32, rows, st);
+    case DENSE_RESIDUAL:
+      return a.M == 1 ? launch_one<DENSE_RESIDUAL>(a, f32, rows, st) : launch_many<DENSE_RESIDUAL>(a, f32, rows, st);
+    case DENSE_F32: return a.M == 1 ? launch_one<DENSE_F32>(a, f32, rows, st) : launch_many<DENSE_F32>(a, f32, rows, st);
+    case DENSE_ARGMAX:
+      AWQ_REQUIRE(a.M == 1 && a.best, "sampling takes one token");
+      return launch_one<DENSE_ARGMAX>(a, f32, rows, st);
+  }
+  awq_set_error("launch_dense: unknown output");
+  return AWQ_ERR_ARG;
+}

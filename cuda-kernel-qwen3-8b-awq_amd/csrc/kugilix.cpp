@@ -1,0 +1,732 @@
+// Kugilix: a decoder-only model of attention layers over a sliding window and linear-attention layers, parallel
+// mixer and feed-forward behind two grouped norms, a causal convolution in front of every mixer, a run of layers
+// that is repeated with the embedding added again, sinusoidal positions at the input.  config.json gives every size
+// and constant; the order of the layers is data.  Runs in bfloat16 (residual, norms, scores and recurrent state in
+// binary32) or wholly in binary32, behind the step driver of engine.cpp.
+//
+// A layer is four launches (five with linear attention):
+//   norms + convolution     x -> h = conv(norm1(x)) and n = norm2(x)
+//   one product             q, k, v (and the gate) of h, and act(W_up n): two segments of one weight block
+//   the mixer               -> ctx
+//   one product             x += [W_o | W_down] [ctx, mid], both halves in one block along k
+#include "engine.hpp"
+
+#include <math.h>
+#include <string.h>
+
+#include <chrono>
+#include <memory>
+
+#include "checkpoint.hpp"
+#include "layers.hpp"
+
+namespace {
+
+enum MixerType { MIX_ATTENTION, MIX_LIGHTNING };
+
+struct LayerSpec {
+  MixerType type = MIX_ATTENTION;
+  int32_t heads = 0, kv_heads = 0, dim = 0, vdim = 0;
+  int32_t window = 0;
+  float scale = 1.0f, temp_coef = 0.0f;
+  double temp_every = 1.0;
+  std::vector<float> decay;
+  int32_t ff = 0;  // 0: no feed-forward
+  int32_t mixed() const { return heads * vdim; }
+};
+
+struct Spec {
+  int32_t vocab = 0, width = 0, taps = 1, groups = 1;
+  float eps = 0.0f, embed_scale = 1.0f;
+  std::vector<LayerSpec> layers;
+  int32_t loop_start = 0, loop_stop = 0, loop_times = 1;
+};
+
+// --- config.json -------------------------------------------------------------------------------------------
+int bad_config(const std::string& why) {
+  awq_set_error("config.json: " + why);
+  return AWQ_ERR_ARG;
+}
+
+int get_number(const Json& j, const std::string& at, const char* key, double* out) {
+  const Json* v = j.find(key);
+  if (!v || !v->is(Json::Number)) return bad_config(at + key + " is missing or no number");
+  *out = v->number;
+  return AWQ_OK;
+}
+int get_int(const Json& j, const std::string& at, const char* key, double lo, double hi, int32_t* out) {
+  double d;
+  if (int rc = get_number(j, at, key, &d)) return rc;
+  if (!(d >= lo && d <= hi) || d != floor(d)) return bad_config(at + key + " is out of range");
+  *out = (int32_t)d;
+  return AWQ_OK;
+}
+int get_float(const Json& j, const std::string& at, const char* key, float* out) {
+  double d;
+  if (int rc = get_number(j, at, key, &d)) return rc;
+  *out = (float)d;
+  return AWQ_OK;
+}
+const Json* section(const Json& j, const char* key) {
+  const Json* v = j.find(key);
+  return v && v->is(Json::Object) ? v : nullptr;
+}
+
+int read_layer(const Json& j, const std::string& at, LayerSpec* s) {
+  const Json *type = j.find("type"), *m = section(j, "mixer");
+  if (!type || !type->is(Json::String) || !m) return bad_config(at + "type or mixer is missing");
+  const std::string mx = at + "mixer.";
+  constexpr double kMany = 1 << 20;
+  if (int rc = get_int(*m, mx, "heads", 1, 65535, &s->heads)) return rc;
+  if (int rc = get_int(*m, mx, "dim", 1, kMany, &s->dim)) return rc;
+  if (int rc = get_int(*m, mx, "vdim", 1, kMany, &s->vdim)) return rc;
+  if (type->str == "attention") {
+    s->type = MIX_ATTENTION;
+    if (int rc = get_int(*m, mx, "kv_heads", 1, 65535, &s->kv_heads)) return rc;
+    if (s->heads % s->kv_heads) return bad_config(mx + "heads is no multiple of kv_heads");
+    if (int rc = get_float(*m, mx, "scale", &s->scale)) return rc;
+    if (const Json* mask = section(*m, "mask"))
+      if (int rc = get_int(*mask, mx + "mask.", "size", 1, 1 << 30, &s->window)) return rc;
+    if (const Json* t = section(*m, "q_temp")) {
+      if (int rc = get_float(*t, mx + "q_temp.", "coef", &s->temp_coef)) return rc;
+      if (int rc = get_number(*t, mx + "q_temp.", "every", &s->temp_every)) return rc;
+      if (!(s->temp_every > 0.0)) return bad_config(mx + "q_temp.every must be positive");
+    }
+  } else if (type->str == "lightning") {
+    s->type = MIX_LIGHTNING;
+    const Json* d = m->find("decay");
+    if (!d || !d->is(Json::Array) || (int32_t)d->items.size() != s->heads) return bad_config(mx + "decay needs one number per head");
+    for (const Json& v : d->items) {
+      if (!v.is(Json::Number)) return bad_config(mx + "decay needs one number per head");
+      s->decay.push_back((float)v.number);
+    }
+  } else {
+    return bad_config(at + "type \"" + type->str + "\" is unknown");
+  }
+  const Json* f = j.find("mlp");
+  if (f && f->is(Json::Object)) {
+    const Json* kind = f->find("kind");
+    if (!kind || kind->str != "dense") return bad_config(at + "mlp.kind is unknown");
+    if (int rc = get_int(*f, at + "mlp.", "ff", 1, 1 << 28, &s->ff)) return rc;
+  }
+  return AWQ_OK;
+}
+
+int read_spec(const std::string& dir, Spec* s) {
+  Json j;
+  if (int rc = awq_read_json(dir + "/config.json", &j)) return rc;
+  if (int rc = get_int(j, "", "vocab", 1, 1 << 28, &s->vocab)) return rc;
+  if (int rc = get_int(j, "", "width", 1, 1 << 24, &s->width)) return rc;
+  const Json *norm = section(j, "norm"), *canon = section(j, "canon"), *emb = section(j, "embedding"), *layers = j.find("layers");
+  if (!norm || !canon || !emb) return bad_config("norm, canon or embedding is missing");
+  if (int rc = get_float(*norm, "norm.", "eps", &s->eps)) return rc;
+  if (int rc = get_int(*norm, "norm.", "groups", 1, 65535, &s->groups)) return rc;
+  if (s->width % s->groups) return bad_config("width is no multiple of norm.groups");
+  if (int rc = get_int(*canon, "canon.", "taps", 1, 1024, &s->taps)) return rc;
+  if (int rc = get_float(*emb, "embedding.", "scale", &s->embed_scale)) return rc;
+  if (!layers || !layers->is(Json::Array) || layers->items.empty() || layers->items.size() > 65535)
+    return bad_config("layers is missing or empty");
+  for (size_t i = 0; i < layers->items.size(); ++i) {
+    s->layers.emplace_back();
+    if (int rc = read_layer(layers->items[i], "layers[" + std::to_string(i) + "].", &s->layers.back())) return rc;
+  }
+  if (const Json* loop = section(j, "loop")) {
+    const double n = (double)s->layers.size();
+    if (int rc = get_int(*loop, "loop.", "start", 0, n, &s->loop_start)) return rc;
+    if (int rc = get_int(*loop, "loop.", "stop", s->loop_start, n, &s->loop_stop)) return rc;
+    if (int rc = get_int(*loop, "loop.", "times", 1, 4096, &s->loop_times)) return rc;
+  }
+  return AWQ_OK;
+}
+
+// --- the model ---------------------------------------------------------------------------------------------
+struct LayerDev {
+  const float *norm1 = nullptr, *norm2 = nullptr, *conv = nullptr;
+  void *w_in = nullptr, *w_out = nullptr;
+  int32_t rows_in = 0;           // of the first segment: q, k, v and the gate
+  int32_t up_row = 0;            // where the second segment, W_up, starts
+  int64_t ldp = 0;               // projections of a token
+  int64_t mixed_k = 0, k_out = 0;  // inputs of W_o and of both, padded
+  float act_pos = 0.0f, act_neg = 0.0f;
+  const float *mix_norm = nullptr, *decay = nullptr, *slope = nullptr;
+};
+
+// one run of a layer: a looped layer has one per pass
+struct LayerRun {
+  int32_t layer = 0;
+  bool add_embedding = false;  // the embedding output is added to x behind this run: another pass of the loop starts
+  float* conv_state[2] = {nullptr, nullptr};
+  float* state = nullptr;
+  void *k_cache = nullptr, *v_cache = nullptr;
+  RingLayout kl, vl;
+};
+
+// activations of a pass of up to `tokens` tokens
+struct Buffers {
+  int64_t tokens = 0;
+  float *x = nullptr, *keep = nullptr, *o = nullptr;
+  void *h = nullptr, *n = nullptr, *proj = nullptr;
+  std::vector<void*> cat;  // [ctx, mid] per layer (layers of one shape share)
+};
+
+constexpr int64_t kPassTokens = 2048;   // prompt positions per pass
+constexpr int64_t kLogitRows = 128;     // rows whose logits are formed at once
+constexpr int64_t kDefaultPositions = 8192;
+
+struct KugilixEngine final : awq_engine {
+  Spec spec;
+  bool f32 = false;
+  int64_t max_pos = 0, pass_tokens = 0;
+  int64_t ld = 0;  // a normalised token vector, padded
+  void *embed = nullptr, *head = nullptr;
+  const float* final_norm = nullptr;
+  const double* freq = nullptr;
+  std::vector<LayerDev> layers;
+  std::vector<LayerRun> runs;
+  Buffers step, pass;
+  int32_t* tokens = nullptr;
+  int32_t* rows = nullptr;  // which rows' logits are asked for
+  void* head_in = nullptr;  // [kLogitRows][ld]
+  float* logits = nullptr;  // [kLogitRows][vocab]
+  unsigned long long* best = nullptr;
+  float* attn_parts = nullptr;
+  int32_t* attn_counters = nullptr;
+  std::vector<int64_t> bounds;
+  bool tap_on = false, tap_saved_graphs = true;
+  float* tap = nullptr;
+  int64_t tap_tokens = 0;
+
+  const char* architecture() const override { return "Kugilix"; }
+  int64_t vocab_size() const override { return spec.vocab; }
+  int64_t hidden_size() const override { return spec.width; }
+  int64_t max_positions() const override { return max_pos; }
+  // nothing to clear: a run at position 0 reads neither convolution inputs nor recurrent state, and attention sees
+  // only rows of the running sequence
+  int begin_sequence() override { return AWQ_OK; }
+  const std::vector<int64_t>& length_bounds() const override { return bounds; }
+  int32_t epoch_step() const override { return 1; }
+  bool refeeds_hidden() const override { return false; }
+  int enqueue_step(StepKind kind, int64_t len_bound) override;
+  int64_t prompt_pass_tokens(int64_t done, int64_t rest) const override;
+  int enqueue_prompt_pass(const int32_t* ids, int64_t pos0, int64_t M) override;
+  int read_rows_logits(bool batched, const int32_t* which, int32_t n, float* host_dst) override;
+  int read_logits_f32(float* host_dst) override;
+  int read_hidden_f32(float* host_dst) override;
+  int set_layer_tap(int on) override;
+  int64_t read_layer_tap(float* host_dst, int64_t capacity) override;
+
+  int64_t unit() const { return f32 ? 4 : 2; }
+  int zeroed(void** p, int64_t bytes) {
+    bytes = round_up(std::max<int64_t>(bytes, 4), 4);
+    if (int rc = dev_alloc(p, bytes)) return rc;
+    return launch_fill_zero(*p, bytes, stream);
+  }
+  int load(const std::string& dir);
+  int make_buffers(Buffers* b, int64_t n_tokens);
+  int make_runs();
+  int run_layers(Buffers& b, int64_t M, PassPos pos);
+  int logits_of(const float* x, const int32_t* which, int64_t n, bool sample);
+};
+
+// --- weights -----------------------------------------------------------------------------------------------
+struct Loader {
+  KugilixEngine* e;
+  const Safetensors& file;
+  void* staging = nullptr;
+
+  // the tensor, its shape checked
+  int get(const std::string& name, const std::vector<int64_t>& shape, const Tensor** out) {
+    const Tensor* t = file.find(name);
+    if (!t) {
+      awq_set_error("model.safetensors has no tensor " + name);
+      return AWQ_ERR_IO;
+    }
+    if (t->shape != shape || (t->dtype != "BF16" && t->dtype != "F32")) {
+      awq_set_error("tensor " + name + " has another shape or type than config.json says");
+      return AWQ_ERR_IO;
+    }
+    *out = t;
+    return AWQ_OK;
+  }
+  int stage(const Tensor* t) {
+    AWQ_HIP_TRY(hipMemcpyAsync(staging, t->data, (size_t)t->bytes, hipMemcpyHostToDevice, e->stream));
+    return AWQ_OK;
+  }
+  static bool wide(const Tensor* t) { return t->dtype == "F32"; }
+  int vector(const std::string& name, std::vector<int64_t> shape, const float** out) {
+    const Tensor* t;
+    if (int rc = get(name, shape, &t)) return rc;
+    int64_t n = 1;
+    for (int64_t d : shape) n *= d;
+    float* dst = nullptr;
+    if (int rc = e->dev_alloc((void**)&dst, n * 4)) return rc;
+    if (int rc = stage(t)) return rc;
+    *out = dst;
+    return launch_convert(staging, wide(t), dst, true, n, e->stream);
+  }
+  int matrix(const std::string& name, int64_t rows, int64_t cols, void* w, int64_t k, int64_t row0, int64_t col0) {
+    const Tensor* t;
+    if (int rc = get(name, {rows, cols}, &t)) return rc;
+    if (int rc = stage(t)) return rc;
+    return launch_dense_pack(staging, wide(t), rows, cols, w, k, row0, col0, e->f32, e->stream);
+  }
+  int block(void** w, int64_t rows, int64_t k) { return e->zeroed(w, dense_weight_bytes(rows, k, e->f32)); }
+  int constants(const std::vector<float>& v, const float** out) {
+    float* dst = nullptr;
+    if (int rc = e->dev_alloc((void**)&dst, (int64_t)v.size() * 4)) return rc;
+    AWQ_HIP_TRY(hipMemcpy(dst, v.data(), v.size() * 4, hipMemcpyHostToDevice));
+    *out = dst;
+    return AWQ_OK;
+  }
+  int numbers(const std::string& name, int64_t n, std::vector<double>* out) {
+    const Tensor* t;
+    if (int rc = get(name, {n}, &t)) return rc;
+    out->clear();
+    for (int64_t i = 0; i < n; ++i) {
+      uint32_t bits;
+      if (wide(t))
+        memcpy(&bits, (const char*)t->data + 4 * i, 4);
+      else {
+        uint16_t h;
+        memcpy(&h, (const char*)t->data + 2 * i, 2);
+        bits = (uint32_t)h << 16;
+      }
+      float f;
+      memcpy(&f, &bits, 4);
+      out->push_back(f);
+    }
+    return AWQ_OK;
+  }
+};
+
+double softplus(double z) { return log1p(exp(-fabs(z))) + fmax(z, 0.0); }
+
+int load_layer(Loader& ld, KugilixEngine* e, int i) {
+  const LayerSpec& s = e->spec.layers[i];
+  const int64_t W = e->spec.width;
+  LayerDev L;
+  const std::string p = "l" + std::to_string(i) + ".", m = p + "mix.";
+  if (int rc = ld.vector(p + "norm1", {W}, &L.norm1)) return rc;
+  if (int rc = ld.vector(p + "canon1", {W, e->spec.taps}, &L.conv)) return rc;
+  struct Part {
+    const char* name;
+    int64_t rows;
+  };
+  std::vector<Part> parts;
+  if (s.type == MIX_ATTENTION)
+    parts = {{"q", (int64_t)s.heads * s.dim}, {"k", (int64_t)s.kv_heads * s.dim}, {"v", (int64_t)s.kv_heads * s.vdim}};
+  else
+    parts = {{"q", (int64_t)s.heads * s.dim}, {"k", (int64_t)s.heads * s.dim}, {"v", s.mixed()}, {"g", s.mixed()}};
+  int64_t rows = 0;
+  for (const Part& q : parts) rows += q.rows;
+  AWQ_REQUIRE(rows + s.ff < (1 << 28), "layer too large");
+  L.rows_in = (int32_t)rows;
+  L.ldp = round_up(rows, 8);
+  L.up_row = (int32_t)round_up(rows, kDenseRowAlign);
+  if (int rc = ld.block(&L.w_in, L.up_row + round_up(s.ff, kDenseRowAlign), e->ld)) return rc;
+  int64_t at = 0;
+  for (const Part& q : parts) {
+    if (int rc = ld.matrix(m + q.name, q.rows, W, L.w_in, e->ld, at, 0)) return rc;
+    at += q.rows;
+  }
+  L.mixed_k = round_up(s.mixed(), kDenseKAlign);
+  L.k_out = L.mixed_k + round_up(s.ff, kDenseKAlign);
+  if (int rc = ld.block(&L.w_out, round_up(W, kDenseRowAlign), L.k_out)) return rc;
+  if (int rc = ld.matrix(m + "o", W, s.mixed(), L.w_out, L.k_out, 0, 0)) return rc;
+  if (s.ff) {
+    if (int rc = ld.vector(p + "norm2", {W}, &L.norm2)) return rc;
+    if (int rc = ld.matrix(p + "mlp.up", s.ff, W, L.w_in, e->ld, L.up_row, 0)) return rc;
+    if (int rc = ld.matrix(p + "mlp.down", W, s.ff, L.w_out, L.k_out, 0, L.mixed_k)) return rc;
+    std::vector<double> act;
+    if (int rc = ld.numbers(p + "mlp.act", 2, &act)) return rc;
+    L.act_pos = (float)softplus(act[0]);
+    L.act_neg = (float)(0.5 + softplus(act[1]));
+  }
+  if (s.type == MIX_LIGHTNING) {
+    if (int rc = ld.vector(m + "norm", {s.mixed()}, &L.mix_norm)) return rc;
+    if (int rc = ld.constants(s.decay, &L.decay)) return rc;
+  } else {
+    std::vector<float> slope;
+    for (int h = 0; h < s.heads; ++h) slope.push_back((float)exp2(-8.0 * (h + 1) / s.heads));
+    if (int rc = ld.constants(slope, &L.slope)) return rc;
+  }
+  e->layers.push_back(L);
+  return AWQ_OK;
+}
+
+int KugilixEngine::load(const std::string& dir) {
+  const auto t0 = std::chrono::steady_clock::now();
+  Safetensors file;
+  if (int rc = file.open(dir + "/model.safetensors")) return rc;
+  Loader ldr{this, file};
+  int64_t largest = 4;
+  for (const auto& t : file.tensors()) largest = std::max(largest, t.second.bytes);
+  AWQ_HIP_TRY(hipMalloc(&ldr.staging, (size_t)largest));
+  const auto all = [&]() -> int {
+    const int64_t W = spec.width, V = spec.vocab;
+    ld = round_up(W, kDenseKAlign);
+    const Tensor* t;
+    if (int rc = ldr.get("embed", {V, W}, &t)) return rc;
+    if (int rc = dev_alloc(&embed, V * W * unit())) return rc;
+    if (int rc = ldr.stage(t)) return rc;
+    if (int rc = launch_convert(ldr.staging, Loader::wide(t), embed, f32, V * W, stream)) return rc;
+    if (int rc = ldr.vector("final.norm", {W}, &final_norm)) return rc;
+    if (int rc = ldr.block(&head, round_up(V, kDenseRowAlign), ld)) return rc;
+    if (int rc = ldr.matrix("head", V, W, head, ld, 0, 0)) return rc;
+    std::vector<double> f;
+    for (int64_t i = 0; 2 * i < W; ++i) f.push_back(pow(10000.0, -2.0 * (double)i / (double)W));
+    double* fd = nullptr;
+    if (int rc = dev_alloc((void**)&fd, (int64_t)f.size() * 8)) return rc;
+    AWQ_HIP_TRY(hipMemcpy(fd, f.data(), f.size() * 8, hipMemcpyHostToDevice));
+    freq = fd;
+    for (size_t i = 0; i < spec.layers.size(); ++i)
+      if (int rc = load_layer(ldr, this, (int)i)) return rc;
+    AWQ_HIP_TRY(hipStreamSynchronize(stream));
+    return AWQ_OK;
+  };
+  const int rc = all();
+  (void)hipStreamSynchronize(stream);  // nothing may still read the staging buffer or the mapped file
+  (void)hipFree(ldr.staging);
+  if (rc == AWQ_OK) awq_note_load_seconds(std::chrono::duration<double>(std::chrono::steady_clock::now() - t0).count());
+  return rc;
+}
+
+// --- activations, caches and recurrent state ---------------------------------------------------------------
+int KugilixEngine::make_buffers(Buffers* b, int64_t n) {
+  const int64_t W = spec.width;
+  int64_t proj = 0, o = 0;
+  b->cat.resize(layers.size());
+  for (size_t i = 0; i < layers.size(); ++i) {
+    proj = std::max(proj, layers[i].ldp);
+    if (spec.layers[i].type == MIX_LIGHTNING) o = std::max<int64_t>(o, spec.layers[i].mixed());
+    for (size_t j = 0; j < i && !b->cat[i]; ++j)
+      if (spec.layers[j].mixed() == spec.layers[i].mixed() && spec.layers[j].ff == spec.layers[i].ff) b->cat[i] = b->cat[j];
+    // the padding between and behind the two halves stays zero
+    if (!b->cat[i])
+      if (int rc = zeroed(&b->cat[i], n * layers[i].k_out * unit())) return rc;
+  }
+  if (int rc = zeroed((void**)&b->x, n * W * 4)) return rc;
+  if (int rc = zeroed((void**)&b->keep, n * W * 4)) return rc;
+  if (int rc = zeroed((void**)&b->o, n * o * 4)) return rc;
+  if (int rc = zeroed(&b->h, n * ld * unit())) return rc;
+  if (int rc = zeroed(&b->n, n * ld * unit())) return rc;
+  if (int rc = zeroed(&b->proj, n * proj * unit())) return rc;
+  b->tokens = n;
+  return AWQ_OK;
+}
+
+int KugilixEngine::make_runs() {
+  const int n = (int)spec.layers.size();
+  for (int i = 0; i < n;) {
+    if (i == spec.loop_start && spec.loop_stop > i) {
+      for (int t = 0; t < spec.loop_times; ++t)
+        for (int l = spec.loop_start; l < spec.loop_stop; ++l) {
+          LayerRun r;
+          r.layer = l;
+          r.add_embedding = l == spec.loop_stop - 1 && t + 1 < spec.loop_times;
+          runs.push_back(r);
+        }
+      i = spec.loop_stop;
+    } else {
+      LayerRun r;
+      r.layer = i++;
+      runs.push_back(r);
+    }
+  }
+  int64_t parts = 4, counters = 4;
+  for (LayerRun& r : runs) {
+    const LayerSpec& s = spec.layers[r.layer];
+    if (spec.taps > 1)
+      for (float*& p : r.conv_state)
+        if (int rc = zeroed((void**)&p, (int64_t)(spec.taps - 1) * spec.width * 4)) return rc;
+    if (s.type == MIX_LIGHTNING) {
+      if (int rc = zeroed((void**)&r.state, linear_state_floats(s.heads, s.dim, s.vdim) * 4)) return rc;
+      continue;
+    }
+    // a pass appends its rows before it attends: the ring holds a window behind the pass's first position
+    const int64_t need = s.window ? std::min<int64_t>(max_pos, (int64_t)s.window - 1 + pass_tokens) : max_pos;
+    r.kl = RingLayout{(int32_t)round_up(need, 64), s.kv_heads, window_row_padded(s.dim)};
+    r.vl = RingLayout{r.kl.slots, s.kv_heads, window_row_padded(s.vdim)};
+    if (int rc = zeroed(&r.k_cache, r.kl.elements() * unit())) return rc;
+    if (int rc = zeroed(&r.v_cache, r.vl.elements() * unit())) return rc;
+    parts = std::max(parts, window_parts_floats(s.heads, s.vdim, s.window, max_pos));
+    counters = std::max(counters, window_counter_count(s.heads, s.kv_heads));
+  }
+  if (int rc = zeroed((void**)&attn_parts, parts * 4)) return rc;
+  return zeroed((void**)&attn_counters, counters * 4);
+}
+
+// --- passes ------------------------------------------------------------------------------------------------
+int KugilixEngine::run_layers(Buffers& b, int64_t M, PassPos pos) {
+  const int64_t W = spec.width;
+  for (size_t ri = 0; ri < runs.size(); ++ri) {
+    const LayerRun& r = runs[ri];
+    const LayerSpec& s = spec.layers[r.layer];
+    const LayerDev& L = layers[r.layer];
+    void* const cat = b.cat[r.layer];
+    char* const mid = (char*)cat + L.mixed_k * unit();
+    {
+      NormConvArgs a;
+      a.x = b.x;
+      a.M = M;
+      a.width = W;
+      a.groups = spec.groups;
+      a.eps = spec.eps;
+      a.w1 = L.norm1;
+      a.conv = L.conv;
+      a.taps = spec.taps;
+      a.state[0] = r.conv_state[0];
+      a.state[1] = r.conv_state[1];
+      a.out1 = b.h;
+      a.w2 = L.norm2;
+      a.out2 = b.n;
+      a.ld = ld;
+      a.pos = pos;
+      if (int rc = launch_norm_conv(a, f32, stream)) return rc;
+    }
+    {
+      DenseArgs a;
+      a.w = L.w_in;
+      a.k = ld;
+      a.M = M;
+      DenseSegment& in = a.seg[0];
+      in.x = b.h;
+      in.ldx = ld;
+      in.y = b.proj;
+      in.ldy = L.ldp;
+      in.rows = L.rows_in;
+      if (s.type == MIX_LIGHTNING) {
+        in.act = DENSE_SILU;
+        in.act_rows = s.heads * (2 * s.dim + s.vdim);
+      }
+      if (s.ff) {
+        a.n_seg = 2;
+        DenseSegment& up = a.seg[1];
+        up.x = b.n;
+        up.ldx = ld;
+        up.y = mid;
+        up.ldy = L.k_out;
+        up.row0 = L.up_row;
+        up.rows = s.ff;
+        up.act = DENSE_XIELU;
+        up.act_pos = L.act_pos;
+        up.act_neg = L.act_neg;
+      }
+      if (int rc = launch_dense(a, f32, stream)) return rc;
+    }
+    if (s.type == MIX_ATTENTION) {
+      WindowAttnArgs a;
+      a.proj = b.proj;
+      a.ldp = L.ldp;
+      a.heads = s.heads;
+      a.kv_heads = s.kv_heads;
+      a.dim = s.dim;
+      a.vdim = s.vdim;
+      a.window = s.window;
+      a.scale = s.scale;
+      a.eps = spec.eps;
+      a.temp_coef = s.temp_coef;
+      a.temp_every = s.temp_every;
+      a.slope = L.slope;
+      a.k_cache = r.k_cache;
+      a.v_cache = r.v_cache;
+      a.kl = r.kl;
+      a.vl = r.vl;
+      a.ctx = cat;
+      a.ldc = L.k_out;
+      a.M = M;
+      a.pos = pos;
+      a.parts = attn_parts;
+      a.counters = attn_counters;
+      a.len_bound = (int32_t)max_pos;
+      if (int rc = launch_window_attention(a, f32, stream)) return rc;
+    } else {
+      LinearAttnArgs a;
+      a.proj = b.proj;
+      a.ldp = L.ldp;
+      a.heads = s.heads;
+      a.dim = s.dim;
+      a.vdim = s.vdim;
+      a.decay = L.decay;
+      a.state = r.state;
+      a.o = b.o;
+      a.M = M;
+      a.pos = pos;
+      if (int rc = launch_linear_attention(a, f32, stream)) return rc;
+      const char* gate = (const char*)b.proj + (int64_t)s.heads * (2 * s.dim + s.vdim) * unit();
+      if (int rc = launch_gated_norm(b.o, s.mixed(), gate, L.ldp, L.mix_norm, cat, L.k_out, s.mixed(), M, spec.eps, f32, stream))
+        return rc;
+    }
+    {
+      DenseArgs a;
+      a.w = L.w_out;
+      a.k = L.k_out;
+      a.M = M;
+      a.out = DENSE_RESIDUAL;
+      a.seg[0].x = cat;
+      a.seg[0].ldx = L.k_out;
+      a.seg[0].y = b.x;
+      a.seg[0].ldy = W;
+      a.seg[0].rows = (int32_t)W;
+      // the tap sees the stream as the layer leaves it
+      if (r.add_embedding && !tap_on) a.addend = b.keep;
+      if (int rc = launch_dense(a, f32, stream)) return rc;
+    }
+    if (tap_on) {
+      AWQ_HIP_TRY(hipMemcpyAsync(tap + (int64_t)ri * M * W, b.x, (size_t)(M * W) * 4, hipMemcpyDeviceToDevice, stream));
+      if (r.add_embedding)
+        if (int rc = launch_add_rows(b.x, b.keep, M * W, stream)) return rc;
+    }
+  }
+  if (tap_on) tap_tokens = M;
+  return AWQ_OK;
+}
+
+int KugilixEngine::logits_of(const float* x, const int32_t* which, int64_t n, bool sample) {
+  NormConvArgs a;
+  a.x = x;
+  a.rows = which;
+  a.M = n;
+  a.width = spec.width;
+  a.groups = spec.groups;
+  a.eps = spec.eps;
+  a.w1 = final_norm;
+  a.out1 = head_in;
+  a.ld = ld;
+  if (int rc = launch_norm_conv(a, f32, stream)) return rc;
+  DenseArgs d;
+  d.w = head;
+  d.k = ld;
+  d.M = n;
+  d.out = sample ? DENSE_ARGMAX : DENSE_F32;
+  d.best = best;
+  d.seg[0].x = head_in;
+  d.seg[0].ldx = ld;
+  d.seg[0].y = logits;
+  d.seg[0].ldy = spec.vocab;
+  d.seg[0].rows = spec.vocab;
+  return launch_dense(d, f32, stream);
+}
+
+int KugilixEngine::enqueue_step(StepKind kind, int64_t) {
+  PassPos pos;
+  pos.dyn = d_state;
+  if (kind != STEP_SAMPLE) {
+    if (int rc = launch_embed_sinusoid(embed, f32, nullptr, d_token, pos, 1, spec.width, spec.embed_scale, freq, step.x,
+                                       step.keep, stream))
+      return rc;
+    if (int rc = run_layers(step, 1, pos)) return rc;
+  }
+  if (kind == STEP_PROMPT) return AWQ_OK;
+  if (int rc = logits_of(step.x, nullptr, 1, true)) return rc;
+  return launch_take_best(best, d_token, d_out, d_state, kind == STEP_GENERATE ? 1 : 0, stream);
+}
+
+int64_t KugilixEngine::prompt_pass_tokens(int64_t, int64_t rest) const {
+  if (rest == 1 || pass_tokens < 2) return 0;
+  // equal passes of whole tiles rather than full ones and a small rest
+  const int64_t passes = (rest + pass_tokens - 1) / pass_tokens;
+  return std::min<int64_t>(rest, std::min<int64_t>(pass_tokens, round_up((rest + passes - 1) / passes, 128)));
+}
+
+int KugilixEngine::enqueue_prompt_pass(const int32_t* ids, int64_t pos0, int64_t M) {
+  PassPos pos;
+  pos.pos0 = (int32_t)pos0;
+  pos.epoch = epoch_next;
+  epoch_next = (epoch_next + 1) & 0x3fffffff;
+  AWQ_HIP_TRY(hipMemcpyAsync(tokens, ids, (size_t)M * 4, hipMemcpyHostToDevice, stream));
+  if (int rc = launch_embed_sinusoid(embed, f32, tokens, d_token, pos, M, spec.width, spec.embed_scale, freq, pass.x,
+                                     pass.keep, stream))
+    return rc;
+  if (int rc = run_layers(pass, M, pos)) return rc;
+  // the row the first generated token is sampled from
+  AWQ_HIP_TRY(hipMemcpyAsync(step.x, pass.x + (M - 1) * spec.width, (size_t)spec.width * 4, hipMemcpyDeviceToDevice, stream));
+  return AWQ_OK;
+}
+
+int KugilixEngine::read_rows_logits(bool batched, const int32_t* which, int32_t n, float* host_dst) {
+  for (int64_t at = 0; at < n; at += kLogitRows) {
+    const int64_t k = std::min<int64_t>(kLogitRows, n - at);
+    if (batched) AWQ_HIP_TRY(hipMemcpyAsync(rows, which + at, (size_t)k * 4, hipMemcpyHostToDevice, stream));
+    if (int rc = logits_of(batched ? pass.x : step.x, batched ? rows : nullptr, k, false)) return rc;
+    AWQ_HIP_TRY(hipMemcpyAsync(host_dst + at * spec.vocab, logits, (size_t)(k * spec.vocab) * 4, hipMemcpyDeviceToHost, stream));
+    AWQ_HIP_TRY(hipStreamSynchronize(stream));
+  }
+  return AWQ_OK;
+}
+
+int KugilixEngine::read_logits_f32(float* host_dst) {
+  AWQ_HIP_TRY(hipStreamSynchronize(stream));
+  AWQ_HIP_TRY(hipMemcpy(host_dst, logits, (size_t)spec.vocab * 4, hipMemcpyDeviceToHost));
+  return AWQ_OK;
+}
+
+int KugilixEngine::read_hidden_f32(float* host_dst) {
+  AWQ_HIP_TRY(hipStreamSynchronize(stream));
+  AWQ_HIP_TRY(hipMemcpy(host_dst, step.x, (size_t)spec.width * 4, hipMemcpyDeviceToHost));
+  return AWQ_OK;
+}
+
+int KugilixEngine::set_layer_tap(int on) {
+  AWQ_HIP_TRY(hipStreamSynchronize(stream));
+  if (on && !tap)
+    if (int rc = dev_alloc((void**)&tap, (int64_t)runs.size() * pass_tokens * spec.width * 4)) return rc;
+  if ((on != 0) != tap_on) {
+    if (on) {
+      tap_saved_graphs = graph_mode;
+      graph_mode = false;
+    } else {
+      graph_mode = tap_saved_graphs;
+    }
+  }
+  tap_on = on != 0;
+  tap_tokens = 0;
+  return AWQ_OK;
+}
+
+int64_t KugilixEngine::read_layer_tap(float* host_dst, int64_t capacity) {
+  if (!tap_on || tap_tokens == 0) {
+    awq_set_error("no pass was tapped");
+    return -1;
+  }
+  const int64_t n = (int64_t)runs.size() * tap_tokens * spec.width;
+  if (host_dst) {
+    if (hipStreamSynchronize(stream) != hipSuccess ||
+        hipMemcpy(host_dst, tap, (size_t)std::min(n, capacity) * 4, hipMemcpyDeviceToHost) != hipSuccess) {
+      awq_set_error("reading the tapped layers failed");
+      return -1;
+    }
+  }
+  return n;
+}
+
+int open_kugilix(const char* dir, const awq_open_options& opt, awq_engine** out) {
+  std::unique_ptr<KugilixEngine> e(new KugilixEngine());
+  if (int rc = read_spec(dir, &e->spec)) return rc;
+  e->f32 = opt.dtype == AWQ_DTYPE_FLOAT32;
+  e->max_pos = opt.max_positions ? opt.max_positions : kDefaultPositions;
+  AWQ_REQUIRE(e->max_pos <= (1 << 24), "max_positions is too large");
+  e->pass_tokens = std::min<int64_t>(kPassTokens, e->max_pos);
+  e->bounds = {1ll << 40};
+  e->batched_prefill = true;
+  if (int rc = e->init_driver(e->max_pos)) return rc;
+  if (int rc = e->load(dir)) return rc;
+  if (int rc = e->make_buffers(&e->step, 1)) return rc;
+  if (int rc = e->make_buffers(&e->pass, e->pass_tokens)) return rc;
+  if (int rc = e->make_runs()) return rc;
+  if (int rc = e->zeroed((void**)&e->tokens, e->pass_tokens * 4)) return rc;
+  if (int rc = e->zeroed((void**)&e->rows, kLogitRows * 4)) return rc;
+  if (int rc = e->zeroed(&e->head_in, kLogitRows * e->ld * e->unit())) return rc;
+  if (int rc = e->zeroed((void**)&e->logits, kLogitRows * e->spec.vocab * 4)) return rc;
+  if (int rc = e->zeroed((void**)&e->best, 8)) return rc;
+  if (int rc = launch_fill_zero(e->d_token, 4, e->stream)) return rc;
+  AWQ_HIP_TRY(hipStreamSynchronize(e->stream));
+  e->finalized = true;
+  if (int rc = awq_reset(e.get())) return rc;
+  *out = e.release();
+  return AWQ_OK;
+}
+
+ModelClass g_class("Kugilix", open_kugilix);
+
+}  // namespace

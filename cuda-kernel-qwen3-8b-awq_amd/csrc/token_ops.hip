@@ -1,0 +1,210 @@
+// Per-token operators of the layers in layers.hpp: embedding with a sinusoidal position vector, grouped RMS norms
+// with a causal convolution over time, a gated norm, and the end of a sampling step.
+#include "layers.hpp"
+
+namespace {
+
+template <typename S, typename D>
+__global__ __launch_bounds__(256) void convert_kernel(const S* __restrict__ src, D* __restrict__ dst, int64_t n) {
+  for (int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x; i < n; i += (int64_t)gridDim.x * 256) dst[i] = (D)(float)src[i];
+}
+
+__global__ __launch_bounds__(256) void add_rows_kernel(float* __restrict__ x, const float* __restrict__ y, int64_t n) {
+  const int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x;
+  if (i < n) x[i] += y[i];
+}
+
+// One thread per pair of entries.  The angle is formed and brought into [-pi, pi] in binary64: at a few thousand
+// positions a binary32 product would already be off by 1e-4.
+template <typename T>
+__global__ __launch_bounds__(256) void embed_sinusoid_kernel(const T* __restrict__ table, const int32_t* __restrict__ tokens,
+                                                             const int32_t* __restrict__ last, PassPos pos, int width,
+                                                             float scale, const double* __restrict__ freq,
+                                                             float* __restrict__ x, float* __restrict__ keep) {
+  const int t = blockIdx.y, i = blockIdx.x * 256 + threadIdx.x;
+  if (2 * i >= width) return;
+  int tok;
+  if (pos.dyn) {
+    tok = pos.dyn->token;
+    if (tok < 0) tok = *last;
+  } else {
+    tok = tokens[t];
+  }
+  const double angle = (double)(pos.position() + t) * freq[i];
+  const double turns = angle * 0.15915494309189533577;  // 1 / 2 pi
+  const float a = (float)((turns - rint(turns)) * 6.28318530717958647693);
+  float v[2] = {sinf(a), cosf(a)};
+#pragma unroll
+  for (int e = 0; e < 2; ++e)
+    if (2 * i + e < width) {
+      const int64_t at = (int64_t)t * width + 2 * i + e;
+      const float y = (float)table[(int64_t)tok * width + 2 * i + e] * scale + v[e];
+      x[at] = y;
+      if (keep) keep[at] = y;
+    }
+}
+
+// Tokens per workgroup.  The convolution needs the norms of the taps - 1 tokens ahead of a token: the workgroup
+// forms their statistics again rather than waiting for another workgroup's.
+constexpr int kNormTokens = 4;
+
+// blockIdx.x: token block, blockIdx.y: part of the vector
+template <typename T>
+__global__ __launch_bounds__(256) void norm_conv_kernel(NormConvArgs a) {
+  extern __shared__ float inv[];  // [kNormTokens + taps - 1]
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const int width = (int)a.width, part = width / a.groups, c0 = blockIdx.y * part;
+  const int t0 = blockIdx.x * kNormTokens, t1 = min(t0 + kNormTokens, (int)a.M);
+  const int back = a.conv ? a.taps - 1 : 0;
+  for (int t = t0 - back + wave; t < t1; t += 4) {
+    if (t < 0) continue;
+    const float* x = a.x + (int64_t)(a.rows ? a.rows[t] : t) * width + c0;
+    float acc = 0.0f;
+    for (int c = lane; c < part; c += 64) acc = __builtin_fmaf(x[c], x[c], acc);
+#pragma unroll
+    for (int off = 32; off > 0; off >>= 1) acc += __shfl_xor(acc, off, 64);
+    if (lane == 0) inv[t - t0 + back] = 1.0f / sqrtf(acc / (float)part + a.eps);
+  }
+  __syncthreads();
+  const int pos0 = a.conv ? a.pos.position() : 0, par = a.conv ? a.pos.parity() : 0;
+  const float* before = a.state[par];
+  float* after = a.state[par ^ 1];
+  const int keep0 = (int)a.M - back;  // tokens from here on go into the state
+  for (int c = c0 + tid; c < c0 + part; c += 256) {
+    const float w1 = a.w1[c], w2 = a.w2 ? a.w2[c] : 0.0f;
+    auto h_at = [&](int t) -> float {  // the first norm's output at token t of the pass, or ahead of it
+      if (t >= 0) return a.x[(int64_t)t * width + c] * inv[t - t0 + back] * w1;
+      return pos0 + t >= 0 ? before[(int64_t)(back + t) * width + c] : 0.0f;
+    };
+    if (blockIdx.x == 0)
+      for (int t = keep0; t < 0; ++t) after[(int64_t)(t - keep0) * width + c] = h_at(t);
+    for (int t = t0; t < t1; ++t) {
+      const float n = a.x[(int64_t)(a.rows ? a.rows[t] : t) * width + c] * inv[t - t0 + back];
+      const float h = n * w1;
+      float y = h;
+      if (a.conv) {
+        const float* k = a.conv + (int64_t)c * a.taps;
+        for (int j = 0; j < back; ++j) y = __builtin_fmaf(k[j], h_at(t - back + j), y);
+        y = __builtin_fmaf(k[back], h, y);
+        if (t >= keep0) after[(int64_t)(t - keep0) * width + c] = h;
+      }
+      reinterpret_cast<T*>(a.out1)[(int64_t)t * a.ld + c] = (T)y;
+      if (a.w2) reinterpret_cast<T*>(a.out2)[(int64_t)t * a.ld + c] = (T)(n * w2);
+    }
+  }
+}
+
+template <typename T>
+__global__ __launch_bounds__(256) void gated_norm_kernel(const float* __restrict__ o, int64_t ldo, const T* __restrict__ g,
+                                                         int64_t ldg, const float* __restrict__ w, T* __restrict__ y,
+                                                         int64_t ldy, int n, float eps) {
+  __shared__ float sums[4];
+  const int tid = threadIdx.x;
+  o += (int64_t)blockIdx.x * ldo;
+  g += (int64_t)blockIdx.x * ldg;
+  y += (int64_t)blockIdx.x * ldy;
+  float acc = 0.0f;
+  for (int i = tid; i < n; i += 256) acc = __builtin_fmaf(o[i], o[i], acc);
+#pragma unroll
+  for (int off = 32; off > 0; off >>= 1) acc += __shfl_xor(acc, off, 64);
+  if ((tid & 63) == 0) sums[tid >> 6] = acc;
+  __syncthreads();
+  const float inv = 1.0f / sqrtf(((sums[0] + sums[1]) + (sums[2] + sums[3])) / (float)n + eps);
+  for (int i = tid; i < n; i += 256) y[i] = (T)(o[i] * inv * w[i] * (1.0f / (1.0f + expf(-(float)g[i]))));
+}
+
+__global__ void take_best_kernel(unsigned long long* best, int32_t* out_token, int32_t* out_array, StepState* state,
+                                 int32_t epoch_step) {
+  if (threadIdx.x != 0) return;
+  const int32_t tok = (int32_t)(0xffffffffu - (uint32_t)(*best & 0xffffffffull));
+  *out_token = tok;
+  StepState s = *state;
+  if (out_array) out_array[s.out_index] = tok;
+  s.pos += 1;
+  s.len_lo = s.pos;
+  s.len_hi = s.pos + 1;
+  s.token = -1;
+  s.out_index += 1;
+  s.epoch += epoch_step;
+  *state = s;
+  *best = 0ull;
+}
+
+unsigned grid_for(int64_t n) { return (unsigned)std::max<int64_t>(1, std::min<int64_t>((n + 255) / 256, 65536)); }
+
+}  // namespace
+
+int launch_convert(const void* src, bool src_f32, void* dst, bool dst_f32, int64_t n, hipStream_t st) {
+  AWQ_REQUIRE(src && dst && n > 0, "bad arguments");
+  const dim3 g(grid_for(n)), b(256);
+  if (src_f32 && dst_f32)
+    hipLaunchKernelGGL((convert_kernel<float, float>), g, b, 0, st, (const float*)src, (float*)dst, n);
+  else if (src_f32)
+    hipLaunchKernelGGL((convert_kernel<float, bf16_t>), g, b, 0, st, (const float*)src, (bf16_t*)dst, n);
+  else if (dst_f32)
+    hipLaunchKernelGGL((convert_kernel<bf16_t, float>), g, b, 0, st, (const bf16_t*)src, (float*)dst, n);
+  else
+    hipLaunchKernelGGL((convert_kernel<bf16_t, bf16_t>), g, b, 0, st, (const bf16_t*)src, (bf16_t*)dst, n);
+  AWQ_HIP_TRY(hipGetLastError());
+  return AWQ_OK;
+}
+
+int launch_embed_sinusoid(const void* table, bool f32, const int32_t* tokens, const int32_t* last, PassPos pos, int64_t M,
+                          int64_t width, float scale, const double* freq, float* x, float* keep, hipStream_t st) {
+  AWQ_REQUIRE(table && freq && x && (pos.dyn ? last != nullptr && M == 1 : tokens != nullptr), "bad arguments");
+  AWQ_REQUIRE(M >= 1 && M <= 65535 && width >= 1 && width < (1 << 30), "bad shape");
+  const dim3 g((unsigned)(((width + 1) / 2 + 255) / 256), (unsigned)M);
+  if (f32)
+    hipLaunchKernelGGL(embed_sinusoid_kernel<float>, g, dim3(256), 0, st, (const float*)table, tokens, last, pos, (int)width,
+                       scale, freq, x, keep);
+  else
+    hipLaunchKernelGGL(embed_sinusoid_kernel<bf16_t>, g, dim3(256), 0, st, (const bf16_t*)table, tokens, last, pos,
+                       (int)width, scale, freq, x, keep);
+  AWQ_HIP_TRY(hipGetLastError());
+  return AWQ_OK;
+}
+
+int launch_norm_conv(const NormConvArgs& a, bool f32, hipStream_t st) {
+  AWQ_REQUIRE(a.x && a.w1 && a.out1 && a.M >= 1 && a.M < (1 << 30), "bad arguments");
+  AWQ_REQUIRE(a.groups >= 1 && a.groups <= 65535 && a.width >= a.groups && a.width % a.groups == 0 && a.ld >= a.width,
+              "bad shape");
+  AWQ_REQUIRE(!a.w2 || a.out2, "the second norm has no output");
+  AWQ_REQUIRE(!a.conv || (a.taps >= 1 && a.taps <= 1024 && !a.rows && (a.taps == 1 || (a.state[0] && a.state[1]))),
+              "bad convolution");
+  const dim3 g((unsigned)((a.M + kNormTokens - 1) / kNormTokens), (unsigned)a.groups);
+  const size_t lds = sizeof(float) * (kNormTokens + (a.conv ? a.taps - 1 : 0));
+  if (f32)
+    hipLaunchKernelGGL(norm_conv_kernel<float>, g, dim3(256), lds, st, a);
+  else
+    hipLaunchKernelGGL(norm_conv_kernel<bf16_t>, g, dim3(256), lds, st, a);
+  AWQ_HIP_TRY(hipGetLastError());
+  return AWQ_OK;
+}
+
+int launch_gated_norm(const float* o, int64_t ldo, const void* g, int64_t ldg, const float* w, void* y, int64_t ldy,
+                      int64_t n, int64_t M, float eps, bool f32, hipStream_t st) {
+  AWQ_REQUIRE(o && g && w && y && n >= 1 && n < (1 << 30) && M >= 1 && M < (1ll << 31), "bad arguments");
+  if (f32)
+    hipLaunchKernelGGL(gated_norm_kernel<float>, dim3((unsigned)M), dim3(256), 0, st, o, ldo, (const float*)g, ldg, w,
+                       (float*)y, ldy, (int)n, eps);
+  else
+    hipLaunchKernelGGL(gated_norm_kernel<bf16_t>, dim3((unsigned)M), dim3(256), 0, st, o, ldo, (const bf16_t*)g, ldg, w,
+                       (bf16_t*)y, ldy, (int)n, eps);
+  AWQ_HIP_TRY(hipGetLastError());
+  return AWQ_OK;
+}
+
+int launch_add_rows(float* x, const float* y, int64_t n, hipStream_t st) {
+  AWQ_REQUIRE(x && y && n > 0 && n < (1ll << 38), "bad arguments");
+  hipLaunchKernelGGL(add_rows_kernel, dim3((unsigned)((n + 255) / 256)), dim3(256), 0, st, x, y, n);
+  AWQ_HIP_TRY(hipGetLastError());
+  return AWQ_OK;
+}
+
+int launch_take_best(unsigned long long* best, int32_t* out_token, int32_t* out_array, StepState* state,
+                     int32_t epoch_step, hipStream_t st) {
+  AWQ_REQUIRE(best && out_token && state, "bad arguments");
+  hipLaunchKernelGGL(take_best_kernel, dim3(1), dim3(64), 0, st, best, out_token, out_array, state, epoch_step);
+  AWQ_HIP_TRY(hipGetLastError());
+  return AWQ_OK;
+}
