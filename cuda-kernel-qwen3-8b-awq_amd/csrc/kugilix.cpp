@@ -30,7 +30,7 @@ struct LayerSpec {
   int32_t window = 0;
   float scale = 1.0f, temp_coef = 0.0f;
   double temp_every = 1.0;
-  std::vector<float> decay;
+  std::vector<double> decay;
   int32_t ff = 0;  // 0: no feed-forward
   int32_t mixed() const { return heads * vdim; }
 };
@@ -98,7 +98,7 @@ int read_layer(const Json& j, const std::string& at, LayerSpec* s) {
     if (!d || !d->is(Json::Array) || (int32_t)d->items.size() != s->heads) return bad_config(mx + "decay needs one number per head");
     for (const Json& v : d->items) {
       if (!v.is(Json::Number)) return bad_config(mx + "decay needs one number per head");
-      s->decay.push_back((float)v.number);
+      s->decay.push_back(v.number);
     }
   } else {
     return bad_config(at + "type \"" + type->str + "\" is unknown");
@@ -148,7 +148,7 @@ struct LayerDev {
   int64_t ldp = 0;               // projections of a token
   int64_t mixed_k = 0, k_out = 0;  // inputs of W_o and of both, padded
   float act_pos = 0.0f, act_neg = 0.0f;
-  const float *mix_norm = nullptr, *decay = nullptr, *slope = nullptr;
+  const float *mix_norm = nullptr, *decay = nullptr, *log2_decay = nullptr, *slope = nullptr;
 };
 
 // one run of a layer: a looped layer has one per pass
@@ -344,7 +344,12 @@ int load_layer(Loader& ld, KugilixEngine* e, int i) {
   }
   if (s.type == MIX_LIGHTNING) {
     if (int rc = ld.vector(m + "norm", {s.mixed()}, &L.mix_norm)) return rc;
-    if (int rc = ld.constants(s.decay, &L.decay)) return rc;
+    if (int rc = ld.constants(std::vector<float>(s.decay.begin(), s.decay.end()), &L.decay)) return rc;
+    std::vector<float> lg;
+    for (double d : s.decay)
+      if (d > 0.0) lg.push_back((float)log2(d));
+    if (lg.size() == s.decay.size())
+      if (int rc = ld.constants(lg, &L.log2_decay)) return rc;
   } else {
     std::vector<float> slope;
     for (int h = 0; h < s.heads; ++h) slope.push_back((float)exp2(-8.0 * (h + 1) / s.heads));
@@ -548,6 +553,7 @@ int KugilixEngine::run_layers(Buffers& b, int64_t M, PassPos pos) {
       a.dim = s.dim;
       a.vdim = s.vdim;
       a.decay = L.decay;
+      a.log2_decay = L.log2_decay;
       a.state = r.state;
       a.o = b.o;
       a.M = M;

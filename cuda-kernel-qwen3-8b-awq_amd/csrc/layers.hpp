@@ -151,7 +151,8 @@ struct LinearAttnArgs {
   const void* proj = nullptr;  // [M][ldp]: heads * dim of q, heads * dim of k, heads * vdim of v
   int64_t ldp = 0;
   int32_t heads = 0, dim = 0, vdim = 0;
-  const float* decay = nullptr;  // [heads]
+  const float* decay = nullptr;       // [heads]
+  const float* log2_decay = nullptr;  // [heads], null unless every decay is positive: many tokens then go in chunks
   float* state = nullptr;
   float* o = nullptr;  // [M][heads * vdim]
   int64_t M = 0;

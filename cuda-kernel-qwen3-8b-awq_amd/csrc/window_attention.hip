@@ -100,11 +100,436 @@ __global__ __launch_bounds__(256) void window_query_kernel(WindowAttnArgs a) {
     if (c * 256 + tid < a.vdim) out[c * 256 + tid] = (T)(acc[c] / l);
 }
 
+// One token.  blockIdx.x: kv head and up to R of its query heads, blockIdx.y: part of the visible keys.  Every
+// workgroup normalises its queries; the one that holds the newest position normalises its key, uses key and value
+// from LDS and appends them.  Scores of a part sit in LDS; the parts' maxima, sums and contexts go to memory and the
+// workgroup that finishes last adds them up.
+constexpr int kPartKeys = 128;
+
+__host__ __device__ inline int window_parts(int64_t window, int64_t max_pos) {
+  const int64_t n = window > 0 && window < max_pos ? window : max_pos;
+  return (int)((n + kPartKeys - 1) / kPartKeys);
+}
+
 template <typename T>
-int launch_simple(const WindowAttnArgs& a, hipStream_t st) {
-  const dim3 ga((unsigned)((a.heads + 2 * a.kv_heads + 3) / 4), (unsigned)a.M);
-  hipLaunchKernelGGL(window_append_kernel<T>, ga, dim3(256), 0, st, a);
+struct Vec8;
+template <>
+struct Vec8<bf16_t> {
+  bf16x8_t v;
+  __device__ __forceinline__ void load(const bf16_t* p) { v = *reinterpret_cast<const bf16x8_t*>(p); }
+};
+template <>
+struct Vec8<float> {
+  typedef float f8 __attribute__((ext_vector_type(8)));
+  f8 v;
+  __device__ __forceinline__ void load(const float* p) { v = *reinterpret_cast<const f8*>(p); }
+};
+
+template <typename T, int R>
+__global__ __launch_bounds__(256) void window_decode_kernel(WindowAttnArgs a, int chunks) {
+  extern __shared__ float lds[];
+  __shared__ float inv[R + 1], part_m[R], part_l[R];
+  __shared__ int last;
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const int g = blockIdx.x / chunks, rz = (blockIdx.x - g * chunks) * R;
+  const int per_group = a.heads / a.kv_heads;
+  const int nr = min(R, per_group - rz), h0 = g * per_group + rz;
+  const int pos = a.pos.position();
+  const int lo = a.window > 0 ? max(0, pos - a.window + 1) : 0;
+  const int parts = (pos + 1 - lo + kPartKeys - 1) / kPartKeys;
+  const int part = blockIdx.y;
+  if (part >= parts) return;
+  const int b = lo + part * kPartKeys, e = min(b + kPartKeys, pos + 1), nk = e - b;
+  const bool newest = part == parts - 1;
+  const int kw = a.kl.row, vw = a.vl.row;
+  float* const sc = lds;                     // [R][kPartKeys]
+  float* const knew = sc + R * kPartKeys;    // [kw]
+  float* const vnew = knew + kw;             // [vw]
+  float* const red = vnew + vw;              // [4][R][vw]
+
+  const T* const proj = reinterpret_cast<const T*>(a.proj);
+  const T* const kp = proj + (int64_t)(a.heads + g) * a.dim;
+  for (int r = wave; r <= nr; r += 4) {  // row nr: the new key
+    const T* x = r < nr ? proj + (int64_t)(h0 + r) * a.dim : kp;
+    float acc = 0.0f;
+    for (int d = lane; d < a.dim; d += 64) acc = __builtin_fmaf((float)x[d], (float)x[d], acc);
+#pragma unroll
+    for (int off = 32; off > 0; off >>= 1) acc += __shfl_xor(acc, off, 64);
+    if (lane == 0) inv[r] = 1.0f / sqrtf(acc / (float)a.dim + a.eps);
+  }
+  __syncthreads();
+  if (newest) {
+    const T* vp = proj + (int64_t)(a.heads + a.kv_heads) * a.dim + (int64_t)g * a.vdim;
+    T* kd = reinterpret_cast<T*>(a.k_cache) + ring_row(a.kl, g, pos % a.kl.slots);
+    T* vd = reinterpret_cast<T*>(a.v_cache) + ring_row(a.vl, g, pos % a.vl.slots);
+    for (int d = tid; d < kw; d += 256) {
+      const T x = d < a.dim ? (T)((float)kp[d] * inv[nr]) : (T)0.0f;
+      knew[d] = (float)x;
+      if (rz == 0) kd[d] = x;
+    }
+    for (int d = tid; d < vw; d += 256) {
+      const T x = d < a.vdim ? vp[d] : (T)0.0f;
+      vnew[d] = (float)x;
+      if (rz == 0) vd[d] = x;
+    }
+  }
+  // lanes of a key: 8 of its elements each
+  const int lpk = kw >> 3, sub = lane / lpk, d0 = (lane - sub * lpk) * 8, kpw = 64 / lpk;
+  float qv[R][8];
+#pragma unroll
+  for (int r = 0; r < R; ++r)
+#pragma unroll
+    for (int i = 0; i < 8; ++i)
+      qv[r][i] = r < nr && d0 + i < a.dim ? (float)(T)((float)proj[(int64_t)(h0 + r) * a.dim + d0 + i] * inv[r]) : 0.0f;
+  __syncthreads();
+  const float mul = a.scale * temperature(a, pos);
+  const T* const kc = reinterpret_cast<const T*>(a.k_cache);
+  // four keys of a lane's group are requested before the first is multiplied
+  for (int k0 = wave * kpw; k0 < nk; k0 += 16 * kpw) {
+    Vec8<T> kv[4];
+#pragma unroll
+    for (int u = 0; u < 4; ++u) {
+      const int key = min(b + k0 + u * 4 * kpw + sub, pos);
+      if (key < pos) kv[u].load(kc + ring_row(a.kl, g, key % a.kl.slots) + d0);
+    }
+#pragma unroll
+    for (int u = 0; u < 4; ++u) {
+      const int i = k0 + u * 4 * kpw + sub, key = b + i;
+      float x[8];
+#pragma unroll
+      for (int j = 0; j < 8; ++j) x[j] = key < pos ? (float)kv[u].v[j] : newest ? knew[d0 + j] : 0.0f;
+#pragma unroll
+      for (int r = 0; r < R; ++r) {
+        float dot = 0.0f;
+#pragma unroll
+        for (int j = 0; j < 8; ++j) dot = __builtin_fmaf(qv[r][j], x[j], dot);
+        for (int off = lpk >> 1; off > 0; off >>= 1) dot += __shfl_xor(dot, off, 64);
+        if (d0 == 0 && i < nk && r < nr) sc[r * kPartKeys + i] = dot * mul - a.slope[h0 + r] * (float)(pos - key);
+      }
+    }
+  }
+  __syncthreads();
+  for (int r = wave; r < nr; r += 4) {
+    const float s0 = lane < nk ? sc[r * kPartKeys + lane] : -INFINITY;
+    const float s1 = lane + 64 < nk ? sc[r * kPartKeys + lane + 64] : -INFINITY;
+    float m = fmaxf(s0, s1);
+#pragma unroll
+    for (int off = 32; off > 0; off >>= 1) m = fmaxf(m, __shfl_xor(m, off, 64));
+    const float e0 = expf(s0 - m), e1 = expf(s1 - m);
+    float l = e0 + e1;
+#pragma unroll
+    for (int off = 32; off > 0; off >>= 1) l += __shfl_xor(l, off, 64);
+    sc[r * kPartKeys + lane] = e0;
+    sc[r * kPartKeys + lane + 64] = e1;
+    if (lane == 0) part_m[r] = m, part_l[r] = l;
+  }
+  __syncthreads();
+  // context: 8 columns of every kth key per thread
+  const int tpv = vw >> 3, c0 = (tid % tpv) * 8, first = tid / tpv, step = 256 / tpv;
+  float acc[R][8] = {};
+  const T* const vc = reinterpret_cast<const T*>(a.v_cache);
+  for (int k0 = first; k0 < nk; k0 += 4 * step) {
+    Vec8<T> vv[4];
+#pragma unroll
+    for (int u = 0; u < 4; ++u) {
+      const int key = min(b + k0 + u * step, pos);
+      if (key < pos) vv[u].load(vc + ring_row(a.vl, g, key % a.vl.slots) + c0);
+    }
+#pragma unroll
+    for (int u = 0; u < 4; ++u) {
+      const int i = k0 + u * step;
+      if (i >= nk) break;
+      float x[8];
+#pragma unroll
+      for (int j = 0; j < 8; ++j) x[j] = b + i < pos ? (float)vv[u].v[j] : vnew[c0 + j];
+#pragma unroll
+      for (int r = 0; r < R; ++r) {
+        if (r >= nr) break;
+        const float p = sc[r * kPartKeys + i];
+#pragma unroll
+        for (int j = 0; j < 8; ++j) acc[r][j] = __builtin_fmaf(p, x[j], acc[r][j]);
+      }
+    }
+  }
+  // lanes of a wavefront that share columns, then the wavefronts
+#pragma unroll
+  for (int r = 0; r < R; ++r)
+#pragma unroll
+    for (int j = 0; j < 8; ++j) {
+      for (int off = tpv; off < 64; off <<= 1) acc[r][j] += __shfl_xor(acc[r][j], off, 64);
+      if (lane < tpv) red[(wave * R + r) * vw + c0 + j] = acc[r][j];
+    }
+  __syncthreads();
+  T* const out = reinterpret_cast<T*>(a.ctx) + (int64_t)h0 * a.vdim;
+  auto total = [&](int r, int c) {
+    return (red[r * vw + c] + red[(R + r) * vw + c]) + (red[(2 * R + r) * vw + c] + red[(3 * R + r) * vw + c]);
+  };
+  if (parts == 1) {
+    for (int i = tid; i < nr * a.vdim; i += 256) {
+      const int r = i / a.vdim, c = i - r * a.vdim;
+      out[i] = (T)(total(r, c) / part_l[r]);
+    }
+    return;
+  }
+  // [head][part][2 + vdim]: maximum, sum, context
+  const int64_t ps = 2 + a.vdim, hs = (int64_t)gridDim.y * ps;
+  float* const mine = a.parts + (int64_t)h0 * hs + part * ps;
+  for (int i = tid; i < nr * a.vdim; i += 256) {
+    const int r = i / a.vdim, c = i - r * a.vdim;
+    __hip_atomic_store(mine + r * hs + 2 + c, total(r, c), __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+  }
+  if (tid < nr) {
+    __hip_atomic_store(mine + tid * hs, part_m[tid], __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+    __hip_atomic_store(mine + tid * hs + 1, part_l[tid], __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+  }
+  __threadfence();
+  __syncthreads();
+  if (tid == 0) {
+    const int n = __hip_atomic_fetch_add(a.counters + blockIdx.x, 1, __ATOMIC_ACQ_REL, __HIP_MEMORY_SCOPE_AGENT);
+    last = n == parts - 1;
+    if (last) __hip_atomic_store(a.counters + blockIdx.x, 0, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
+  }
+  __syncthreads();
+  if (!last) return;
+  __threadfence();
+  for (int i = tid; i < nr * a.vdim; i += 256) {
+    const int r = i / a.vdim, c = i - r * a.vdim;
+    const float* p = a.parts + (int64_t)(h0 + r) * hs;
+    float m = -INFINITY, l = 0.0f, x = 0.0f;
+    for (int s = 0; s < parts; ++s)
+      m = fmaxf(m, __hip_atomic_load(p + s * ps, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT));
+    for (int s = 0; s < parts; ++s) {
+      const float w = expf(__hip_atomic_load(p + s * ps, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT) - m);
+      l = __builtin_fmaf(w, __hip_atomic_load(p + s * ps + 1, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT), l);
+      x = __builtin_fmaf(w, __hip_atomic_load(p + s * ps + 2 + c, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT), x);
+    }
+    out[i] = (T)(x / l);
+  }
+}
+
+int decode_rows(const WindowAttnArgs& a) {
+  const int per = a.heads / a.kv_heads;
+  return per >= 8 ? 8 : per > 2 ? (per > 4 ? 8 : 4) : per;
+}
+
+template <typename T, int R>
+int launch_decode_rows(const WindowAttnArgs& a, hipStream_t st) {
+  const int chunks = (a.heads / a.kv_heads + R - 1) / R;
+  const int parts = window_parts(a.window, a.len_bound);
+  AWQ_REQUIRE(parts >= 1 && parts <= 65535, "too many keys");
+  const size_t lds = sizeof(float) * ((size_t)R * kPartKeys + a.kl.row + a.vl.row + (size_t)4 * R * a.vl.row);
+  hipLaunchKernelGGL((window_decode_kernel<T, R>), dim3((unsigned)(a.kv_heads * chunks), (unsigned)parts), dim3(256), lds, st,
+                     a, chunks);
   AWQ_HIP_TRY(hipGetLastError());
+  return AWQ_OK;
+}
+
+template <typename T>
+int launch_decode(const WindowAttnArgs& a, hipStream_t st) {
+  switch (decode_rows(a)) {
+    case 1: return launch_decode_rows<T, 1>(a, st);
+    case 2: return launch_decode_rows<T, 2>(a, st);
+    case 4: return launch_decode_rows<T, 4>(a, st);
+    default: return launch_decode_rows<T, 8>(a, st);
+  }
+}
+
+// Many tokens, bfloat16.  128 queries of one head per workgroup, 32 per wavefront; keys and values of 32 positions at
+// a time go through LDS.  Operands of v_mfma_f32_32x32x16_bf16, lane (n, kh) = (lane % 32, lane / 32), queries as
+// columns throughout:
+//     S^T[key][query] = K Q^T,   O^T[c][query] += V^T P^T
+// so that a query's maximum, sum and rescaling stay in a lane and its partner, and the weights a lane forms are the
+// elements it supplies to the second product (slice j: keys 16 j + 8 (e / 4) + 4 kh + e % 4; V^T by the transposing
+// LDS read).  Scores and weights are binary32; a weight enters the product as the sum of two bfloat16 terms.
+typedef float f32x16_t __attribute__((ext_vector_type(16)));
+typedef short short4_t __attribute__((ext_vector_type(4)));
+constexpr int kTileQueries = 128, kTileKeys = 32;
+
+template <int DK, int DV>
+__global__ __launch_bounds__(256, (DK + DV > 256) ? 1 : 2) void window_tile_kernel(WindowAttnArgs a) {
+  constexpr int KS = DK + 8, VS = DV + 16;
+  constexpr int KP = DK / 64, VP = DV / 64;  // 16-byte pieces of a tile per thread
+  __shared__ __attribute__((aligned(16))) bf16_t ks2[2 * kTileKeys * KS];
+  __shared__ __attribute__((aligned(16))) bf16_t vs2[2 * kTileKeys * VS];
+  const int h = blockIdx.x, g = h / (a.heads / a.kv_heads);
+  const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const int n = lane & 31, kh = lane >> 5;
+  const int M = (int)a.M, pos0 = a.pos.pos0;
+  const int q_first = blockIdx.y * kTileQueries;
+  const int qi = q_first + wave * 32 + n, qc = min(qi, M - 1);
+  const int pq = pos0 + qc;  // this lane's position
+  auto oldest = [&](int p) { return a.window > 0 ? max(0, p - a.window + 1) : 0; };
+  const int w_first = pos0 + min(q_first + wave * 32, M - 1), w_last = pos0 + min(q_first + wave * 32 + 31, M - 1);
+  const int lo_q = oldest(pq), lo_wave = oldest(w_first), lo_full = oldest(w_last);
+  const int k_begin = oldest(pos0 + q_first) & ~(kTileKeys - 1);
+  const int k_end = pos0 + min(q_first + kTileQueries - 1, M - 1) + 1;
+
+  const bf16_t* q = reinterpret_cast<const bf16_t*>(a.proj) + (int64_t)qc * a.ldp + (int64_t)h * a.dim;
+  bf16x8_t qop[DK / 16];
+#pragma unroll
+  for (int s = 0; s < DK / 16; ++s) {
+    const int at = 16 * s + 8 * kh;
+    if (a.dim == DK) {
+      qop[s] = *reinterpret_cast<const bf16x8_t*>(q + at);
+    } else {
+#pragma unroll
+      for (int e = 0; e < 8; ++e) qop[s][e] = at + e < a.dim ? q[at + e] : (bf16_t)0.0f;
+    }
+  }
+  f32x16_t o[DV / 32];
+#pragma unroll
+  for (int d = 0; d < DV / 32; ++d)
+#pragma unroll
+    for (int i = 0; i < 16; ++i) o[d][i] = 0.0f;
+  float m_run = -1e30f, l_run = 0.0f;
+  constexpr float kLog2e = 1.44269504088896340736f;
+  const float mul = a.scale * temperature(a, pq) * kLog2e, slope = a.slope[h] * kLog2e;
+
+  const bf16_t* const kc = reinterpret_cast<const bf16_t*>(a.k_cache);
+  const bf16_t* const vc = reinterpret_cast<const bf16_t*>(a.v_cache);
+  struct TileRegs {
+    bf16x8_t k[KP > 0 ? KP : 1], v[VP > 0 ? VP : 1];
+  };
+  TileRegs ra, rb;
+  auto load_tile = [&](int k0, TileRegs& r) __attribute__((always_inline)) {
+    if (k0 >= k_end) return;
+    const int slot = k0 % a.kl.slots;  // 32 positions from a multiple of 32 on never wrap
+#pragma unroll
+    for (int i = 0; i < KP; ++i) {
+      const int pc = tid + i * 256, key = pc / (DK / 8), at = (pc % (DK / 8)) * 8;
+      r.k[i] = *reinterpret_cast<const bf16x8_t*>(kc + ring_row(a.kl, g, slot + key) + at);
+    }
+#pragma unroll
+    for (int i = 0; i < VP; ++i) {
+      const int pc = tid + i * 256, key = pc / (DV / 8), at = (pc % (DV / 8)) * 8;
+      r.v[i] = *reinterpret_cast<const bf16x8_t*>(vc + ring_row(a.vl, g, slot + key) + at);
+    }
+  };
+  auto store_tile = [&](int half, const TileRegs& r) __attribute__((always_inline)) {
+#pragma unroll
+    for (int i = 0; i < KP; ++i) {
+      const int pc = tid + i * 256, key = pc / (DK / 8), at = (pc % (DK / 8)) * 8;
+      *reinterpret_cast<bf16x8_t*>(ks2 + (half * kTileKeys + key) * KS + at) = r.k[i];
+    }
+#pragma unroll
+    for (int i = 0; i < VP; ++i) {
+      const int pc = tid + i * 256, key = pc / (DV / 8), at = (pc % (DV / 8)) * 8;
+      *reinterpret_cast<bf16x8_t*>(vs2 + (half * kTileKeys + key) * VS + at) = r.v[i];
+    }
+  };
+  auto step = [&](int k0, int half) __attribute__((always_inline)) {
+    if (k0 > w_last || k0 + kTileKeys <= lo_wave) return;  // no query of this wavefront sees a key of the tile
+    const bf16_t* ks = ks2 + half * kTileKeys * KS;
+    const bf16_t* vs = vs2 + half * kTileKeys * VS;
+    f32x16_t s;
+#pragma unroll
+    for (int i = 0; i < 16; ++i) s[i] = 0.0f;
+#pragma unroll
+    for (int d = 0; d < DK / 16; ++d)
+      s = __builtin_amdgcn_mfma_f32_32x32x16_bf16(*reinterpret_cast<const bf16x8_t*>(ks + n * KS + 16 * d + 8 * kh), qop[d], s,
+                                                  0, 0, 0);
+    // s[i]: key k0 + 8 (i / 4) + 4 kh + i % 4 for this lane's query
+    const int base = k0 + 4 * kh - pq;
+#pragma unroll
+    for (int i = 0; i < 16; ++i) s[i] = __builtin_fmaf(s[i], mul, slope * (float)(base + 8 * (i >> 2) + (i & 3)));
+    if (k0 + kTileKeys - 1 > w_first || k0 < lo_full) {
+#pragma unroll
+      for (int i = 0; i < 16; ++i) {
+        const int key = k0 + 8 * (i >> 2) + 4 * kh + (i & 3);
+        s[i] = key <= pq && key >= lo_q ? s[i] : -INFINITY;
+      }
+    }
+    float mx = s[0];
+#pragma unroll
+    for (int i = 1; i < 16; ++i) mx = fmaxf(mx, s[i]);
+    mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
+    const float m_new = fmaxf(m_run, mx);
+    const float alpha = __builtin_amdgcn_exp2f(m_run - m_new);
+    float rs = 0.0f;
+    bf16x8_t hi[2], lo[2];
+#pragma unroll
+    for (int i = 0; i < 16; ++i) {
+      const float p = __builtin_amdgcn_exp2f(s[i] - m_new);
+      rs += p;
+      hi[i >> 3][i & 7] = (bf16_t)p;
+      lo[i >> 3][i & 7] = (bf16_t)(p - (float)hi[i >> 3][i & 7]);
+    }
+    rs += __shfl_xor(rs, 32, 64);
+    l_run = l_run * alpha + rs;
+    m_run = m_new;
+    if (__builtin_amdgcn_ballot_w64(alpha != 1.0f) != 0) {
+#pragma unroll
+      for (int d = 0; d < DV / 32; ++d)
+#pragma unroll
+        for (int i = 0; i < 16; ++i) o[d][i] *= alpha;
+    }
+    const int L16 = lane & 15;
+    const bf16_t* vlane = vs + (4 * kh + (L16 >> 2)) * VS + 16 * ((lane >> 4) & 1) + 4 * (L16 & 3);
+#pragma unroll
+    for (int j = 0; j < 2; ++j)
+#pragma unroll
+      for (int d = 0; d < DV / 32; ++d) {
+        const bf16_t* vp = vlane + 16 * j * VS + d * 32;
+        const short4_t l = __builtin_amdgcn_ds_read_tr16_b64_v4i16((short4_t __attribute__((address_space(3)))*)vp);
+        const short4_t u = __builtin_amdgcn_ds_read_tr16_b64_v4i16((short4_t __attribute__((address_space(3)))*)(vp + 8 * VS));
+        const bf16x4_t l4 = __builtin_bit_cast(bf16x4_t, l), u4 = __builtin_bit_cast(bf16x4_t, u);
+        const bf16x8_t vv = {l4[0], l4[1], l4[2], l4[3], u4[0], u4[1], u4[2], u4[3]};
+        o[d] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(vv, hi[j], o[d], 0, 0, 0);
+        o[d] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(vv, lo[j], o[d], 0, 0, 0);
+      }
+  };
+  load_tile(k_begin, ra);
+  load_tile(k_begin + kTileKeys, rb);
+  for (int k0 = k_begin; k0 < k_end; k0 += 2 * kTileKeys) {
+    __syncthreads();  // the previous tiles' readers are done
+    store_tile(0, ra);
+    if (k0 + kTileKeys < k_end) store_tile(1, rb);
+    __syncthreads();
+    load_tile(k0 + 2 * kTileKeys, ra);
+    load_tile(k0 + 3 * kTileKeys, rb);
+    step(k0, 0);
+    if (k0 + kTileKeys < k_end) step(k0 + kTileKeys, 1);
+  }
+  if (qi >= M) return;
+  // o[d][i]: column 32 d + 8 (i / 4) + 4 kh + i % 4
+  const float inv = 1.0f / l_run;
+  bf16_t* out = reinterpret_cast<bf16_t*>(a.ctx) + (int64_t)qi * a.ldc + (int64_t)h * a.vdim;
+#pragma unroll
+  for (int d = 0; d < DV / 32; ++d)
+#pragma unroll
+    for (int u = 0; u < 4; ++u) {
+      const int c = 32 * d + 8 * u + 4 * kh;
+      if (c + 3 < a.vdim && (a.vdim & 3) == 0) {
+        bf16x4_t v;
+#pragma unroll
+        for (int j = 0; j < 4; ++j) v[j] = (bf16_t)(o[d][4 * u + j] * inv);
+        *reinterpret_cast<bf16x4_t*>(out + c) = v;
+      } else {
+#pragma unroll
+        for (int j = 0; j < 4; ++j)
+          if (c + j < a.vdim) out[c + j] = (bf16_t)(o[d][4 * u + j] * inv);
+      }
+    }
+}
+
+template <int DK>
+void launch_tiles(const WindowAttnArgs& a, hipStream_t st) {
+  const dim3 g((unsigned)a.heads, (unsigned)((a.M + kTileQueries - 1) / kTileQueries));
+  if (a.vl.row == 64) hipLaunchKernelGGL((window_tile_kernel<DK, 64>), g, dim3(256), 0, st, a);
+  else if (a.vl.row == 128) hipLaunchKernelGGL((window_tile_kernel<DK, 128>), g, dim3(256), 0, st, a);
+  else hipLaunchKernelGGL((window_tile_kernel<DK, 256>), g, dim3(256), 0, st, a);
+}
+
+template <typename T>
+int launch_append(const WindowAttnArgs& a, hipStream_t st) {
+  const dim3 g((unsigned)((a.heads + 2 * a.kv_heads + 3) / 4), (unsigned)a.M);
+  hipLaunchKernelGGL(window_append_kernel<T>, g, dim3(256), 0, st, a);
+  AWQ_HIP_TRY(hipGetLastError());
+  return AWQ_OK;
+}
+
+template <typename T>
+int launch_queries(const WindowAttnArgs& a, hipStream_t st) {
   hipLaunchKernelGGL(window_query_kernel<T>, dim3((unsigned)a.heads, (unsigned)a.M), dim3(256),
                      (size_t)(a.dim + 256 + 4) * sizeof(float), st, a);
   AWQ_HIP_TRY(hipGetLastError());
@@ -113,17 +538,30 @@ int launch_simple(const WindowAttnArgs& a, hipStream_t st) {
 
 }  // namespace
 
-// rows are padded so that a row is whole 16-byte pieces of the matrix instructions' operands
-int32_t window_row_padded(int32_t dim) { return (int32_t)round_up(dim, 32); }
+// the tiled and the one-token kernel have rows of 64, 128 or 256 elements; longer ones go a query at a time
+int32_t window_row_padded(int32_t dim) { return dim <= 64 ? 64 : dim <= 128 ? 128 : (int32_t)round_up(dim, 256); }
 
-int64_t window_parts_floats(int32_t heads, int32_t vdim, int64_t window, int64_t max_pos) { return 4; }
-int64_t window_counter_count(int32_t heads, int32_t kv_heads) { return 4; }
+int64_t window_parts_floats(int32_t heads, int32_t vdim, int64_t window, int64_t max_pos) {
+  return (int64_t)heads * window_parts(window, max_pos) * (2 + vdim);
+}
+int64_t window_counter_count(int32_t heads, int32_t kv_heads) { return heads; }
 
 int launch_window_attention(const WindowAttnArgs& a, bool f32, hipStream_t st) {
   AWQ_REQUIRE(a.proj && a.k_cache && a.v_cache && a.ctx && a.slope && a.M >= 1 && a.M <= 65535, "bad arguments");
   AWQ_REQUIRE(a.heads >= 1 && a.kv_heads >= 1 && a.heads % a.kv_heads == 0, "heads must be a multiple of kv_heads");
   AWQ_REQUIRE(a.dim >= 1 && a.dim <= 1024 && a.vdim >= 1 && a.vdim <= 256 * kMaxColsPerThread, "head sizes must be at most 1024");
-  AWQ_REQUIRE(a.kl.slots > 0 && a.kl.slots % 64 == 0 && a.vl.slots == a.kl.slots && a.kl.row >= a.dim && a.vl.row >= a.vdim,
+  AWQ_REQUIRE(a.kl.slots > 0 && a.kl.slots % 64 == 0 && a.vl.slots == a.kl.slots && a.kl.row == window_row_padded(a.dim) &&
+                  a.vl.row == window_row_padded(a.vdim) && a.ldp % 8 == 0 && a.ldc % 8 == 0,
               "bad cache layout");
-  return f32 ? launch_simple<float>(a, st) : launch_simple<bf16_t>(a, st);
+  const bool tiled = a.kl.row <= 256 && a.vl.row <= 256;
+  if (a.M == 1 && tiled && a.parts && a.counters && a.len_bound > 0)
+    return f32 ? launch_decode<float>(a, st) : launch_decode<bf16_t>(a, st);
+  if (int rc = f32 ? launch_append<float>(a, st) : launch_append<bf16_t>(a, st)) return rc;
+  if (f32) return launch_queries<float>(a, st);
+  if (!tiled || a.pos.dyn) return launch_queries<bf16_t>(a, st);
+  if (a.kl.row == 64) launch_tiles<64>(a, st);
+  else if (a.kl.row == 128) launch_tiles<128>(a, st);
+  else launch_tiles<256>(a, st);
+  AWQ_HIP_TRY(hipGetLastError());
+  return AWQ_OK;
 }
