@@ -137,6 +137,44 @@ PRO_NONE, PRO_RMSNORM = 0, 1
 EPI_STORE, EPI_RESIDUAL, EPI_GELU, EPI_QKV_ROPE, EPI_ARGMAX = range(5)
 SIGNATURES["awq_gemv_fused"] = (ctypes.c_int, [ctypes.POINTER(AwqLinearArgs), _vp])
 
+
+
+class AwqDenseSegment(ctypes.Structure):
+    """struct awq_dense_segment"""
+    _fields_ = [("x", _vp), ("y", _vp), ("ldx", _i64), ("ldy", _i64), ("row0", _i32), ("rows", _i32), ("act", _i32),
+                ("act_rows", _i32), ("act_pos", _f32), ("act_neg", _f32)]
+
+
+class AwqDenseArgs(ctypes.Structure):
+    """struct awq_dense_args"""
+    _fields_ = [("w", _vp), ("k", _i64), ("tokens", _i64), ("n_segments", _i32), ("out", _i32),
+                ("segment", AwqDenseSegment * 2), ("addend", _vp), ("workspace", _vp), ("workspace_floats", _i64)]
+
+
+class AwqWindowArgs(ctypes.Structure):
+    """struct awq_window_args"""
+    _fields_ = [("proj", _vp), ("ldp", _i64), ("heads", _i32), ("kv_heads", _i32), ("dim", _i32), ("vdim", _i32),
+                ("window", _i32), ("slots", _i32), ("scale", _f32), ("eps", _f32), ("temp_coef", _f32), ("reserved", _f32),
+                ("temp_every", ctypes.c_double), ("slope", _vp), ("k_cache", _vp), ("v_cache", _vp), ("ctx", _vp),
+                ("ldc", _i64), ("n_tokens", _i64), ("pos0", _i64), ("max_pos", _i64), ("workspace", _vp)]
+
+
+ACT_NONE, ACT_SILU, ACT_XIELU = range(3)
+DENSE_STORE, DENSE_RESIDUAL, DENSE_F32 = range(3)
+SIGNATURES.update({
+    "awq_dense_weight_bytes": (_i64, [_i64, _i64, _i32]),
+    "awq_dense_pack": (ctypes.c_int, [_vp, _i32, _i64, _i64, _vp, _i64, _i64, _i64, _i32, _vp]),
+    "awq_dense": (ctypes.c_int, [ctypes.POINTER(AwqDenseArgs), _i32, _vp]),
+    "awq_embed_sinusoid": (ctypes.c_int, [_vp, _i32, _vp, _i64, _i64, _i64, _f32, _vp, _vp, _vp]),
+    "awq_norm_conv": (ctypes.c_int, [_vp, _i64, _i64, _i32, _f32, _vp, _vp, _i32, _vp, _vp, _vp, _vp, _vp, _i64, _i64, _i32,
+                                     _vp]),
+    "awq_gated_norm": (ctypes.c_int, [_vp, _i64, _vp, _i64, _vp, _vp, _i64, _i64, _i64, _f32, _i32, _vp]),
+    "awq_window_row": (_i32, [_i32]),
+    "awq_window_workspace_floats": (_i64, [_i32, _i32, _i64, _i64]),
+    "awq_window_attention": (ctypes.c_int, [ctypes.POINTER(AwqWindowArgs), _i32, _vp]),
+    "awq_linear_attention": (ctypes.c_int, [_vp, _i64, _i32, _i32, _i32, _vp, _vp, _vp, _vp, _i64, _i64, _i32, _vp]),
+})
+
 _lib = None
 
 

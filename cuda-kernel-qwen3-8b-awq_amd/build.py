@@ -24,9 +24,9 @@ TRACE = os.path.join(HERE, "trace_run")
 CORE_SOURCES = ["engine.cpp", "checkpoint.cpp", "ops.hip"]
 # models described by a config.json
 CONFIG_MODEL_SOURCES = ["kugilix.cpp", "dense.hip", "token_ops.hip", "window_attention.hip", "linear_attention.hip"]
-# the int4 model of the raw weight directory and the kernel-level entry points
+# the int4 model of the raw weight directory and the entry points for single kernels
 INT4_SOURCES = ["gemv.hip", "gemm.hip", "prefill.hip", "attention.hip", "fused.hip", "qkv_attn.hip", "qwen3.cpp",
-                "kernel_api.cpp", "synth.cpp"]
+                "kernel_api.cpp", "layer_api.cpp", "synth.cpp"]
 
 # -ffp-contract=off: every fma in the sources is written out; a contracted
 #   a*b-c*d would break bit parity with the reference's __hmul/__hsub sequence.

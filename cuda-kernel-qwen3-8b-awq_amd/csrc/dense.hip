@@ -121,21 +121,27 @@ __global__ __launch_bounds__(NW * 64) void dense_one_kernel(DenseArgs a) {
 // A workgroup of four wavefronts takes 256 rows and 32 TT tokens: 64 rows per wavefront as 2 x TT accumulators of
 // v_mfma_f32_32x32x16_bf16.  The weights go from memory into registers in operand order, every byte once per
 // workgroup; the tokens go through LDS (global_load_lds_dwordx4, 128 bytes per token and step of 64 inputs, the
-// eight 16-byte pieces of row r at positions c ^ (r & 7)).  Both are requested a step ahead.
+// eight 16-byte pieces of row r at positions c ^ (r & 7)).  Both are requested a step ahead.  Where the tiles do not
+// fill the device, k is cut over `cuts` workgroups whose sums go to the workspace, [cut][token][row]; a second launch
+// adds them in order.
+constexpr int DENSE_PART = 100;
 template <int TT, int OUT>
-__global__ __launch_bounds__(256, 2) void dense_many_kernel(DenseArgs a, int row_tiles, int tok_tiles) {
+__global__ __launch_bounds__(256, 2) void dense_many_kernel(DenseArgs a, int row_tiles, int tok_tiles, int cuts) {
   __shared__ __attribute__((aligned(16))) bf16_t tile0[32 * TT * 64];
   __shared__ __attribute__((aligned(16))) bf16_t tile1[32 * TT * 64];
-  const int total = row_tiles * tok_tiles;
+  const int total = row_tiles * tok_tiles * cuts;
   // workgroups whose indices agree modulo 8 share a die: each die walks its own run of row tiles
   const int per = (total + 7) >> 3;
   const int work = (blockIdx.x & 7) * per + (blockIdx.x >> 3);
   if (work >= total) return;
-  const int rt = work / tok_tiles, tt0 = (work - rt * tok_tiles) * 32 * TT;
+  const int rc = work / tok_tiles, tt0 = (work - rc * tok_tiles) * 32 * TT;
+  const int rt = rc / cuts, cut = rc - rt * cuts;
   const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
   const int n = lane & 31, kh = lane >> 5;
   const DenseSegment& s = segment_of(a, rt * 256);
-  const int steps = (int)(a.k >> 6);
+  const int all_steps = (int)(a.k >> 6);
+  const int first_step = (int)((int64_t)all_steps * cut / cuts);
+  const int steps = (int)((int64_t)all_steps * (cut + 1) / cuts) - first_step;
   const int64_t k16 = a.k >> 4;
 
   // this lane's pieces of the token tile
@@ -144,14 +150,14 @@ __global__ __launch_bounds__(256, 2) void dense_many_kernel(DenseArgs a, int row
   for (int i = 0; i < TT; ++i) {
     const int row = (wave * TT + i) * 8 + (lane >> 3);
     const int64_t tok = min((int64_t)tt0 + row, a.M - 1);
-    src[i] = reinterpret_cast<const bf16_t*>(s.x) + tok * s.ldx + (((lane & 7) ^ (row & 7)) << 3);
+    src[i] = reinterpret_cast<const bf16_t*>(s.x) + tok * s.ldx + first_step * 64 + (((lane & 7) ^ (row & 7)) << 3);
   }
   auto request = [&](bf16_t* tile, int step) __attribute__((always_inline)) {
 #pragma unroll
     for (int i = 0; i < TT; ++i)
       __builtin_amdgcn_global_load_lds((gptr_t)(src[i] + step * 64), (lptr_t)(tile + (wave * TT + i) * 8 * 64), 16, 0, 0);
   };
-  const bf16x8_t* wp = reinterpret_cast<const bf16x8_t*>(a.w) + (int64_t)(rt * 8 + wave * 2) * k16 * 64 + lane;
+  const bf16x8_t* wp = reinterpret_cast<const bf16x8_t*>(a.w) + ((int64_t)(rt * 8 + wave * 2) * k16 + first_step * 4) * 64 + lane;
   auto weights = [&](bf16x8_t (&wv)[2][4], int step) __attribute__((always_inline)) {
 #pragma unroll
     for (int b = 0; b < 2; ++b)
@@ -206,6 +212,14 @@ __global__ __launch_bounds__(256, 2) void dense_many_kernel(DenseArgs a, int row
     for (int b = 0; b < 2; ++b)
 #pragma unroll
       for (int g = 0; g < 4; ++g) {
+        if constexpr (OUT == DENSE_PART) {
+          f32x4_t v;
+#pragma unroll
+          for (int j = 0; j < 4; ++j) v[j] = acc[b][t][4 * g + j];
+          *reinterpret_cast<f32x4_t*>(a.workspace + ((int64_t)cut * a.M + tok) * row_tiles * 256 + rt * 256 + wave * 64 + 32 * b +
+                                      8 * g + 4 * kh) = v;
+          continue;
+        }
         const int row = rt * 256 + wave * 64 + 32 * b + 8 * g + 4 * kh - s.row0;
         const int64_t at = tok * s.ldy + row;
         if (row + 3 < s.rows && (s.ldy & 3) == 0) {
@@ -232,6 +246,24 @@ __global__ __launch_bounds__(256, 2) void dense_many_kernel(DenseArgs a, int row
         }
       }
   }
+}
+
+// adds the sums of the workgroups that shared k: a thread takes four rows of a token
+template <int OUT>
+__global__ __launch_bounds__(256) void dense_parts_kernel(DenseArgs a, int rows, int cuts) {
+  const int row = (blockIdx.x * 256 + threadIdx.x) * 4;
+  const int64_t tok = blockIdx.y;
+  if (row >= rows) return;
+  const DenseSegment& s = segment_of(a, row);
+  const int local = row - s.row0;
+  if (local >= s.rows) return;
+  const f32x4_t* p = reinterpret_cast<const f32x4_t*>(a.workspace + tok * rows + row);
+  const int64_t stride = a.M * rows / 4;
+  f32x4_t sum = p[0];
+  for (int c = 1; c < cuts; ++c) sum = sum + p[c * stride];
+#pragma unroll
+  for (int j = 0; j < 4; ++j)
+    if (local + j < s.rows) finish_one<bf16_t, OUT>(a, s, tok, local + j, sum[j]);
 }
 
 // --- binary32 ----------------------------------------------------------------------------------------------
@@ -331,15 +363,28 @@ int launch_many(const DenseArgs& a, bool f32, int64_t rows, hipStream_t st) {
                        st, a);
   } else {
     const int row_tiles = (int)(rows / 256);
-    // wide tiles once they fill the device
-    const int64_t wide = (a.M + 127) / 128;
-    if (row_tiles * wide >= 256) {
-      const unsigned grid = (unsigned)((row_tiles * wide + 7) / 8 * 8);
-      hipLaunchKernelGGL((dense_many_kernel<4, OUT>), dim3(grid), dim3(256), 0, st, a, row_tiles, (int)wide);
+    const bool wide = a.M > 64;
+    const int64_t tok_tiles = wide ? (a.M + 127) / 128 : (a.M + 63) / 64;
+    const int64_t tiles = row_tiles * tok_tiles;
+    // two workgroups per compute unit, at least eight steps each
+    int64_t cuts = 1;
+    if (a.workspace && a.M <= 65535 && tiles < 384) {
+      cuts = std::min<int64_t>((512 + tiles / 2) / tiles, (a.k >> 6) / 8);
+      cuts = std::max<int64_t>(1, std::min<int64_t>(cuts, a.workspace_floats / (a.M * rows)));
+    }
+    const unsigned grid = (unsigned)((tiles * cuts + 7) / 8 * 8);
+    if (cuts > 1) {
+      if (wide)
+        hipLaunchKernelGGL((dense_many_kernel<4, DENSE_PART>), dim3(grid), dim3(256), 0, st, a, row_tiles, (int)tok_tiles, (int)cuts);
+      else
+        hipLaunchKernelGGL((dense_many_kernel<2, DENSE_PART>), dim3(grid), dim3(256), 0, st, a, row_tiles, (int)tok_tiles, (int)cuts);
+      AWQ_HIP_TRY(hipGetLastError());
+      hipLaunchKernelGGL(dense_parts_kernel<OUT>, dim3((unsigned)((rows / 4 + 255) / 256), (unsigned)a.M), dim3(256), 0, st, a,
+                         (int)rows, (int)cuts);
+    } else if (wide) {
+      hipLaunchKernelGGL((dense_many_kernel<4, OUT>), dim3(grid), dim3(256), 0, st, a, row_tiles, (int)tok_tiles, 1);
     } else {
-      const int64_t narrow = (a.M + 63) / 64;
-      const unsigned grid = (unsigned)((row_tiles * narrow + 7) / 8 * 8);
-      hipLaunchKernelGGL((dense_many_kernel<2, OUT>), dim3(grid), dim3(256), 0, st, a, row_tiles, (int)narrow);
+      hipLaunchKernelGGL((dense_many_kernel<2, OUT>), dim3(grid), dim3(256), 0, st, a, row_tiles, (int)tok_tiles, 1);
     }
   }
   AWQ_HIP_TRY(hipGetLastError());

@@ -172,6 +172,7 @@ struct Buffers {
 constexpr int64_t kPassTokens = 2048;   // prompt positions per pass
 constexpr int64_t kLogitRows = 128;     // rows whose logits are formed at once
 constexpr int64_t kDefaultPositions = 8192;
+constexpr int64_t kDenseWorkspace = 32ll << 20;  // floats, for products that are cut along k
 
 struct KugilixEngine final : awq_engine {
   Spec spec;
@@ -190,7 +191,8 @@ struct KugilixEngine final : awq_engine {
   float* logits = nullptr;  // [kLogitRows][vocab]
   unsigned long long* best = nullptr;
   float* attn_parts = nullptr;
-  int32_t* attn_counters = nullptr;
+  float* dense_ws = nullptr;
+  int64_t dense_ws_floats = 0;
   std::vector<int64_t> bounds;
   bool tap_on = false, tap_saved_graphs = true;
   float* tap = nullptr;
@@ -438,7 +440,7 @@ int KugilixEngine::make_runs() {
       runs.push_back(r);
     }
   }
-  int64_t parts = 4, counters = 4;
+  int64_t parts = 4;
   for (LayerRun& r : runs) {
     const LayerSpec& s = spec.layers[r.layer];
     if (spec.taps > 1)
@@ -455,10 +457,8 @@ int KugilixEngine::make_runs() {
     if (int rc = zeroed(&r.k_cache, r.kl.elements() * unit())) return rc;
     if (int rc = zeroed(&r.v_cache, r.vl.elements() * unit())) return rc;
     parts = std::max(parts, window_parts_floats(s.heads, s.vdim, s.window, max_pos));
-    counters = std::max(counters, window_counter_count(s.heads, s.kv_heads));
   }
-  if (int rc = zeroed((void**)&attn_parts, parts * 4)) return rc;
-  return zeroed((void**)&attn_counters, counters * 4);
+  return zeroed((void**)&attn_parts, parts * 4);
 }
 
 // --- passes ------------------------------------------------------------------------------------------------
@@ -494,6 +494,8 @@ int KugilixEngine::run_layers(Buffers& b, int64_t M, PassPos pos) {
       a.w = L.w_in;
       a.k = ld;
       a.M = M;
+      a.workspace = dense_ws;
+      a.workspace_floats = dense_ws_floats;
       DenseSegment& in = a.seg[0];
       in.x = b.h;
       in.ldx = ld;
@@ -542,7 +544,6 @@ int KugilixEngine::run_layers(Buffers& b, int64_t M, PassPos pos) {
       a.M = M;
       a.pos = pos;
       a.parts = attn_parts;
-      a.counters = attn_counters;
       a.len_bound = (int32_t)max_pos;
       if (int rc = launch_window_attention(a, f32, stream)) return rc;
     } else {
@@ -569,6 +570,8 @@ int KugilixEngine::run_layers(Buffers& b, int64_t M, PassPos pos) {
       a.k = L.k_out;
       a.M = M;
       a.out = DENSE_RESIDUAL;
+      a.workspace = dense_ws;
+      a.workspace_floats = dense_ws_floats;
       a.seg[0].x = cat;
       a.seg[0].ldx = L.k_out;
       a.seg[0].y = b.x;
@@ -606,6 +609,8 @@ int KugilixEngine::logits_of(const float* x, const int32_t* which, int64_t n, bo
   d.M = n;
   d.out = sample ? DENSE_ARGMAX : DENSE_F32;
   d.best = best;
+  d.workspace = dense_ws;
+  d.workspace_floats = dense_ws_floats;
   d.seg[0].x = head_in;
   d.seg[0].ldx = ld;
   d.seg[0].y = logits;
@@ -720,6 +725,10 @@ int open_kugilix(const char* dir, const awq_open_options& opt, awq_engine** out)
   if (int rc = e->make_buffers(&e->step, 1)) return rc;
   if (int rc = e->make_buffers(&e->pass, e->pass_tokens)) return rc;
   if (int rc = e->make_runs()) return rc;
+  if (!e->f32) {
+    e->dense_ws_floats = std::min<int64_t>(kDenseWorkspace, 4 * e->pass_tokens * round_up(e->spec.width, kDenseRowAlign));
+    if (int rc = e->dev_alloc((void**)&e->dense_ws, e->dense_ws_floats * 4)) return rc;
+  }
   if (int rc = e->zeroed((void**)&e->tokens, e->pass_tokens * 4)) return rc;
   if (int rc = e->zeroed((void**)&e->rows, kLogitRows * 4)) return rc;
   if (int rc = e->zeroed(&e->head_in, kLogitRows * e->ld * e->unit())) return rc;

@@ -63,6 +63,8 @@ struct DenseArgs {
   DenseSegment seg[2];
   const float* addend = nullptr;
   unsigned long long* best = nullptr;  // DENSE_ARGMAX: zero between launches
+  float* workspace = nullptr;          // sums of products that are cut along k; may be null
+  int64_t workspace_floats = 0;
 };
 int64_t dense_weight_bytes(int64_t rows_padded, int64_t k_padded, bool f32);
 // src [rows][cols] bfloat16 or float, row major on the device, into rows row0.., inputs col0.. of a block (col0 a
@@ -135,12 +137,10 @@ struct WindowAttnArgs {
   PassPos pos;
   // one-token form: partial results of the parts a window is cut into
   float* parts = nullptr;
-  int32_t* counters = nullptr;  // zero between launches
-  int32_t len_bound = 0;        // >= positions the sequence will hold
+  int32_t len_bound = 0;  // >= positions the sequence will hold
 };
 int32_t window_row_padded(int32_t dim);
 int64_t window_parts_floats(int32_t heads, int32_t vdim, int64_t window, int64_t max_pos);
-int64_t window_counter_count(int32_t heads, int32_t kv_heads);
 // normalise q and k, append k and v, attend
 int launch_window_attention(const WindowAttnArgs& a, bool f32, hipStream_t st);
 

@@ -64,8 +64,9 @@ __global__ __launch_bounds__(256) void linear_step_kernel(LinearAttnArgs a) {
 // chunk and S the state ahead of it,
 //     o_t = decay^(t+1) S^T q_t + sum over s <= t of decay^(t-s) (k_s . q_t) v_s
 //     S  <- decay^n S + sum over t < n of k_t (decay^(n-1-t) v_t)^T
-// A workgroup takes 32 columns of one head's state and all chunks in turn; wavefront w computes the outputs of
-// tokens 32 w .. + 31 of a chunk and keeps 32 (64 at dim 256) of the state's rows in its accumulators.  q, k and v
+// A workgroup takes 32 columns of one head's state and all chunks in turn.  Wavefronts 0 .. 3 compute the outputs of 32
+// tokens of a chunk each; wavefronts 4 .. 7 keep 32 (64 at dim 256) of the state's rows each in their accumulators and
+// carry them over the chunk at the same time.  q, k and v
 // are bfloat16 as projected, so their products are exact; the binary32 factors enter as sums of bfloat16 terms
 // (three for the state and for the decayed values, two for the weights inside a chunk) and every accumulation is
 // binary32.  Operands of v_mfma_f32_32x32x16_bf16, lane (n, kh) = (lane % 32, lane / 32):
@@ -86,16 +87,18 @@ constexpr int linear_chunk_lds() {
 }
 
 template <int D>
-__global__ __launch_bounds__(256) void linear_chunk_kernel(LinearAttnArgs a) {
+__global__ __launch_bounds__(512) void linear_chunk_kernel(LinearAttnArgs a) {
   extern __shared__ __attribute__((aligned(16))) char lds_raw[];
   constexpr int KS = D + 16, SS = D + 8, NT = D / 32;  // NT tiles of 32 state rows, over four wavefronts
   constexpr int TPW = NT < 4 ? 1 : NT / 4;             // ... per wavefront
-  constexpr int KP = D / 16;                           // 16-byte pieces of k per thread
+  constexpr int KP = D / 32;                           // 16-byte pieces of k per thread
   bf16_t* const ks = reinterpret_cast<bf16_t*>(lds_raw);       // [128][KS]
   bf16_t* const vt = ks + kChunk * KS;                         // [4][32][kVStride]: v, then three terms of v'
   bf16_t* const st = vt + 4 * 32 * kVStride;                   // [3][32][SS]
   const int head = blockIdx.x, v0 = blockIdx.y * 32;
-  const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const int tid = threadIdx.x, lane = tid & 63, wave8 = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const int wave = wave8 & 3;
+  const bool outputs = wave8 < 4;
   const int n = lane & 31, kh = lane >> 5;
   const int M = (int)a.M;
   const bf16_t* const p = reinterpret_cast<const bf16_t*>(a.proj);
@@ -123,7 +126,7 @@ __global__ __launch_bounds__(256) void linear_chunk_kernel(LinearAttnArgs a) {
 
   // the state: rows 32 (wave + 4 i) + 8 g + 4 kh + j of column n in s[i][4 g + j]
   f32x16_t s[TPW];
-  const bool holds = wave < NT;
+  const bool holds = !outputs && wave < NT;
   const bool fresh = a.pos.position() == 0;
 #pragma unroll
   for (int i = 0; i < TPW; ++i)
@@ -140,11 +143,12 @@ __global__ __launch_bounds__(256) void linear_chunk_kernel(LinearAttnArgs a) {
   auto load = [&](int c0) __attribute__((always_inline)) {
 #pragma unroll
     for (int i = 0; i < KP; ++i) {
-      const int pc = tid + 256 * i, row = pc / (D / 8), at = (pc % (D / 8)) * 8;
+      const int pc = tid + 512 * i, row = pc / (D / 8), at = (pc % (D / 8)) * 8;
       kr[i] = piece(k + (int64_t)min(c0 + row, M - 1) * a.ldp, at, a.dim);
     }
 #pragma unroll
-    for (int i = 0; i < 2; ++i) vr[i] = piece(v + (int64_t)min(c0 + 2 * lane + i, M - 1) * a.ldp, 8 * wave, nv);
+    for (int i = 0; i < 2; ++i)
+      if (outputs) vr[i] = piece(v + (int64_t)min(c0 + 2 * lane + i, M - 1) * a.ldp, 8 * wave, nv);
   };
   load(0);
   for (int c0 = 0; c0 < M; c0 += kChunk) {
@@ -152,10 +156,10 @@ __global__ __launch_bounds__(256) void linear_chunk_kernel(LinearAttnArgs a) {
     __syncthreads();  // the previous chunk's readers are done
 #pragma unroll
     for (int i = 0; i < KP; ++i) {
-      const int pc = tid + 256 * i, row = pc / (D / 8), at = (pc % (D / 8)) * 8;
+      const int pc = tid + 512 * i, row = pc / (D / 8), at = (pc % (D / 8)) * 8;
       *reinterpret_cast<bf16x8_t*>(ks + row * KS + at) = kr[i];
     }
-    {
+    if (outputs) {
       // tokens 2 lane, 2 lane + 1, columns 8 wave ..; v' = decay^(len - 1 - t) v, nothing behind the last token
       float w[2];
 #pragma unroll
@@ -205,35 +209,43 @@ __global__ __launch_bounds__(256) void linear_chunk_kernel(LinearAttnArgs a) {
     // this lane's query: token 32 wave + n
     const int tq = 32 * wave + n;
     bf16x8_t qop[D / 16];
+    if (outputs)
 #pragma unroll
-    for (int i = 0; i < D / 16; ++i)
-      qop[i] = piece(q + (int64_t)min(c0 + tq, M - 1) * a.ldp, 16 * i + 8 * kh, a.dim);
+      for (int i = 0; i < D / 16; ++i)
+        qop[i] = piece(q + (int64_t)min(c0 + tq, M - 1) * a.ldp, 16 * i + 8 * kh, a.dim);
     __syncthreads();
     if (c0 + kChunk < M) load(c0 + kChunk);
 
-    if (32 * wave < len) {
-      f32x16_t o;
+    if (outputs && 32 * wave < len) {
+      // one accumulator per term of the state: three independent chains of matrix instructions
+      f32x16_t om[3];
 #pragma unroll
-      for (int i = 0; i < 16; ++i) o[i] = 0.0f;
+      for (int m = 0; m < 3; ++m)
+#pragma unroll
+        for (int i = 0; i < 16; ++i) om[m][i] = 0.0f;
 #pragma unroll
       for (int i = 0; i < D / 16; ++i)
 #pragma unroll
         for (int m = 0; m < 3; ++m) {
           const bf16x8_t sv = *reinterpret_cast<const bf16x8_t*>(st + (m * 32 + n) * SS + 16 * i + 8 * kh);
-          o = __builtin_amdgcn_mfma_f32_32x32x16_bf16(sv, qop[i], o, 0, 0, 0);
+          om[m] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(sv, qop[i], om[m], 0, 0, 0);
         }
       const float wq = __builtin_amdgcn_exp2f((float)(tq + 1) * lg);
+      f32x16_t o, o2;
 #pragma unroll
-      for (int i = 0; i < 16; ++i) o[i] *= wq;
+      for (int i = 0; i < 16; ++i) o[i] = (om[0][i] + (om[1][i] + om[2][i])) * wq, o2[i] = 0.0f;
       for (int s0 = 0; s0 <= 32 * wave; s0 += 32) {
-        f32x16_t w;
+        f32x16_t w, w2;
 #pragma unroll
-        for (int i = 0; i < 16; ++i) w[i] = 0.0f;
+        for (int i = 0; i < 16; ++i) w[i] = 0.0f, w2[i] = 0.0f;
 #pragma unroll
-        for (int i = 0; i < D / 16; ++i) {
-          const bf16x8_t kv = *reinterpret_cast<const bf16x8_t*>(ks + (s0 + n) * KS + 16 * i + 8 * kh);
-          w = __builtin_amdgcn_mfma_f32_32x32x16_bf16(kv, qop[i], w, 0, 0, 0);
+        for (int i = 0; i < D / 16; i += 2) {
+          const bf16_t* at = ks + (s0 + n) * KS + 16 * i + 8 * kh;
+          w = __builtin_amdgcn_mfma_f32_32x32x16_bf16(*reinterpret_cast<const bf16x8_t*>(at), qop[i], w, 0, 0, 0);
+          w2 = __builtin_amdgcn_mfma_f32_32x32x16_bf16(*reinterpret_cast<const bf16x8_t*>(at + 16), qop[i + 1], w2, 0, 0, 0);
         }
+#pragma unroll
+        for (int i = 0; i < 16; ++i) w[i] += w2[i];
         bf16x8_t hi[2], lo[2];
 #pragma unroll
         for (int i = 0; i < 16; ++i) {
@@ -248,9 +260,11 @@ __global__ __launch_bounds__(256) void linear_chunk_kernel(LinearAttnArgs a) {
           const bf16x4_t l4 = *reinterpret_cast<const bf16x4_t*>(at), h4 = *reinterpret_cast<const bf16x4_t*>(at + 8);
           const bf16x8_t vv = {l4[0], l4[1], l4[2], l4[3], h4[0], h4[1], h4[2], h4[3]};
           o = __builtin_amdgcn_mfma_f32_32x32x16_bf16(vv, hi[j], o, 0, 0, 0);
-          o = __builtin_amdgcn_mfma_f32_32x32x16_bf16(vv, lo[j], o, 0, 0, 0);
+          o2 = __builtin_amdgcn_mfma_f32_32x32x16_bf16(vv, lo[j], o2, 0, 0, 0);
         }
       }
+#pragma unroll
+      for (int i = 0; i < 16; ++i) o[i] += o2[i];
       if (tq < len) {
         float* out = a.o + (int64_t)(c0 + tq) * a.heads * a.vdim + (int64_t)head * a.vdim + v0;
 #pragma unroll
@@ -270,10 +284,11 @@ __global__ __launch_bounds__(256) void linear_chunk_kernel(LinearAttnArgs a) {
       const float ws = __builtin_amdgcn_exp2f((float)len * lg);
       const int L16 = lane & 15;
       const bf16_t* const klane = ks + (4 * kh + (L16 >> 2)) * KS + 16 * ((lane >> 4) & 1) + 4 * (L16 & 3);
+      f32x16_t sl[TPW];  // the smaller terms, apart: two chains
 #pragma unroll
       for (int i = 0; i < TPW; ++i)
 #pragma unroll
-        for (int j = 0; j < 16; ++j) s[i][j] *= ws;
+        for (int j = 0; j < 16; ++j) s[i][j] *= ws, sl[i][j] = 0.0f;
       for (int t0 = 0; t0 < len; t0 += 16) {
         bf16x8_t vv[3];
 #pragma unroll
@@ -290,9 +305,16 @@ __global__ __launch_bounds__(256) void linear_chunk_kernel(LinearAttnArgs a) {
           const bf16x4_t l4 = __builtin_bit_cast(bf16x4_t, l), h4 = __builtin_bit_cast(bf16x4_t, h);
           const bf16x8_t kv = {l4[0], l4[1], l4[2], l4[3], h4[0], h4[1], h4[2], h4[3]};
 #pragma unroll
-          for (int m = 0; m < 3; ++m) s[i] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(kv, vv[m], s[i], 0, 0, 0);
+          for (int m = 0; m < 3; ++m) {
+            if (m == 0) s[i] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(kv, vv[m], s[i], 0, 0, 0);
+            else sl[i] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(kv, vv[m], sl[i], 0, 0, 0);
+          }
         }
       }
+#pragma unroll
+      for (int i = 0; i < TPW; ++i)
+#pragma unroll
+        for (int j = 0; j < 16; ++j) s[i][j] += sl[i][j];
     }
   }
   if (holds && n < nv)
@@ -314,7 +336,7 @@ int launch_chunks(const LinearAttnArgs& a, hipStream_t st) {
                                     linear_chunk_lds<D>()));
     raised = true;
   }
-  hipLaunchKernelGGL(linear_chunk_kernel<D>, dim3((unsigned)a.heads, (unsigned)((a.vdim + 31) / 32)), dim3(256),
+  hipLaunchKernelGGL(linear_chunk_kernel<D>, dim3((unsigned)a.heads, (unsigned)((a.vdim + 31) / 32)), dim3(512),
                      linear_chunk_lds<D>(), st, a);
   AWQ_HIP_TRY(hipGetLastError());
   return AWQ_OK;

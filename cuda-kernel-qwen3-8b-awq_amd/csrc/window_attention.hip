@@ -38,6 +38,42 @@ __global__ __launch_bounds__(256) void window_append_kernel(WindowAttnArgs a) {
   }
 }
 
+// The same for head sizes that are whole 16-byte pieces: a group of lanes per row, 8 elements each.
+__global__ __launch_bounds__(256) void window_append8_kernel(WindowAttnArgs a, int lanes) {
+  const int items = a.heads + 2 * a.kv_heads;
+  const int64_t at = (int64_t)blockIdx.x * (256 / lanes) + threadIdx.x / lanes;
+  const int t = (int)(at / items), item = (int)(at - (int64_t)t * items), d0 = (threadIdx.x % lanes) * 8;
+  if (t >= (int)a.M) return;
+  bf16_t* row = reinterpret_cast<bf16_t*>(a.proj) + (int64_t)t * a.ldp;
+  const int pos = a.pos.position() + t;
+  const bool value = item >= a.heads + a.kv_heads;
+  bf16_t* src = value ? row + (int64_t)(a.heads + a.kv_heads) * a.dim + (int64_t)(item - a.heads - a.kv_heads) * a.vdim
+                      : row + (int64_t)item * a.dim;
+  const int n = value ? a.vdim : a.dim;
+  bf16x8_t x;
+#pragma unroll
+  for (int i = 0; i < 8; ++i) x[i] = (bf16_t)0.0f;
+  if (d0 < n) x = *reinterpret_cast<const bf16x8_t*>(src + d0);
+  float acc = 0.0f;
+#pragma unroll
+  for (int i = 0; i < 8; ++i) acc = __builtin_fmaf((float)x[i], (float)x[i], acc);
+  for (int off = lanes >> 1; off > 0; off >>= 1) acc += __shfl_xor(acc, off, 64);
+  if (value) {
+    if (d0 < a.vl.row)
+      *reinterpret_cast<bf16x8_t*>(reinterpret_cast<bf16_t*>(a.v_cache) +
+                                   ring_row(a.vl, item - a.heads - a.kv_heads, pos % a.vl.slots) + d0) = x;
+    return;
+  }
+  const float inv = 1.0f / sqrtf(acc / (float)a.dim + a.eps);
+#pragma unroll
+  for (int i = 0; i < 8; ++i) x[i] = (bf16_t)((float)x[i] * inv);
+  if (item < a.heads) {
+    if (d0 < a.dim) *reinterpret_cast<bf16x8_t*>(src + d0) = x;
+  } else if (d0 < a.kl.row) {
+    *reinterpret_cast<bf16x8_t*>(reinterpret_cast<bf16_t*>(a.k_cache) + ring_row(a.kl, item - a.heads, pos % a.kl.slots) + d0) = x;
+  }
+}
+
 // A query at a time: a workgroup per (token, head), a thread per key, blocks of 256 keys with a running maximum.
 // Any sizes; the binary32 form and what the tiled kernel has no instance for.
 constexpr int kMaxColsPerThread = 4;
@@ -100,11 +136,11 @@ __global__ __launch_bounds__(256) void window_query_kernel(WindowAttnArgs a) {
     if (c * 256 + tid < a.vdim) out[c * 256 + tid] = (T)(acc[c] / l);
 }
 
-// One token.  blockIdx.x: kv head and up to R of its query heads, blockIdx.y: part of the visible keys.  Every
-// workgroup normalises its queries; the one that holds the newest position normalises its key, uses key and value
-// from LDS and appends them.  Scores of a part sit in LDS; the parts' maxima, sums and contexts go to memory and the
-// workgroup that finishes last adds them up.
-constexpr int kPartKeys = 128;
+// One token.  blockIdx.x: kv head and up to R of its query heads, blockIdx.y: 64 of the visible keys.  The rows a
+// workgroup needs are requested before anything else; every lane group normalises the queries for itself, and the
+// workgroup of the newest position takes its key and value from the projections and appends them.  A wavefront's
+// lane holds the weight of one key.  With more than one part a second launch adds the parts up.
+constexpr int kPartKeys = 64;
 
 __host__ __device__ inline int window_parts(int64_t window, int64_t max_pos) {
   const int64_t n = window > 0 && window < max_pos ? window : max_pos;
@@ -116,20 +152,30 @@ struct Vec8;
 template <>
 struct Vec8<bf16_t> {
   bf16x8_t v;
-  __device__ __forceinline__ void load(const bf16_t* p) { v = *reinterpret_cast<const bf16x8_t*>(p); }
 };
 template <>
 struct Vec8<float> {
   typedef float f8 __attribute__((ext_vector_type(8)));
   f8 v;
-  __device__ __forceinline__ void load(const float* p) { v = *reinterpret_cast<const f8*>(p); }
 };
+// elements at .. at + 7 of a row of n, zeros behind it
+template <typename T>
+__device__ __forceinline__ void row_piece(const T* row, int at, int n, bool aligned, float (&x)[8]) {
+  if (aligned && at + 8 <= n) {
+    const Vec8<T> v = *reinterpret_cast<const Vec8<T>*>(row + at);
+#pragma unroll
+    for (int i = 0; i < 8; ++i) x[i] = (float)v.v[i];
+  } else {
+#pragma unroll
+    for (int i = 0; i < 8; ++i) x[i] = at + i < n ? (float)row[at + i] : 0.0f;
+  }
+}
 
-template <typename T, int R>
+// U: cache rows of a lane, row length / 32
+template <typename T, int R, int U>
 __global__ __launch_bounds__(256) void window_decode_kernel(WindowAttnArgs a, int chunks) {
-  extern __shared__ float lds[];
-  __shared__ float inv[R + 1], part_m[R], part_l[R];
-  __shared__ int last;
+  extern __shared__ float red[];      // [4][R][vw]
+  __shared__ float sc[R][kPartKeys];
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int g = blockIdx.x / chunks, rz = (blockIdx.x - g * chunks) * R;
   const int per_group = a.heads / a.kv_heads;
@@ -139,116 +185,102 @@ __global__ __launch_bounds__(256) void window_decode_kernel(WindowAttnArgs a, in
   const int parts = (pos + 1 - lo + kPartKeys - 1) / kPartKeys;
   const int part = blockIdx.y;
   if (part >= parts) return;
-  const int b = lo + part * kPartKeys, e = min(b + kPartKeys, pos + 1), nk = e - b;
+  const int b = lo + part * kPartKeys, nk = min(kPartKeys, pos + 1 - b);
   const bool newest = part == parts - 1;
   const int kw = a.kl.row, vw = a.vl.row;
-  float* const sc = lds;                     // [R][kPartKeys]
-  float* const knew = sc + R * kPartKeys;    // [kw]
-  float* const vnew = knew + kw;             // [vw]
-  float* const red = vnew + vw;              // [4][R][vw]
-
-  const T* const proj = reinterpret_cast<const T*>(a.proj);
-  const T* const kp = proj + (int64_t)(a.heads + g) * a.dim;
-  for (int r = wave; r <= nr; r += 4) {  // row nr: the new key
-    const T* x = r < nr ? proj + (int64_t)(h0 + r) * a.dim : kp;
-    float acc = 0.0f;
-    for (int d = lane; d < a.dim; d += 64) acc = __builtin_fmaf((float)x[d], (float)x[d], acc);
-#pragma unroll
-    for (int off = 32; off > 0; off >>= 1) acc += __shfl_xor(acc, off, 64);
-    if (lane == 0) inv[r] = 1.0f / sqrtf(acc / (float)a.dim + a.eps);
-  }
-  __syncthreads();
-  if (newest) {
-    const T* vp = proj + (int64_t)(a.heads + a.kv_heads) * a.dim + (int64_t)g * a.vdim;
-    T* kd = reinterpret_cast<T*>(a.k_cache) + ring_row(a.kl, g, pos % a.kl.slots);
-    T* vd = reinterpret_cast<T*>(a.v_cache) + ring_row(a.vl, g, pos % a.vl.slots);
-    for (int d = tid; d < kw; d += 256) {
-      const T x = d < a.dim ? (T)((float)kp[d] * inv[nr]) : (T)0.0f;
-      knew[d] = (float)x;
-      if (rz == 0) kd[d] = x;
-    }
-    for (int d = tid; d < vw; d += 256) {
-      const T x = d < a.vdim ? vp[d] : (T)0.0f;
-      vnew[d] = (float)x;
-      if (rz == 0) vd[d] = x;
-    }
-  }
-  // lanes of a key: 8 of its elements each
-  const int lpk = kw >> 3, sub = lane / lpk, d0 = (lane - sub * lpk) * 8, kpw = 64 / lpk;
-  float qv[R][8];
-#pragma unroll
-  for (int r = 0; r < R; ++r)
-#pragma unroll
-    for (int i = 0; i < 8; ++i)
-      qv[r][i] = r < nr && d0 + i < a.dim ? (float)(T)((float)proj[(int64_t)(h0 + r) * a.dim + d0 + i] * inv[r]) : 0.0f;
-  __syncthreads();
-  const float mul = a.scale * temperature(a, pos);
+  // lanes of a key and of a value row: 8 elements each
+  const int lpk = kw >> 3, sub = lane / lpk, d0 = (lane - sub * lpk) * 8, kpw = 64 / lpk, uk = kw >> 5;
+  const int tpv = vw >> 3, c0 = (tid % tpv) * 8, first = tid / tpv, step = 256 / tpv, uv = vw >> 5;
   const T* const kc = reinterpret_cast<const T*>(a.k_cache);
-  // four keys of a lane's group are requested before the first is multiplied
-  for (int k0 = wave * kpw; k0 < nk; k0 += 16 * kpw) {
-    Vec8<T> kv[4];
+  const T* const vc = reinterpret_cast<const T*>(a.v_cache);
+  Vec8<T> kv[U], vv[U];
 #pragma unroll
-    for (int u = 0; u < 4; ++u) {
-      const int key = min(b + k0 + u * 4 * kpw + sub, pos);
-      if (key < pos) kv[u].load(kc + ring_row(a.kl, g, key % a.kl.slots) + d0);
+  for (int u = 0; u < U; ++u) {
+    const int key = b + (u * 4 + wave) * kpw + sub;
+    if (u < uk && key < pos) kv[u] = *reinterpret_cast<const Vec8<T>*>(kc + ring_row(a.kl, g, key % a.kl.slots) + d0);
+  }
+#pragma unroll
+  for (int u = 0; u < U; ++u) {
+    const int key = b + u * step + first;
+    if (u < uv && key < pos) vv[u] = *reinterpret_cast<const Vec8<T>*>(vc + ring_row(a.vl, g, key % a.vl.slots) + c0);
+  }
+  const T* const proj = reinterpret_cast<const T*>(a.proj);
+  const bool dim8 = (a.dim & 7) == 0, vdim8 = ((a.dim | a.vdim) & 7) == 0;
+  auto normalised = [&](const T* row, float (&x)[8]) {
+    row_piece(row, d0, a.dim, dim8, x);
+    float acc = 0.0f;
+#pragma unroll
+    for (int i = 0; i < 8; ++i) acc = __builtin_fmaf(x[i], x[i], acc);
+    for (int off = lpk >> 1; off > 0; off >>= 1) acc += __shfl_xor(acc, off, 64);
+    const float inv = 1.0f / sqrtf(acc / (float)a.dim + a.eps);
+#pragma unroll
+    for (int i = 0; i < 8; ++i) x[i] = (float)(T)(x[i] * inv);
+  };
+  float qv[R][8], kn[8] = {}, vn[8] = {};
+#pragma unroll
+  for (int r = 0; r < R; ++r) normalised(proj + (int64_t)(h0 + min(r, nr - 1)) * a.dim, qv[r]);
+  if (newest) {
+    normalised(proj + (int64_t)(a.heads + g) * a.dim, kn);
+    row_piece(proj + (int64_t)(a.heads + a.kv_heads) * a.dim + (int64_t)g * a.vdim, c0, a.vdim, vdim8, vn);
+    Vec8<T> out;
+    if (rz == 0 && tid < lpk) {
+#pragma unroll
+      for (int i = 0; i < 8; ++i) out.v[i] = (T)kn[i];
+      *reinterpret_cast<Vec8<T>*>(reinterpret_cast<T*>(a.k_cache) + ring_row(a.kl, g, pos % a.kl.slots) + d0) = out;
     }
+    if (rz == 0 && tid < tpv) {
 #pragma unroll
-    for (int u = 0; u < 4; ++u) {
-      const int i = k0 + u * 4 * kpw + sub, key = b + i;
-      float x[8];
+      for (int i = 0; i < 8; ++i) out.v[i] = (T)vn[i];
+      *reinterpret_cast<Vec8<T>*>(reinterpret_cast<T*>(a.v_cache) + ring_row(a.vl, g, pos % a.vl.slots) + c0) = out;
+    }
+  }
+  const float mul = a.scale * temperature(a, pos);
 #pragma unroll
-      for (int j = 0; j < 8; ++j) x[j] = key < pos ? (float)kv[u].v[j] : newest ? knew[d0 + j] : 0.0f;
+  for (int u = 0; u < U; ++u) {
+    if (u >= uk) break;
+    const int i = (u * 4 + wave) * kpw + sub, key = b + i;
+    float x[8];
 #pragma unroll
-      for (int r = 0; r < R; ++r) {
-        float dot = 0.0f;
+    for (int j = 0; j < 8; ++j) x[j] = key < pos ? (float)kv[u].v[j] : kn[j];
 #pragma unroll
-        for (int j = 0; j < 8; ++j) dot = __builtin_fmaf(qv[r][j], x[j], dot);
-        for (int off = lpk >> 1; off > 0; off >>= 1) dot += __shfl_xor(dot, off, 64);
-        if (d0 == 0 && i < nk && r < nr) sc[r * kPartKeys + i] = dot * mul - a.slope[h0 + r] * (float)(pos - key);
-      }
+    for (int r = 0; r < R; ++r) {
+      float dot = 0.0f;
+#pragma unroll
+      for (int j = 0; j < 8; ++j) dot = __builtin_fmaf(qv[r][j], x[j], dot);
+      for (int off = lpk >> 1; off > 0; off >>= 1) dot += __shfl_xor(dot, off, 64);
+      if (d0 == 0) sc[r][i] = dot;
     }
   }
   __syncthreads();
-  for (int r = wave; r < nr; r += 4) {
-    const float s0 = lane < nk ? sc[r * kPartKeys + lane] : -INFINITY;
-    const float s1 = lane + 64 < nk ? sc[r * kPartKeys + lane + 64] : -INFINITY;
-    float m = fmaxf(s0, s1);
+  // every wavefront: lane = key
+  float p[R], pm[R], pl[R];
+#pragma unroll
+  for (int r = 0; r < R; ++r) {
+    const float s = lane < nk && r < nr ? sc[r][lane] * mul - a.slope[h0 + r] * (float)(pos - b - lane) : -INFINITY;
+    float m = s;
 #pragma unroll
     for (int off = 32; off > 0; off >>= 1) m = fmaxf(m, __shfl_xor(m, off, 64));
-    const float e0 = expf(s0 - m), e1 = expf(s1 - m);
-    float l = e0 + e1;
+    const float e = r < nr ? expf(s - m) : 0.0f;
+    float l = e;
 #pragma unroll
     for (int off = 32; off > 0; off >>= 1) l += __shfl_xor(l, off, 64);
-    sc[r * kPartKeys + lane] = e0;
-    sc[r * kPartKeys + lane + 64] = e1;
-    if (lane == 0) part_m[r] = m, part_l[r] = l;
+    p[r] = e;
+    pm[r] = m;
+    pl[r] = l;
   }
-  __syncthreads();
-  // context: 8 columns of every kth key per thread
-  const int tpv = vw >> 3, c0 = (tid % tpv) * 8, first = tid / tpv, step = 256 / tpv;
   float acc[R][8] = {};
-  const T* const vc = reinterpret_cast<const T*>(a.v_cache);
-  for (int k0 = first; k0 < nk; k0 += 4 * step) {
-    Vec8<T> vv[4];
 #pragma unroll
-    for (int u = 0; u < 4; ++u) {
-      const int key = min(b + k0 + u * step, pos);
-      if (key < pos) vv[u].load(vc + ring_row(a.vl, g, key % a.vl.slots) + c0);
-    }
+  for (int u = 0; u < U; ++u) {
+    if (u >= uv) break;
+    const int i = u * step + first;
+    float x[8];
 #pragma unroll
-    for (int u = 0; u < 4; ++u) {
-      const int i = k0 + u * step;
-      if (i >= nk) break;
-      float x[8];
+    for (int j = 0; j < 8; ++j) x[j] = b + i < pos ? (float)vv[u].v[j] : vn[j];
 #pragma unroll
-      for (int j = 0; j < 8; ++j) x[j] = b + i < pos ? (float)vv[u].v[j] : vnew[c0 + j];
+    for (int r = 0; r < R; ++r) {
+      const float w = __shfl(p[r], i, 64);
 #pragma unroll
-      for (int r = 0; r < R; ++r) {
-        if (r >= nr) break;
-        const float p = sc[r * kPartKeys + i];
-#pragma unroll
-        for (int j = 0; j < 8; ++j) acc[r][j] = __builtin_fmaf(p, x[j], acc[r][j]);
-      }
+      for (int j = 0; j < 8; ++j) acc[r][j] = __builtin_fmaf(w, i < nk ? x[j] : 0.0f, acc[r][j]);
     }
   }
   // lanes of a wavefront that share columns, then the wavefronts
@@ -260,56 +292,53 @@ __global__ __launch_bounds__(256) void window_decode_kernel(WindowAttnArgs a, in
       if (lane < tpv) red[(wave * R + r) * vw + c0 + j] = acc[r][j];
     }
   __syncthreads();
-  T* const out = reinterpret_cast<T*>(a.ctx) + (int64_t)h0 * a.vdim;
-  auto total = [&](int r, int c) {
-    return (red[r * vw + c] + red[(R + r) * vw + c]) + (red[(2 * R + r) * vw + c] + red[(3 * R + r) * vw + c]);
-  };
-  if (parts == 1) {
-    for (int i = tid; i < nr * a.vdim; i += 256) {
-      const int r = i / a.vdim, c = i - r * a.vdim;
-      out[i] = (T)(total(r, c) / part_l[r]);
+  const int n_parts = gridDim.y;
+#pragma unroll
+  for (int r = 0; r < R; ++r) {
+    if (r >= nr) break;
+    float* const mine = a.parts + ((int64_t)(h0 + r) * n_parts + part) * (2 + a.vdim);
+    for (int c = tid; c < a.vdim; c += 256) {
+      const float x = (red[r * vw + c] + red[(R + r) * vw + c]) + (red[(2 * R + r) * vw + c] + red[(3 * R + r) * vw + c]);
+      if (n_parts == 1)
+        reinterpret_cast<T*>(a.ctx)[(int64_t)(h0 + r) * a.vdim + c] = (T)(x / pl[r]);
+      else
+        mine[2 + c] = x;
     }
-    return;
-  }
-  // [head][part][2 + vdim]: maximum, sum, context
-  const int64_t ps = 2 + a.vdim, hs = (int64_t)gridDim.y * ps;
-  float* const mine = a.parts + (int64_t)h0 * hs + part * ps;
-  for (int i = tid; i < nr * a.vdim; i += 256) {
-    const int r = i / a.vdim, c = i - r * a.vdim;
-    __hip_atomic_store(mine + r * hs + 2 + c, total(r, c), __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
-  }
-  if (tid < nr) {
-    __hip_atomic_store(mine + tid * hs, part_m[tid], __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
-    __hip_atomic_store(mine + tid * hs + 1, part_l[tid], __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
-  }
-  __threadfence();
-  __syncthreads();
-  if (tid == 0) {
-    const int n = __hip_atomic_fetch_add(a.counters + blockIdx.x, 1, __ATOMIC_ACQ_REL, __HIP_MEMORY_SCOPE_AGENT);
-    last = n == parts - 1;
-    if (last) __hip_atomic_store(a.counters + blockIdx.x, 0, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
-  }
-  __syncthreads();
-  if (!last) return;
-  __threadfence();
-  for (int i = tid; i < nr * a.vdim; i += 256) {
-    const int r = i / a.vdim, c = i - r * a.vdim;
-    const float* p = a.parts + (int64_t)(h0 + r) * hs;
-    float m = -INFINITY, l = 0.0f, x = 0.0f;
-    for (int s = 0; s < parts; ++s)
-      m = fmaxf(m, __hip_atomic_load(p + s * ps, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT));
-    for (int s = 0; s < parts; ++s) {
-      const float w = expf(__hip_atomic_load(p + s * ps, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT) - m);
-      l = __builtin_fmaf(w, __hip_atomic_load(p + s * ps + 1, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT), l);
-      x = __builtin_fmaf(w, __hip_atomic_load(p + s * ps + 2 + c, __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT), x);
-    }
-    out[i] = (T)(x / l);
+    if (n_parts > 1 && tid == 0) mine[0] = pm[r], mine[1] = pl[r];
   }
 }
 
-int decode_rows(const WindowAttnArgs& a) {
-  const int per = a.heads / a.kv_heads;
-  return per >= 8 ? 8 : per > 2 ? (per > 4 ? 8 : 4) : per;
+// a workgroup per head; a part is [maximum, sum, context]
+template <typename T>
+__global__ __launch_bounds__(256) void window_combine_kernel(WindowAttnArgs a, int n_parts) {
+  __shared__ float red[256];
+  const int h = blockIdx.x, tid = threadIdx.x, lane = tid & 63;
+  const int pos = a.pos.position();
+  const int parts = ((a.window > 0 ? min(a.window, pos + 1) : pos + 1) + kPartKeys - 1) / kPartKeys;
+  const int64_t ps = 2 + a.vdim;
+  const float* p = a.parts + (int64_t)h * n_parts * ps;
+  float m = -INFINITY, l = 0.0f;
+  for (int s = lane; s < parts; s += 64) m = fmaxf(m, p[s * ps]);
+#pragma unroll
+  for (int off = 32; off > 0; off >>= 1) m = fmaxf(m, __shfl_xor(m, off, 64));
+  for (int s = lane; s < parts; s += 64) l = __builtin_fmaf(expf(p[s * ps] - m), p[s * ps + 1], l);
+#pragma unroll
+  for (int off = 32; off > 0; off >>= 1) l += __shfl_xor(l, off, 64);
+  // columns, and as many runs of parts next to each other as there are threads left
+  const int cols = min(256, a.vdim), runs = 256 / cols, run = tid / cols;
+  for (int c = tid % cols; c < (a.vdim + cols - 1) / cols * cols; c += cols) {
+    float x = 0.0f;
+    if (run < runs && c < a.vdim)
+#pragma unroll 4
+      for (int s = run; s < parts; s += runs) x = __builtin_fmaf(expf(p[s * ps] - m), p[s * ps + 2 + c], x);
+    red[tid] = x;
+    __syncthreads();
+    if (run == 0 && c < a.vdim) {
+      for (int i = 1; i < runs; ++i) x += red[tid + i * cols];
+      reinterpret_cast<T*>(a.ctx)[(int64_t)h * a.vdim + c] = (T)(x / l);
+    }
+    __syncthreads();
+  }
 }
 
 template <typename T, int R>
@@ -317,21 +346,27 @@ int launch_decode_rows(const WindowAttnArgs& a, hipStream_t st) {
   const int chunks = (a.heads / a.kv_heads + R - 1) / R;
   const int parts = window_parts(a.window, a.len_bound);
   AWQ_REQUIRE(parts >= 1 && parts <= 65535, "too many keys");
-  const size_t lds = sizeof(float) * ((size_t)R * kPartKeys + a.kl.row + a.vl.row + (size_t)4 * R * a.vl.row);
-  hipLaunchKernelGGL((window_decode_kernel<T, R>), dim3((unsigned)(a.kv_heads * chunks), (unsigned)parts), dim3(256), lds, st,
-                     a, chunks);
+  const dim3 g((unsigned)(a.kv_heads * chunks), (unsigned)parts);
+  const size_t lds = sizeof(float) * 4 * R * a.vl.row;
+  const int row = std::max(a.kl.row, a.vl.row);
+  if (row == 64) hipLaunchKernelGGL((window_decode_kernel<T, R, 2>), g, dim3(256), lds, st, a, chunks);
+  else if (row == 128) hipLaunchKernelGGL((window_decode_kernel<T, R, 4>), g, dim3(256), lds, st, a, chunks);
+  else hipLaunchKernelGGL((window_decode_kernel<T, R, 8>), g, dim3(256), lds, st, a, chunks);
   AWQ_HIP_TRY(hipGetLastError());
+  if (parts > 1) {
+    hipLaunchKernelGGL(window_combine_kernel<T>, dim3((unsigned)a.heads), dim3(256), 0, st, a, parts);
+    AWQ_HIP_TRY(hipGetLastError());
+  }
   return AWQ_OK;
 }
 
 template <typename T>
 int launch_decode(const WindowAttnArgs& a, hipStream_t st) {
-  switch (decode_rows(a)) {
-    case 1: return launch_decode_rows<T, 1>(a, st);
-    case 2: return launch_decode_rows<T, 2>(a, st);
-    case 4: return launch_decode_rows<T, 4>(a, st);
-    default: return launch_decode_rows<T, 8>(a, st);
-  }
+  const int per = a.heads / a.kv_heads;
+  if (per == 1) return launch_decode_rows<T, 1>(a, st);
+  if (per == 2) return launch_decode_rows<T, 2>(a, st);
+  if (per <= 4) return launch_decode_rows<T, 4>(a, st);
+  return launch_decode_rows<T, 8>(a, st);
 }
 
 // Many tokens, bfloat16.  128 queries of one head per workgroup, 32 per wavefront; keys and values of 32 positions at
@@ -522,6 +557,14 @@ void launch_tiles(const WindowAttnArgs& a, hipStream_t st) {
 
 template <typename T>
 int launch_append(const WindowAttnArgs& a, hipStream_t st) {
+  const int row = std::max(a.kl.row, a.vl.row);
+  if (sizeof(T) == 2 && ((a.dim | a.vdim) & 7) == 0 && row <= 256) {
+    const int lanes = row / 8, per = 256 / lanes;
+    const int64_t n = (int64_t)(a.heads + 2 * a.kv_heads) * a.M;
+    hipLaunchKernelGGL(window_append8_kernel, dim3((unsigned)((n + per - 1) / per)), dim3(256), 0, st, a, lanes);
+    AWQ_HIP_TRY(hipGetLastError());
+    return AWQ_OK;
+  }
   const dim3 g((unsigned)((a.heads + 2 * a.kv_heads + 3) / 4), (unsigned)a.M);
   hipLaunchKernelGGL(window_append_kernel<T>, g, dim3(256), 0, st, a);
   AWQ_HIP_TRY(hipGetLastError());
@@ -544,7 +587,6 @@ int32_t window_row_padded(int32_t dim) { return dim <= 64 ? 64 : dim <= 128 ? 12
 int64_t window_parts_floats(int32_t heads, int32_t vdim, int64_t window, int64_t max_pos) {
   return (int64_t)heads * window_parts(window, max_pos) * (2 + vdim);
 }
-int64_t window_counter_count(int32_t heads, int32_t kv_heads) { return heads; }
 
 int launch_window_attention(const WindowAttnArgs& a, bool f32, hipStream_t st) {
   AWQ_REQUIRE(a.proj && a.k_cache && a.v_cache && a.ctx && a.slope && a.M >= 1 && a.M <= 65535, "bad arguments");
@@ -554,7 +596,7 @@ int launch_window_attention(const WindowAttnArgs& a, bool f32, hipStream_t st) {
                   a.vl.row == window_row_padded(a.vdim) && a.ldp % 8 == 0 && a.ldc % 8 == 0,
               "bad cache layout");
   const bool tiled = a.kl.row <= 256 && a.vl.row <= 256;
-  if (a.M == 1 && tiled && a.parts && a.counters && a.len_bound > 0)
+  if (a.M == 1 && tiled && a.parts && a.len_bound > 0)
     return f32 ? launch_decode<float>(a, st) : launch_decode<bf16_t>(a, st);
   if (int rc = f32 ? launch_append<float>(a, st) : launch_append<bf16_t>(a, st)) return rc;
   if (f32) return launch_queries<float>(a, st);

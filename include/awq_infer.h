@@ -442,6 +442,101 @@ int awq_logits_argmax(const void* logits, int64_t n, void* out_token, void* work
 int awq_embed_gather(const void* packed, const void* scale, const void* zp, int64_t hidden, int64_t vocab,
                      int32_t tok, void* out, void* stream);
 
+/* ----------------------------------------------------------------------------
+ * Layer building blocks of the models that a config.json describes; no
+ * counterpart in the reference.  `f32` != 0: weights and activations are
+ * binary32 and so is every product; 0: they are bfloat16 with binary32 sums.
+ * What is float * here is binary32 in both forms.  Device pointers, 16-byte
+ * aligned; all sizes are arguments.
+ * ------------------------------------------------------------------------- */
+
+/* Dense products y[t][r] = act(sum_k w[r][k] x[t][k]) of one weight block whose
+ * rows form one or two segments, each with its own input and output.  A block
+ * has rows padded to a multiple of 256 per segment and k padded with zeros to a
+ * multiple of 64 (both chosen by the caller, who zero-fills the block, then
+ * packs each matrix [rows][cols] into it with awq_dense_pack). */
+#define AWQ_ACT_NONE 0
+#define AWQ_ACT_SILU 1  /* z * sigmoid(z) on the first act_rows rows of the segment */
+#define AWQ_ACT_XIELU 2 /* z > 0: act_pos z^2 + z/2; z <= 0: act_neg (exp(z) - 1 - z) + z/2 */
+#define AWQ_DENSE_STORE 0    /* y in the activations' type */
+#define AWQ_DENSE_RESIDUAL 1 /* y is float: y = (y + sum) + addend (may be NULL) */
+#define AWQ_DENSE_F32 2      /* y is float */
+typedef struct awq_dense_segment {
+  const void* x; /* [tokens][ldx], ldx a multiple of 8 */
+  void* y;       /* [tokens][ldy] */
+  int64_t ldx, ldy;
+  int32_t row0, rows; /* row0 a multiple of 256 */
+  int32_t act, act_rows;
+  float act_pos, act_neg;
+} awq_dense_segment;
+typedef struct awq_dense_args {
+  const void* w;
+  int64_t k, tokens;
+  int32_t n_segments, out;
+  awq_dense_segment segment[2];
+  const float* addend;
+  float* workspace; /* NULL, or workspace_floats of scratch for products that are cut along k */
+  int64_t workspace_floats;
+} awq_dense_args;
+int64_t awq_dense_weight_bytes(int64_t rows_padded, int64_t k_padded, int32_t f32);
+int awq_dense_pack(const void* src, int32_t src_f32, int64_t rows, int64_t cols, void* w, int64_t k_padded, int64_t row0,
+                   int64_t col0, int32_t f32, void* stream);
+int awq_dense(const awq_dense_args* args, int32_t f32, void* stream);
+
+/* x[t][i] = table[tokens[t]][i] * scale + (i even: sin, odd: cos)(position *
+ * freq[i / 2]); freq binary64 on the device */
+int awq_embed_sinusoid(const void* table, int32_t f32, const int32_t* tokens, int64_t pos0, int64_t n_tokens, int64_t width,
+                       float scale, const double* freq, float* x, void* stream);
+
+/* RMS norm in `groups` equal parts; out1 = h + conv(h) with h = norm(x) * w1 and
+ * conv a causal convolution over time per channel ([width][taps], NULL: none),
+ * out2 = norm(x) * w2 (w2 NULL: not formed).  state_in / state_out
+ * [taps - 1][width] float: the inputs h ahead of position pos0 and at the end
+ * (different buffers; rows ahead of position 0 count as zero). */
+int awq_norm_conv(const float* x, int64_t n_tokens, int64_t width, int32_t groups, float eps, const float* w1,
+                  const float* conv, int32_t taps, const float* state_in, float* state_out, void* out1, const float* w2,
+                  void* out2, int64_t ld, int64_t pos0, int32_t f32, void* stream);
+
+/* y = RMS norm over n of o, times w, times sigmoid(g) */
+int awq_gated_norm(const float* o, int64_t ldo, const void* g, int64_t ldg, const float* w, void* y, int64_t ldy, int64_t n,
+                   int64_t n_tokens, float eps, int32_t f32, void* stream);
+
+/* Attention of n_tokens new positions pos0.. over a window of `window` positions
+ * (0: all), query head h on key/value head h / (heads / kv_heads): q and k are
+ * divided by their RMS per head, the score at position p of a key at distance d
+ * is (q . k) * scale * (1 + temp_coef ln(floor((p + 1) / temp_every) + 1)) -
+ * slope[h] * d, softmax, weighted sum of v.  proj [n_tokens][ldp] holds q, k, v
+ * side by side (q is normalised in place).  The caches hold rows of
+ * awq_window_row(dim) / awq_window_row(vdim) elements, [slots / 64][kv_heads][64]
+ * of them; a position's slot is position % slots, slots a multiple of 64 and at
+ * least window - 1 + n_tokens (or every position).  workspace:
+ * awq_window_workspace_floats floats, needed for single tokens. */
+typedef struct awq_window_args {
+  void* proj;
+  int64_t ldp;
+  int32_t heads, kv_heads, dim, vdim, window, slots;
+  float scale, eps, temp_coef, reserved;
+  double temp_every;
+  const float* slope;
+  void* k_cache;
+  void* v_cache;
+  void* ctx;
+  int64_t ldc, n_tokens, pos0, max_pos;
+  float* workspace;
+} awq_window_args;
+int32_t awq_window_row(int32_t dim);
+int64_t awq_window_workspace_floats(int32_t heads, int32_t vdim, int64_t window, int64_t max_pos);
+int awq_window_attention(const awq_window_args* args, int32_t f32, void* stream);
+
+/* Linear attention: per head S <- decay S + k v^T, o = S^T q for n_tokens
+ * positions from pos0; the state [heads][vdim][dim padded to 64] float (S
+ * transposed) is zero ahead of position 0 and carried from call to call.
+ * log2_decay: NULL, or the decays' logarithms, all finite: many tokens then go
+ * through the matrix cores in chunks. */
+int awq_linear_attention(const void* proj, int64_t ldp, int32_t heads, int32_t dim, int32_t vdim, const float* decay,
+                         const float* log2_decay, float* state, float* o, int64_t n_tokens, int64_t pos0, int32_t f32,
+                         void* stream);
+
 #ifdef __cplusplus
 }
 #endif
