@@ -139,6 +139,49 @@ int read_spec(const std::string& dir, Spec* s) {
   return AWQ_OK;
 }
 
+// every tensor of the model and its shape
+std::vector<std::pair<std::string, std::vector<int64_t>>> expected_tensors(const Spec& c) {
+  const int64_t W = c.width;
+  std::vector<std::pair<std::string, std::vector<int64_t>>> v = {{"embed", {c.vocab, W}}, {"final.norm", {W}}, {"head", {c.vocab, W}}};
+  for (size_t i = 0; i < c.layers.size(); ++i) {
+    const LayerSpec& s = c.layers[i];
+    const std::string p = "l" + std::to_string(i) + ".", m = p + "mix.";
+    const int64_t mixed = s.mixed(), kv = s.type == MIX_ATTENTION ? s.kv_heads : s.heads;
+    v.push_back({p + "norm1", {W}});
+    v.push_back({p + "canon1", {W, c.taps}});
+    v.push_back({m + "q", {(int64_t)s.heads * s.dim, W}});
+    v.push_back({m + "k", {kv * s.dim, W}});
+    v.push_back({m + "v", {kv * s.vdim, W}});
+    v.push_back({m + "o", {W, mixed}});
+    if (s.type == MIX_LIGHTNING) {
+      v.push_back({m + "g", {mixed, W}});
+      v.push_back({m + "norm", {mixed}});
+    }
+    if (s.ff) {
+      v.push_back({p + "norm2", {W}});
+      v.push_back({p + "mlp.up", {s.ff, W}});
+      v.push_back({p + "mlp.down", {W, s.ff}});
+      v.push_back({p + "mlp.act", {2}});
+    }
+  }
+  return v;
+}
+
+int check_tensors(const Spec& c, const Safetensors& file) {
+  for (const auto& want : expected_tensors(c)) {
+    const Tensor* t = file.find(want.first);
+    if (!t) {
+      awq_set_error("model.safetensors has no tensor " + want.first);
+      return AWQ_ERR_IO;
+    }
+    if (t->shape != want.second || (t->dtype != "BF16" && t->dtype != "F32")) {
+      awq_set_error("tensor " + want.first + " has another shape or type than config.json says");
+      return AWQ_ERR_IO;
+    }
+  }
+  return AWQ_OK;
+}
+
 // --- the model ---------------------------------------------------------------------------------------------
 struct LayerDev {
   const float *norm1 = nullptr, *norm2 = nullptr, *conv = nullptr;
@@ -223,7 +266,7 @@ struct KugilixEngine final : awq_engine {
     if (int rc = dev_alloc(p, bytes)) return rc;
     return launch_fill_zero(*p, bytes, stream);
   }
-  int load(const std::string& dir);
+  int load(const Safetensors& file);
   int make_buffers(Buffers* b, int64_t n_tokens);
   int make_runs();
   int run_layers(Buffers& b, int64_t M, PassPos pos);
@@ -236,41 +279,25 @@ struct Loader {
   const Safetensors& file;
   void* staging = nullptr;
 
-  // the tensor, its shape checked
-  int get(const std::string& name, const std::vector<int64_t>& shape, const Tensor** out) {
-    const Tensor* t = file.find(name);
-    if (!t) {
-      awq_set_error("model.safetensors has no tensor " + name);
-      return AWQ_ERR_IO;
-    }
-    if (t->shape != shape || (t->dtype != "BF16" && t->dtype != "F32")) {
-      awq_set_error("tensor " + name + " has another shape or type than config.json says");
-      return AWQ_ERR_IO;
-    }
-    *out = t;
-    return AWQ_OK;
-  }
   int stage(const Tensor* t) {
     AWQ_HIP_TRY(hipMemcpyAsync(staging, t->data, (size_t)t->bytes, hipMemcpyHostToDevice, e->stream));
     return AWQ_OK;
   }
   static bool wide(const Tensor* t) { return t->dtype == "F32"; }
-  int vector(const std::string& name, std::vector<int64_t> shape, const float** out) {
-    const Tensor* t;
-    if (int rc = get(name, shape, &t)) return rc;
+  int vector(const std::string& name, const float** out) {
+    const Tensor* t = file.find(name);
     int64_t n = 1;
-    for (int64_t d : shape) n *= d;
+    for (int64_t d : t->shape) n *= d;
     float* dst = nullptr;
     if (int rc = e->dev_alloc((void**)&dst, n * 4)) return rc;
     if (int rc = stage(t)) return rc;
     *out = dst;
     return launch_convert(staging, wide(t), dst, true, n, e->stream);
   }
-  int matrix(const std::string& name, int64_t rows, int64_t cols, void* w, int64_t k, int64_t row0, int64_t col0) {
-    const Tensor* t;
-    if (int rc = get(name, {rows, cols}, &t)) return rc;
+  int matrix(const std::string& name, void* w, int64_t k, int64_t row0, int64_t col0) {
+    const Tensor* t = file.find(name);
     if (int rc = stage(t)) return rc;
-    return launch_dense_pack(staging, wide(t), rows, cols, w, k, row0, col0, e->f32, e->stream);
+    return launch_dense_pack(staging, wide(t), t->shape[0], t->shape[1], w, k, row0, col0, e->f32, e->stream);
   }
   int block(void** w, int64_t rows, int64_t k) { return e->zeroed(w, dense_weight_bytes(rows, k, e->f32)); }
   int constants(const std::vector<float>& v, const float** out) {
@@ -280,11 +307,10 @@ struct Loader {
     *out = dst;
     return AWQ_OK;
   }
-  int numbers(const std::string& name, int64_t n, std::vector<double>* out) {
-    const Tensor* t;
-    if (int rc = get(name, {n}, &t)) return rc;
+  void numbers(const std::string& name, std::vector<double>* out) {
+    const Tensor* t = file.find(name);
     out->clear();
-    for (int64_t i = 0; i < n; ++i) {
+    for (int64_t i = 0; i < t->shape[0]; ++i) {
       uint32_t bits;
       if (wide(t))
         memcpy(&bits, (const char*)t->data + 4 * i, 4);
@@ -297,7 +323,6 @@ struct Loader {
       memcpy(&f, &bits, 4);
       out->push_back(f);
     }
-    return AWQ_OK;
   }
 };
 
@@ -308,8 +333,8 @@ int load_layer(Loader& ld, KugilixEngine* e, int i) {
   const int64_t W = e->spec.width;
   LayerDev L;
   const std::string p = "l" + std::to_string(i) + ".", m = p + "mix.";
-  if (int rc = ld.vector(p + "norm1", {W}, &L.norm1)) return rc;
-  if (int rc = ld.vector(p + "canon1", {W, e->spec.taps}, &L.conv)) return rc;
+  if (int rc = ld.vector(p + "norm1", &L.norm1)) return rc;
+  if (int rc = ld.vector(p + "canon1", &L.conv)) return rc;
   struct Part {
     const char* name;
     int64_t rows;
@@ -328,24 +353,24 @@ int load_layer(Loader& ld, KugilixEngine* e, int i) {
   if (int rc = ld.block(&L.w_in, L.up_row + round_up(s.ff, kDenseRowAlign), e->ld)) return rc;
   int64_t at = 0;
   for (const Part& q : parts) {
-    if (int rc = ld.matrix(m + q.name, q.rows, W, L.w_in, e->ld, at, 0)) return rc;
+    if (int rc = ld.matrix(m + q.name, L.w_in, e->ld, at, 0)) return rc;
     at += q.rows;
   }
   L.mixed_k = round_up(s.mixed(), kDenseKAlign);
   L.k_out = L.mixed_k + round_up(s.ff, kDenseKAlign);
   if (int rc = ld.block(&L.w_out, round_up(W, kDenseRowAlign), L.k_out)) return rc;
-  if (int rc = ld.matrix(m + "o", W, s.mixed(), L.w_out, L.k_out, 0, 0)) return rc;
+  if (int rc = ld.matrix(m + "o", L.w_out, L.k_out, 0, 0)) return rc;
   if (s.ff) {
-    if (int rc = ld.vector(p + "norm2", {W}, &L.norm2)) return rc;
-    if (int rc = ld.matrix(p + "mlp.up", s.ff, W, L.w_in, e->ld, L.up_row, 0)) return rc;
-    if (int rc = ld.matrix(p + "mlp.down", W, s.ff, L.w_out, L.k_out, 0, L.mixed_k)) return rc;
+    if (int rc = ld.vector(p + "norm2", &L.norm2)) return rc;
+    if (int rc = ld.matrix(p + "mlp.up", L.w_in, e->ld, L.up_row, 0)) return rc;
+    if (int rc = ld.matrix(p + "mlp.down", L.w_out, L.k_out, 0, L.mixed_k)) return rc;
     std::vector<double> act;
-    if (int rc = ld.numbers(p + "mlp.act", 2, &act)) return rc;
+    ld.numbers(p + "mlp.act", &act);
     L.act_pos = (float)softplus(act[0]);
     L.act_neg = (float)(0.5 + softplus(act[1]));
   }
   if (s.type == MIX_LIGHTNING) {
-    if (int rc = ld.vector(m + "norm", {s.mixed()}, &L.mix_norm)) return rc;
+    if (int rc = ld.vector(m + "norm", &L.mix_norm)) return rc;
     if (int rc = ld.constants(std::vector<float>(s.decay.begin(), s.decay.end()), &L.decay)) return rc;
     std::vector<float> lg;
     for (double d : s.decay)
@@ -361,10 +386,8 @@ int load_layer(Loader& ld, KugilixEngine* e, int i) {
   return AWQ_OK;
 }
 
-int KugilixEngine::load(const std::string& dir) {
+int KugilixEngine::load(const Safetensors& file) {
   const auto t0 = std::chrono::steady_clock::now();
-  Safetensors file;
-  if (int rc = file.open(dir + "/model.safetensors")) return rc;
   Loader ldr{this, file};
   int64_t largest = 4;
   for (const auto& t : file.tensors()) largest = std::max(largest, t.second.bytes);
@@ -372,14 +395,13 @@ int KugilixEngine::load(const std::string& dir) {
   const auto all = [&]() -> int {
     const int64_t W = spec.width, V = spec.vocab;
     ld = round_up(W, kDenseKAlign);
-    const Tensor* t;
-    if (int rc = ldr.get("embed", {V, W}, &t)) return rc;
+    const Tensor* t = file.find("embed");
     if (int rc = dev_alloc(&embed, V * W * unit())) return rc;
     if (int rc = ldr.stage(t)) return rc;
     if (int rc = launch_convert(ldr.staging, Loader::wide(t), embed, f32, V * W, stream)) return rc;
-    if (int rc = ldr.vector("final.norm", {W}, &final_norm)) return rc;
+    if (int rc = ldr.vector("final.norm", &final_norm)) return rc;
     if (int rc = ldr.block(&head, round_up(V, kDenseRowAlign), ld)) return rc;
-    if (int rc = ldr.matrix("head", V, W, head, ld, 0, 0)) return rc;
+    if (int rc = ldr.matrix("head", head, ld, 0, 0)) return rc;
     std::vector<double> f;
     for (int64_t i = 0; 2 * i < W; ++i) f.push_back(pow(10000.0, -2.0 * (double)i / (double)W));
     double* fd = nullptr;
@@ -713,7 +735,11 @@ int64_t KugilixEngine::read_layer_tap(float* host_dst, int64_t capacity) {
 
 int open_kugilix(const char* dir, const awq_open_options& opt, awq_engine** out) {
   std::unique_ptr<KugilixEngine> e(new KugilixEngine());
+  // look at the folder before touching the GPU
+  Safetensors file;
   if (int rc = read_spec(dir, &e->spec)) return rc;
+  if (int rc = file.open(std::string(dir) + "/model.safetensors")) return rc;
+  if (int rc = check_tensors(e->spec, file)) return rc;
   e->f32 = opt.dtype == AWQ_DTYPE_FLOAT32;
   e->max_pos = opt.max_positions ? opt.max_positions : kDefaultPositions;
   AWQ_REQUIRE(e->max_pos <= (1 << 24), "max_positions is too large");
@@ -721,7 +747,7 @@ int open_kugilix(const char* dir, const awq_open_options& opt, awq_engine** out)
   e->bounds = {1ll << 40};
   e->batched_prefill = true;
   if (int rc = e->init_driver(e->max_pos)) return rc;
-  if (int rc = e->load(dir)) return rc;
+  if (int rc = e->load(file)) return rc;
   if (int rc = e->make_buffers(&e->step, 1)) return rc;
   if (int rc = e->make_buffers(&e->pass, e->pass_tokens)) return rc;
   if (int rc = e->make_runs()) return rc;

@@ -86,7 +86,8 @@ constexpr int linear_chunk_lds() {
   return (kChunk * (D + 16) + 4 * 32 * kVStride + 3 * 32 * (D + 8)) * 2;
 }
 
-template <int D>
+// WHOLE: rows of q, k and v are 16-byte pieces
+template <int D, bool WHOLE>
 __global__ __launch_bounds__(512) void linear_chunk_kernel(LinearAttnArgs a) {
   extern __shared__ __attribute__((aligned(16))) char lds_raw[];
   constexpr int KS = D + 16, SS = D + 8, NT = D / 32;  // NT tiles of 32 state rows, over four wavefronts
@@ -106,14 +107,13 @@ __global__ __launch_bounds__(512) void linear_chunk_kernel(LinearAttnArgs a) {
   const bf16_t* const k = p + (int64_t)(a.heads + head) * a.dim;
   const bf16_t* const v = p + (int64_t)2 * a.heads * a.dim + (int64_t)head * a.vdim + v0;
   const int nv = min(32, a.vdim - v0);
-  const bool whole = (a.dim & 7) == 0 && (a.vdim & 7) == 0;  // rows of 16-byte pieces
   const float lg = a.log2_decay[head];
   const int dimp = (a.dim + 63) & ~63;
   float* const state = a.state + ((int64_t)head * a.vdim + v0 + n) * dimp;
 
   auto piece = [&](const bf16_t* row, int at, int len) __attribute__((always_inline)) {
     bf16x8_t r;
-    if (whole) {
+    if constexpr (WHOLE) {
       if (at < len) return *reinterpret_cast<const bf16x8_t*>(row + at);
 #pragma unroll
       for (int e = 0; e < 8; ++e) r[e] = (bf16_t)0.0f;
@@ -150,7 +150,20 @@ __global__ __launch_bounds__(512) void linear_chunk_kernel(LinearAttnArgs a) {
     for (int i = 0; i < 2; ++i)
       if (outputs) vr[i] = piece(v + (int64_t)min(c0 + 2 * lane + i, M - 1) * a.ldp, 8 * wave, nv);
   };
+  // this lane's query: token 32 wave + n
+  const int tq = 32 * wave + n;
+  bf16x8_t qop[D / 16];
+  auto load_q = [&](int c0) __attribute__((always_inline)) {
+#pragma unroll
+    for (int i = 0; i < D / 16; ++i)
+      qop[i] = piece(q + (int64_t)min(c0 + tq, M - 1) * a.ldp, 16 * i + 8 * kh, a.dim);
+  };
+  // decay^(31 - s) for this lane's rows s of a tile of 32
+  float wr[16];
+#pragma unroll
+  for (int i = 0; i < 16; ++i) wr[i] = __builtin_amdgcn_exp2f((float)(31 - (8 * (i >> 2) + 4 * kh + (i & 3))) * lg);
   load(0);
+  if (outputs) load_q(0);
   for (int c0 = 0; c0 < M; c0 += kChunk) {
     const int len = min(kChunk, M - c0);
     __syncthreads();  // the previous chunk's readers are done
@@ -206,13 +219,6 @@ __global__ __launch_bounds__(512) void linear_chunk_kernel(LinearAttnArgs a) {
             *reinterpret_cast<bf16x4_t*>(st + (m * 32 + n) * SS + 32 * (wave + 4 * i) + 8 * g + 4 * kh) = out[m];
         }
     }
-    // this lane's query: token 32 wave + n
-    const int tq = 32 * wave + n;
-    bf16x8_t qop[D / 16];
-    if (outputs)
-#pragma unroll
-      for (int i = 0; i < D / 16; ++i)
-        qop[i] = piece(q + (int64_t)min(c0 + tq, M - 1) * a.ldp, 16 * i + 8 * kh, a.dim);
     __syncthreads();
     if (c0 + kChunk < M) load(c0 + kChunk);
 
@@ -246,11 +252,22 @@ __global__ __launch_bounds__(512) void linear_chunk_kernel(LinearAttnArgs a) {
         }
 #pragma unroll
         for (int i = 0; i < 16; ++i) w[i] += w2[i];
+        // decay^(t - s) = decay^(t - 31 - s0) decay^(31 + s0 - s); in the diagonal tile only s <= t counts
+        if (s0 < 32 * wave) {
+          const float wc = __builtin_amdgcn_exp2f((float)(tq - 31 - s0) * lg);
+#pragma unroll
+          for (int i = 0; i < 16; ++i) w[i] *= wr[i] * wc;
+        } else {
+#pragma unroll
+          for (int i = 0; i < 16; ++i) {
+            const int back = tq - (s0 + 8 * (i >> 2) + 4 * kh + (i & 3));
+            w[i] = back >= 0 ? w[i] * __builtin_amdgcn_exp2f((float)back * lg) : 0.0f;
+          }
+        }
         bf16x8_t hi[2], lo[2];
 #pragma unroll
         for (int i = 0; i < 16; ++i) {
-          const int back = tq - (s0 + 8 * (i >> 2) + 4 * kh + (i & 3));
-          const float x = back >= 0 ? w[i] * __builtin_amdgcn_exp2f((float)back * lg) : 0.0f;
+          const float x = w[i];
           hi[i >> 3][i & 7] = (bf16_t)x;
           lo[i >> 3][i & 7] = (bf16_t)(x - (float)hi[i >> 3][i & 7]);
         }
@@ -265,6 +282,7 @@ __global__ __launch_bounds__(512) void linear_chunk_kernel(LinearAttnArgs a) {
       }
 #pragma unroll
       for (int i = 0; i < 16; ++i) o[i] += o2[i];
+      if (c0 + kChunk < M) load_q(c0 + kChunk);
       if (tq < len) {
         float* out = a.o + (int64_t)(c0 + tq) * a.heads * a.vdim + (int64_t)head * a.vdim + v0;
 #pragma unroll
@@ -328,15 +346,15 @@ __global__ __launch_bounds__(512) void linear_chunk_kernel(LinearAttnArgs a) {
       }
 }
 
-template <int D>
+template <int D, bool WHOLE>
 int launch_chunks(const LinearAttnArgs& a, hipStream_t st) {
   static bool raised = false;  // more LDS than the default limit of a launch
   if (!raised) {
-    AWQ_HIP_TRY(hipFuncSetAttribute((const void*)linear_chunk_kernel<D>, hipFuncAttributeMaxDynamicSharedMemorySize,
+    AWQ_HIP_TRY(hipFuncSetAttribute((const void*)linear_chunk_kernel<D, WHOLE>, hipFuncAttributeMaxDynamicSharedMemorySize,
                                     linear_chunk_lds<D>()));
     raised = true;
   }
-  hipLaunchKernelGGL(linear_chunk_kernel<D>, dim3((unsigned)a.heads, (unsigned)((a.vdim + 31) / 32)), dim3(512),
+  hipLaunchKernelGGL((linear_chunk_kernel<D, WHOLE>), dim3((unsigned)a.heads, (unsigned)((a.vdim + 31) / 32)), dim3(512),
                      linear_chunk_lds<D>(), st, a);
   AWQ_HIP_TRY(hipGetLastError());
   return AWQ_OK;
@@ -374,9 +392,10 @@ int launch_linear_attention(const LinearAttnArgs& a, bool f32, hipStream_t st) {
               "bad shape");
   if (f32) return launch_step<float>(a, st);
   if (a.log2_decay && a.M >= kChunkFrom && a.M < (1 << 30) && a.dim <= 256) {
-    if (a.dim <= 64) return launch_chunks<64>(a, st);
-    if (a.dim <= 128) return launch_chunks<128>(a, st);
-    return launch_chunks<256>(a, st);
+    const bool whole = ((a.dim | a.vdim) & 7) == 0;
+    if (a.dim <= 64) return whole ? launch_chunks<64, true>(a, st) : launch_chunks<64, false>(a, st);
+    if (a.dim <= 128) return whole ? launch_chunks<128, true>(a, st) : launch_chunks<128, false>(a, st);
+    return whole ? launch_chunks<256, true>(a, st) : launch_chunks<256, false>(a, st);
   }
   return launch_step<bf16_t>(a, st);
 }

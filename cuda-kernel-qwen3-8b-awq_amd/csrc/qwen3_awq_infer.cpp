@@ -16,6 +16,10 @@ QWen3AWQInfer::QWen3AWQInfer(const std::string& weight_dir, PromptMode prompt_mo
   if (prompt_mode == PromptMode::Batched) setBatchedPrefill(true);
 }
 
+QWen3AWQInfer::QWen3AWQInfer(const std::string& model_dir, const awq_open_options& options) : engine_(nullptr) {
+  die_on(awq_open(model_dir.c_str(), &options, &engine_), "QWen3AWQInfer");
+}
+
 QWen3AWQInfer::~QWen3AWQInfer() { awq_destroy(engine_); }
 
 std::vector<int> QWen3AWQInfer::generateResponse(const std::vector<int>& prompt_ids, int max_new_tokens) {

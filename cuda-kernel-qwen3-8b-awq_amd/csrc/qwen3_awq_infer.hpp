@@ -20,11 +20,14 @@
 #include <vector>
 
 struct awq_engine;
+struct awq_open_options;
 
 class QWen3AWQInfer {
  public:
   enum class PromptMode { TokenByToken, Batched };
   explicit QWen3AWQInfer(const std::string& weight_dir, PromptMode prompt_mode = PromptMode::TokenByToken);
+  // a folder of any model class (awq_open): its config.json names the class, options choose number format and capacity
+  QWen3AWQInfer(const std::string& model_dir, const awq_open_options& options);
   ~QWen3AWQInfer();
   QWen3AWQInfer(const QWen3AWQInfer&) = delete;
   QWen3AWQInfer& operator=(const QWen3AWQInfer&) = delete;
