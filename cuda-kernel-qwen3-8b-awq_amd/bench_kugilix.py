@@ -127,11 +127,12 @@ def measure(widths, only=False, prompts=(128, 1024), steps=128):
     lib = awq.load_library()
     from bench import _synthetic_engine
     res = {}
+    positions = max(prompts) + 8 + 2 * steps
     for width in widths:
         cfg = config(width)
         with tempfile.TemporaryDirectory() as d:
             write_model(d, cfg)
-            eng = awq.open_model(d, max_positions=4096)
+            eng = awq.open_model(d, max_positions=positions)
         r = run_engine(eng, VOCAB, prompts, steps)
         eng.close()
         params = matrix_params(cfg)
@@ -142,7 +143,7 @@ def measure(widths, only=False, prompts=(128, 1024), steps=128):
         res["kugilix_%d" % width] = r
         if only:
             continue
-        c = awq.make_config(n_layers=LAYERS, hidden=width, inter=3 * width, vocab=VOCAB, max_pos=4096)
+        c = awq.make_config(n_layers=LAYERS, hidden=width, inter=3 * width, vocab=VOCAB, max_pos=positions)
         eng = _synthetic_engine(awq, lib, c, 1, awq.SYNTH_BALANCED)
         r = run_engine(eng, VOCAB, prompts, steps)
         eng.close()

@@ -1,5 +1,5 @@
 // Shared declarations of the HIP side: FP16 vector types, error plumbing and
-// the launcher prototypes that the C ABI (api.cpp) and the engine call.
+// the launcher prototypes that the C ABI (kernel_api.cpp) and the int4 model (qwen3.cpp) call.
 #pragma once
 
 #include <hip/hip_runtime.h>

@@ -65,9 +65,13 @@ __device__ __forceinline__ void finish_one(const DenseArgs& a, const DenseSegmen
 // A workgroup owns 16 rows and all of k, its wavefronts a run of k each; a load of a wavefront is four pieces of 256
 // contiguous bytes of the block.  v_mfma_f32_16x16x32_bf16 with the token in every column: the matrix unit does the
 // additions, and nothing but loads stands between the wavefront and memory.
-template <int NW, int OUT>
+// GATED: the first gate_k inputs are formed here, RMS norm of o times w times sigmoid(g) (token_ops.hip has it as a
+// launch of its own for many tokens): every workgroup normalises for itself while its first weights are on their way.
+template <int NW, int OUT, bool GATED>
 __global__ __launch_bounds__(NW * 64) void dense_one_kernel(DenseArgs a) {
+  extern __shared__ __attribute__((aligned(16))) bf16_t gated[];  // [gate_k]
   __shared__ float part[NW][16];
+  __shared__ float squares[NW];
   const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
   const int row0 = blockIdx.x * 16;
   const DenseSegment& s = segment_of(a, row0);
@@ -83,18 +87,55 @@ __global__ __launch_bounds__(NW * 64) void dense_one_kernel(DenseArgs a) {
   const bf16x8_t* x = reinterpret_cast<const bf16x8_t*>(s.x) + c;
   f32x4_t acc = {0.0f, 0.0f, 0.0f, 0.0f};
   constexpr int U = 8;
-  int i = s0;
-  for (; i + U <= s1; i += U) {
-    bf16x8_t wv[U], xv[U];
+  bf16x8_t wv[U], xv[U];
+  auto weights = [&](int i) __attribute__((always_inline)) {
 #pragma unroll
     for (int u = 0; u < U; ++u) wv[u] = __builtin_nontemporal_load(w + (int64_t)(i + u) * 128);
+  };
+  auto input = [&](int i) __attribute__((always_inline)) {
+    if (GATED && i * 32 < a.gate_k) return reinterpret_cast<const bf16x8_t*>(gated)[i * 4 + c];
+    return x[i * 4];
+  };
+  int i = s0;
+  if (i + U <= s1) weights(i);
+  if constexpr (GATED) {
+    constexpr int NT = NW * 64;
+    const bf16_t* gate = reinterpret_cast<const bf16_t*>(a.gate_g);
+    float sq = 0.0f;
+    for (int j = tid * 4; j < a.gate_n; j += NT * 4) {
+      const f32x4_t o = *reinterpret_cast<const f32x4_t*>(a.gate_o + j);
 #pragma unroll
-    for (int u = 0; u < U; ++u) xv[u] = x[(i + u) * 4];
+      for (int e = 0; e < 4; ++e) sq = __builtin_fmaf(o[e], o[e], sq);
+    }
+#pragma unroll
+    for (int off = 32; off > 0; off >>= 1) sq += __shfl_xor(sq, off, 64);
+    if (lane == 0) squares[wave] = sq;
+    __syncthreads();
+    float all = 0.0f;
+#pragma unroll
+    for (int v = 0; v < NW; ++v) all += squares[v];
+    const float inv = 1.0f / sqrtf(all / (float)a.gate_n + a.gate_eps);
+    for (int j = tid * 4; j < a.gate_k; j += NT * 4) {
+      bf16x4_t y = {(bf16_t)0.0f, (bf16_t)0.0f, (bf16_t)0.0f, (bf16_t)0.0f};
+      if (j < a.gate_n) {
+        const f32x4_t o = *reinterpret_cast<const f32x4_t*>(a.gate_o + j), gw = *reinterpret_cast<const f32x4_t*>(a.gate_w + j);
+        const bf16x4_t g = *reinterpret_cast<const bf16x4_t*>(gate + j);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) y[e] = (bf16_t)(o[e] * inv * gw[e] * sigmoid_exact((float)g[e]));
+      }
+      *reinterpret_cast<bf16x4_t*>(gated + j) = y;
+    }
+    __syncthreads();
+  }
+  for (; i + U <= s1; i += U) {
+    if (i != s0) weights(i);
+#pragma unroll
+    for (int u = 0; u < U; ++u) xv[u] = input(i + u);
 #pragma unroll
     for (int u = 0; u < U; ++u) acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wv[u], xv[u], acc, 0, 0, 0);
   }
   for (; i < s1; ++i)
-    acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_nontemporal_load(w + (int64_t)i * 128), x[i * 4], acc, 0, 0, 0);
+    acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_nontemporal_load(w + (int64_t)i * 128), input(i), acc, 0, 0, 0);
   if (r == 0) {
 #pragma unroll
     for (int j = 0; j < 4; ++j) part[wave][4 * c + j] = acc[j];
@@ -345,12 +386,21 @@ template <int OUT>
 int launch_one(const DenseArgs& a, bool f32, int64_t rows, hipStream_t st) {
   if (f32) {
     hipLaunchKernelGGL(dense_one_f32_kernel<OUT>, dim3((unsigned)(rows / 4)), dim3(256), 0, st, a);
-  } else if (a.k > 8192) {
-    hipLaunchKernelGGL((dense_one_kernel<16, OUT>), dim3((unsigned)(rows / 16)), dim3(1024), 0, st, a);
-  } else if (a.k > 1024) {
-    hipLaunchKernelGGL((dense_one_kernel<8, OUT>), dim3((unsigned)(rows / 16)), dim3(512), 0, st, a);
   } else {
-    hipLaunchKernelGGL((dense_one_kernel<4, OUT>), dim3((unsigned)(rows / 16)), dim3(256), 0, st, a);
+    const dim3 g((unsigned)(rows / 16));
+    if constexpr (OUT == DENSE_RESIDUAL) {
+      if (a.gate_o) {
+        const size_t lds = (size_t)a.gate_k * 2;
+        if (a.k > 8192) hipLaunchKernelGGL((dense_one_kernel<16, OUT, true>), g, dim3(1024), lds, st, a);
+        else if (a.k > 1024) hipLaunchKernelGGL((dense_one_kernel<8, OUT, true>), g, dim3(512), lds, st, a);
+        else hipLaunchKernelGGL((dense_one_kernel<4, OUT, true>), g, dim3(256), lds, st, a);
+        AWQ_HIP_TRY(hipGetLastError());
+        return AWQ_OK;
+      }
+    }
+    if (a.k > 8192) hipLaunchKernelGGL((dense_one_kernel<16, OUT, false>), g, dim3(1024), 0, st, a);
+    else if (a.k > 1024) hipLaunchKernelGGL((dense_one_kernel<8, OUT, false>), g, dim3(512), 0, st, a);
+    else hipLaunchKernelGGL((dense_one_kernel<4, OUT, false>), g, dim3(256), 0, st, a);
   }
   AWQ_HIP_TRY(hipGetLastError());
   return AWQ_OK;
@@ -393,6 +443,10 @@ int launch_many(const DenseArgs& a, bool f32, int64_t rows, hipStream_t st) {
 
 }  // namespace
 
+bool dense_gate_fused(int64_t n, int64_t k_padded, int64_t M, bool f32) {
+  return !f32 && M == 1 && n % 4 == 0 && n > 0 && n <= k_padded && k_padded % kDenseKAlign == 0 && k_padded <= 16384;
+}
+
 int64_t dense_weight_bytes(int64_t rows_padded, int64_t k_padded, bool f32) { return rows_padded * k_padded * (f32 ? 4 : 2); }
 
 int launch_dense_pack(const void* src, bool src_f32, int64_t rows, int64_t cols, void* w, int64_t k_padded, int64_t row0,
@@ -416,6 +470,9 @@ int launch_dense(const DenseArgs& a, bool f32, hipStream_t st) {
     AWQ_REQUIRE(a.seg[i].x && a.seg[i].y && a.seg[i].rows > 0 && a.seg[i].row0 % kDenseRowAlign == 0 && a.seg[i].ldx % 8 == 0,
                 "bad segment");
   AWQ_REQUIRE(a.n_seg == 1 || a.seg[1].row0 >= a.seg[0].row0 + a.seg[0].rows, "segments overlap");
+  AWQ_REQUIRE(!a.gate_o || (a.out == DENSE_RESIDUAL && a.n_seg == 1 && dense_gate_fused(a.gate_n, a.gate_k, a.M, f32) && a.gate_g &&
+                            a.gate_w && a.gate_k <= a.k),
+              "the gated norm cannot be part of this product");
   const DenseSegment& last = a.seg[a.n_seg - 1];
   const int64_t rows = round_up(last.row0 + last.rows, kDenseRowAlign);
   AWQ_REQUIRE(rows < (1ll << 30) && a.M < (1ll << 30), "too large");

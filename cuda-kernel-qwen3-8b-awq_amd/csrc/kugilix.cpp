@@ -4,7 +4,7 @@
 // and constant; the order of the layers is data.  Runs in bfloat16 (residual, norms, scores and recurrent state in
 // binary32) or wholly in binary32, behind the step driver of engine.cpp.
 //
-// A layer is four launches (five with linear attention):
+// A layer is four launches (five in a pass with linear attention, and with attention over more than 64 keys):
 //   norms + convolution     x -> h = conv(norm1(x)) and n = norm2(x)
 //   one product             q, k, v (and the gate) of h, and act(W_up n): two segments of one weight block
 //   the mixer               -> ctx
@@ -543,6 +543,8 @@ int KugilixEngine::run_layers(Buffers& b, int64_t M, PassPos pos) {
       }
       if (int rc = launch_dense(a, f32, stream)) return rc;
     }
+    const char* gate = nullptr;
+    bool gate_fused = false;
     if (s.type == MIX_ATTENTION) {
       WindowAttnArgs a;
       a.proj = b.proj;
@@ -582,9 +584,12 @@ int KugilixEngine::run_layers(Buffers& b, int64_t M, PassPos pos) {
       a.M = M;
       a.pos = pos;
       if (int rc = launch_linear_attention(a, f32, stream)) return rc;
-      const char* gate = (const char*)b.proj + (int64_t)s.heads * (2 * s.dim + s.vdim) * unit();
-      if (int rc = launch_gated_norm(b.o, s.mixed(), gate, L.ldp, L.mix_norm, cat, L.k_out, s.mixed(), M, spec.eps, f32, stream))
-        return rc;
+      gate = (const char*)b.proj + (int64_t)s.heads * (2 * s.dim + s.vdim) * unit();
+      // a single token's gated norm is part of the product below
+      gate_fused = dense_gate_fused(s.mixed(), L.mixed_k, M, f32) && ((uintptr_t)gate & 7) == 0;
+      if (!gate_fused)
+        if (int rc = launch_gated_norm(b.o, s.mixed(), gate, L.ldp, L.mix_norm, cat, L.k_out, s.mixed(), M, spec.eps, f32, stream))
+          return rc;
     }
     {
       DenseArgs a;
@@ -599,6 +604,14 @@ int KugilixEngine::run_layers(Buffers& b, int64_t M, PassPos pos) {
       a.seg[0].y = b.x;
       a.seg[0].ldy = W;
       a.seg[0].rows = (int32_t)W;
+      if (gate_fused) {
+        a.gate_o = b.o;
+        a.gate_g = gate;
+        a.gate_w = L.mix_norm;
+        a.gate_n = s.mixed();
+        a.gate_k = (int32_t)L.mixed_k;
+        a.gate_eps = spec.eps;
+      }
       // the tap sees the stream as the layer leaves it
       if (r.add_embedding && !tap_on) a.addend = b.keep;
       if (int rc = launch_dense(a, f32, stream)) return rc;

@@ -63,6 +63,13 @@ struct DenseArgs {
   DenseSegment seg[2];
   const float* addend = nullptr;
   unsigned long long* best = nullptr;  // DENSE_ARGMAX: zero between launches
+  // one token, DENSE_RESIDUAL: the first gate_k inputs of segment 0 are not read from x but formed in the launch, the RMS
+  // norm of o over gate_n values times w times sigmoid(g), zeros behind them (dense_gate_fused says where it can be)
+  const float* gate_o = nullptr;
+  const void* gate_g = nullptr;
+  const float* gate_w = nullptr;
+  int32_t gate_n = 0, gate_k = 0;
+  float gate_eps = 0.0f;
   float* workspace = nullptr;          // sums of products that are cut along k; may be null
   int64_t workspace_floats = 0;
 };
@@ -72,6 +79,7 @@ int64_t dense_weight_bytes(int64_t rows_padded, int64_t k_padded, bool f32);
 int launch_dense_pack(const void* src, bool src_f32, int64_t rows, int64_t cols, void* w, int64_t k_padded, int64_t row0,
                       int64_t col0, bool f32, hipStream_t st);
 int launch_dense(const DenseArgs& a, bool f32, hipStream_t st);
+bool dense_gate_fused(int64_t n, int64_t k_padded, int64_t M, bool f32);
 
 // --- per-token operators (token_ops.hip) -------------------------------------------------------------------
 // src [n] -> dst [n], each bfloat16 or float

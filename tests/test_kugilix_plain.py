@@ -3,6 +3,7 @@ GPU."""
 import ctypes
 import json
 import os
+import subprocess
 
 import numpy as np
 import pytest
@@ -148,3 +149,18 @@ def test_folders_are_checked_before_the_gpu(awq, lib, tmp_path):
     assert open_rc(awq, lib, tmp_path)[0] == 1
     (tmp_path / "config.json").unlink()   # without one it is a raw weight directory, and an empty one
     assert "could not open" in open_rc(awq, lib, tmp_path)[1]
+
+
+def test_trace_runner_refuses_what_it_cannot_do(tmp_path):
+    root = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
+    runner = os.path.join(root, "bin", "trace_run")
+
+    def rc(*args):
+        run = subprocess.run([runner, *args], input="", capture_output=True, text=True, timeout=60)
+        assert run.stderr
+        return run.returncode
+
+    assert rc("--model", str(tmp_path)) == 1                                         # no --out
+    assert rc("--model", str(tmp_path), "--out", str(tmp_path), "--dtype", "int8") == 1
+    assert rc("--model", str(tmp_path), "--out", str(tmp_path), "--speed", "1") == 1
+    assert rc("--model", str(tmp_path / "none"), "--out", str(tmp_path)) == 1
