@@ -3,7 +3,7 @@
 //   trace_run --model DIR --dtype bfloat16|float32 --out DIR --max-tokens N
 //
 // Steps come from standard input, one JSON object a line:
-//   {"step": 0, "entries": [{"id": "a", "tokens": [5, 17, 3], "want": [0, 2]}], "end": []}
+//   {"step": 4, "entries": [{"id": "x7", "tokens": [12, 8], "want": [1]}], "end": ["x7"]}
 // A step's entry brings the next tokens of a request; a request that was not running starts a new sequence, and
 // requests come one after the other.  A step in which something is wanted writes DIR/<step>.f32, [wanted][vocab]
 // little-endian binary32; every step prints "done <step>".
