@@ -23,7 +23,9 @@ TRACE = os.path.join(HERE, "trace_run")
 # the step driver with the model registry and the operators every model uses
 CORE_SOURCES = ["engine.cpp", "checkpoint.cpp", "ops.hip"]
 # models described by a config.json
-CONFIG_MODEL_SOURCES = ["kugilix.cpp", "dense.hip", "token_ops.hip", "window_attention.hip", "linear_attention.hip"]
+CONFIG_MODEL_SOURCES = ["config_model.cpp", "kugilix.cpp", "tudasun.cpp", "dense.hip", "token_ops.hip", "sublayer_ops.hip",
+                        "window_attention.hip", "linear_attention.hip", "latent_attention.hip", "gated_state.hip",
+                        "experts.hip"]
 # the int4 model of the raw weight directory and the entry points for single kernels
 INT4_SOURCES = ["gemv.hip", "gemm.hip", "prefill.hip", "attention.hip", "fused.hip", "qkv_attn.hip", "qwen3.cpp",
                 "kernel_api.cpp", "layer_api.cpp", "synth.cpp"]

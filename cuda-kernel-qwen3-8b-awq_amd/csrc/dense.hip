@@ -31,7 +31,27 @@ __device__ __forceinline__ float activate(const DenseSegment& s, int row, float 
     const float h = 0.5f * z;
     return z > 0.0f ? __builtin_fmaf(s.act_pos * z, z, h) : __builtin_fmaf(s.act_neg, exp_minus_1_minus(z), h);
   }
+  if (s.act == DENSE_SIGMOID) {
+    z += s.bias[row];
+    return F32 ? sigmoid_exact(z) : sigmoid_f32(z);
+  }
+  if (s.act == DENSE_GELU) {  // (1 + tanh u) / 2 = sigmoid(2 u)
+    const float u2 = 1.5957691216057307117f * __builtin_fmaf(0.044715f * z * z, z, z);
+    return z * (F32 ? sigmoid_exact(u2) : sigmoid_f32(u2));
+  }
+  if (s.act == DENSE_LOG_DECAY) {
+    z += s.bias[row];
+    return -s.act_pos * (log1pf(expf(-fabsf(z))) + fmaxf(-z, 0.0f));
+  }
+  if (s.act == DENSE_FORGET) return (1.0f - s.lower[row]) * sigmoid_exact(-(z + s.bias[row]));
   return z;
+}
+
+__device__ __forceinline__ float softcap(const DenseSegment& s, float z) { return s.act_pos * tanhf(z / s.act_pos); }
+
+template <bool F32>
+__device__ __forceinline__ float glu(float gate, float up) {
+  return gate * (F32 ? sigmoid_exact(gate) : sigmoid_f32(gate)) * up;
 }
 
 __device__ __forceinline__ int32_t f32_key(float v) {
@@ -42,22 +62,34 @@ __device__ __forceinline__ int32_t f32_key(float v) {
 }
 
 __device__ __forceinline__ const DenseSegment& segment_of(const DenseArgs& a, int row) {
-  return a.n_seg > 1 && row >= a.seg[1].row0 ? a.seg[1] : a.seg[0];
+  int i = 0;
+#pragma unroll
+  for (int j = 1; j < kDenseSegments; ++j) i += j < a.n_seg && row >= a.start[j] ? 1 : 0;
+  return a.seg[i];
+}
+
+// one output of one token (DENSE_STORE), `y0` elements into the segment's output
+template <typename T>
+__device__ __forceinline__ void store_one(const DenseSegment& s, int64_t y0, int64_t t, int row, float v) {
+  if (s.act == DENSE_GELU && s.mul) v *= (float)reinterpret_cast<const T*>(s.mul)[t * s.ldmul + row];
+  const int64_t at = y0 + t * s.ldy + row;
+  if (s.y_f32) reinterpret_cast<float*>(s.y)[at] = v;
+  else reinterpret_cast<T*>(s.y)[at] = (T)v;
 }
 
 // one finished sum of one token
 template <typename T, int OUT>
-__device__ __forceinline__ void finish_one(const DenseArgs& a, const DenseSegment& s, int64_t t, int row, float sum) {
-  const int64_t at = t * s.ldy + row;
+__device__ __forceinline__ void finish_one(const DenseArgs& a, const DenseSegment& s, int64_t t, int row, float sum, int64_t y0 = 0) {
   if constexpr (OUT == DENSE_STORE) {
-    reinterpret_cast<T*>(s.y)[at] = (T)activate<sizeof(T) == 4>(s, row, sum);
+    store_one<T>(s, y0, t, row, activate<sizeof(T) == 4>(s, row, sum));
   } else if constexpr (OUT == DENSE_RESIDUAL) {
+    const int64_t at = t * s.ldy + row;
     float* y = reinterpret_cast<float*>(s.y);
     float v = y[at] + sum;
     if (a.addend) v += a.addend[at];
     y[at] = v;
   } else {
-    reinterpret_cast<float*>(s.y)[at] = sum;
+    reinterpret_cast<float*>(s.y)[t * s.ldy + row] = s.act == DENSE_SOFTCAP ? softcap(s, sum) : sum;
   }
 }
 
@@ -77,14 +109,19 @@ __global__ __launch_bounds__(NW * 64) void dense_one_kernel(DenseArgs a) {
   const DenseSegment& s = segment_of(a, row0);
   const int local = row0 - s.row0;
   if (local >= s.rows) return;  // padding
+  int group = blockIdx.y;
+  if (a.ids) {
+    group = a.ids[blockIdx.y];
+    if (group >= a.n_groups) return;
+  }
   const int steps = (int)(a.k >> 5);  // even: k is a multiple of 64
   const int per = (steps + NW - 1) / NW;
   const int s0 = min(wave * per, steps), s1 = min(s0 + per, steps);
   const int r = lane & 15, c = lane >> 4;
   // piece of (row, 8-wide chunk c of step i): block (row / 32, 2 i + c / 2), lane 32 (c % 2) + row % 32
-  const bf16x8_t* w = reinterpret_cast<const bf16x8_t*>(a.w) + ((int64_t)(row0 >> 5) * (a.k >> 4) + (c >> 1)) * 64 +
-                      32 * (c & 1) + (row0 & 16) + r;
-  const bf16x8_t* x = reinterpret_cast<const bf16x8_t*>(s.x) + c;
+  const bf16x8_t* w = reinterpret_cast<const bf16x8_t*>(reinterpret_cast<const bf16_t*>(a.w) + group * a.w_batch) +
+                      ((int64_t)(row0 >> 5) * (a.k >> 4) + (c >> 1)) * 64 + 32 * (c & 1) + (row0 & 16) + r;
+  const bf16x8_t* x = reinterpret_cast<const bf16x8_t*>(reinterpret_cast<const bf16_t*>(s.x) + blockIdx.y * a.x_batch) + c;
   f32x4_t acc = {0.0f, 0.0f, 0.0f, 0.0f};
   constexpr int U = 8;
   bf16x8_t wv[U], xv[U];
@@ -146,8 +183,17 @@ __global__ __launch_bounds__(NW * 64) void dense_one_kernel(DenseArgs a) {
 #pragma unroll
   for (int v = 0; v < NW; ++v) sum += part[v][tid];
   const int row = local + tid;
-  if (row < s.rows) finish_one<bf16_t, OUT>(a, s, 0, row, sum);
+  const int64_t y0 = blockIdx.y * a.y_batch;
+  if constexpr (OUT == DENSE_STORE) {
+    if (s.act == DENSE_GLU) {
+      const float up = __shfl_down(sum, 8, 16);
+      if (tid < 8 && local / 2 + tid < s.glu_rows) store_one<bf16_t>(s, y0, 0, local / 2 + tid, glu<false>(sum, up));
+      return;
+    }
+  }
+  if (row < s.rows) finish_one<bf16_t, OUT>(a, s, 0, row, sum, y0);
   if constexpr (OUT == DENSE_ARGMAX) {
+    if (s.act == DENSE_SOFTCAP) sum = softcap(s, sum);
     unsigned long long b = row < s.rows ? awq_pack_candidate(f32_key(sum), (uint32_t)row) : 0ull;
 #pragma unroll
     for (int off = 8; off > 0; off >>= 1) {
@@ -166,7 +212,8 @@ __global__ __launch_bounds__(NW * 64) void dense_one_kernel(DenseArgs a) {
 // fill the device, k is cut over `cuts` workgroups whose sums go to the workspace, [cut][token][row]; a second launch
 // adds them in order.
 constexpr int DENSE_PART = 100;
-template <int TT, int OUT>
+// LISTED: the tokens come from runs of a list, each with a weight block of its own.
+template <int TT, int OUT, bool LISTED = false>
 __global__ __launch_bounds__(256, 2) void dense_many_kernel(DenseArgs a, int row_tiles, int tok_tiles, int cuts) {
   __shared__ __attribute__((aligned(16))) bf16_t tile0[32 * TT * 64];
   __shared__ __attribute__((aligned(16))) bf16_t tile1[32 * TT * 64];
@@ -175,8 +222,18 @@ __global__ __launch_bounds__(256, 2) void dense_many_kernel(DenseArgs a, int row
   const int per = (total + 7) >> 3;
   const int work = (blockIdx.x & 7) * per + (blockIdx.x >> 3);
   if (work >= total) return;
-  const int rc = work / tok_tiles, tt0 = (work - rc * tok_tiles) * 32 * TT;
+  const int rc = work / tok_tiles, tile = work - rc * tok_tiles, tt0 = LISTED ? 0 : tile * 32 * TT;
   const int rt = rc / cuts, cut = rc - rt * cuts;
+  int64_t group = blockIdx.y;
+  int n_tok = (int)min((int64_t)1 << 30, a.M);
+  const int32_t* list = nullptr;
+  if constexpr (LISTED) {
+    const DenseTile run = a.tiles[tile];
+    if (run.count == 0) return;
+    group = run.group;
+    n_tok = run.count;
+    list = a.list + run.first;
+  }
   const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
   const int n = lane & 31, kh = lane >> 5;
   const DenseSegment& s = segment_of(a, rt * 256);
@@ -190,15 +247,18 @@ __global__ __launch_bounds__(256, 2) void dense_many_kernel(DenseArgs a, int row
 #pragma unroll
   for (int i = 0; i < TT; ++i) {
     const int row = (wave * TT + i) * 8 + (lane >> 3);
-    const int64_t tok = min((int64_t)tt0 + row, a.M - 1);
-    src[i] = reinterpret_cast<const bf16_t*>(s.x) + tok * s.ldx + first_step * 64 + (((lane & 7) ^ (row & 7)) << 3);
+    int64_t tok = min(tt0 + row, n_tok - 1);
+    if constexpr (LISTED) tok = list[tok] / a.list_div;
+    src[i] = reinterpret_cast<const bf16_t*>(s.x) + blockIdx.y * a.x_batch + tok * s.ldx + first_step * 64 +
+             (((lane & 7) ^ (row & 7)) << 3);
   }
   auto request = [&](bf16_t* tile, int step) __attribute__((always_inline)) {
 #pragma unroll
     for (int i = 0; i < TT; ++i)
       __builtin_amdgcn_global_load_lds((gptr_t)(src[i] + step * 64), (lptr_t)(tile + (wave * TT + i) * 8 * 64), 16, 0, 0);
   };
-  const bf16x8_t* wp = reinterpret_cast<const bf16x8_t*>(a.w) + ((int64_t)(rt * 8 + wave * 2) * k16 + first_step * 4) * 64 + lane;
+  const bf16x8_t* wp = reinterpret_cast<const bf16x8_t*>(reinterpret_cast<const bf16_t*>(a.w) + group * a.w_batch) +
+                       ((int64_t)(rt * 8 + wave * 2) * k16 + first_step * 4) * 64 + lane;
   auto weights = [&](bf16x8_t (&wv)[2][4], int step) __attribute__((always_inline)) {
 #pragma unroll
     for (int b = 0; b < 2; ++b)
@@ -245,47 +305,80 @@ __global__ __launch_bounds__(256, 2) void dense_many_kernel(DenseArgs a, int row
     }
   }
   // acc[b][t][i]: row 32 b + 8 (i / 4) + 4 kh + i % 4 of the wavefront's 64, token 32 t + n
+  const int row_w = rt * 256 + wave * 64;
+  if constexpr (OUT == DENSE_STORE) {
 #pragma unroll
-  for (int t = 0; t < TT; ++t) {
-    const int64_t tok = (int64_t)tt0 + 32 * t + n;
-    if (tok >= a.M) continue;
+    for (int b = 0; b < 2; ++b) {
+      const DenseSegment& out = segment_of(a, row_w + 32 * b);
+      const int local_b = row_w + 32 * b - out.row0 + 4 * kh;
 #pragma unroll
-    for (int b = 0; b < 2; ++b)
+      for (int t = 0; t < TT; ++t) {
+        if (out.act == DENSE_GLU) {
+#pragma unroll
+          for (int i = 0; i < 16; ++i)
+            if ((i & 4) == 0) acc[b][t][i] = glu<false>(acc[b][t][i], acc[b][t][i + 4]);
+        } else if (out.act != DENSE_NONE) {
+#pragma unroll
+          for (int i = 0; i < 16; ++i) {
+            const int row = local_b + 8 * (i >> 2) + (i & 3);
+            if (row < out.rows) acc[b][t][i] = activate<false>(out, row, acc[b][t][i]);
+          }
+        }
+      }
+    }
+  }
+  const int64_t y0 = blockIdx.y * a.y_batch;
+#pragma unroll
+  for (int b = 0; b < 2; ++b) {
+    const DenseSegment& out = segment_of(a, row_w + 32 * b);
+    const int local_b = row_w + 32 * b - out.row0;
+    const bool gated = OUT == DENSE_STORE && out.act == DENSE_GLU;
+    const int n_rows = gated ? out.glu_rows : out.rows;
+    if (OUT != DENSE_PART && local_b >= out.rows) continue;  // padding
+    const bool by_four = ((out.ldy | a.y_batch) & 3) == 0 && !(OUT == DENSE_STORE && out.mul);
+#pragma unroll
+    for (int t = 0; t < TT; ++t) {
+      int64_t tok = tt0 + 32 * t + n;
+      if (tok >= n_tok) continue;
+      if constexpr (LISTED) tok = list[tok];
 #pragma unroll
       for (int g = 0; g < 4; ++g) {
+        if (gated && (g & 1)) continue;
+        f32x4_t v;
+#pragma unroll
+        for (int j = 0; j < 4; ++j) v[j] = acc[b][t][4 * g + j];
         if constexpr (OUT == DENSE_PART) {
-          f32x4_t v;
+          *reinterpret_cast<f32x4_t*>(a.workspace + ((int64_t)cut * a.M + tok) * row_tiles * 256 + row_w + 32 * b + 8 * g + 4 * kh) = v;
+        } else {
+          const int row = gated ? local_b / 2 + 4 * g + 4 * kh : local_b + 8 * g + 4 * kh;
+          const int64_t at = y0 + tok * out.ldy + row;
+          if (row + 3 < n_rows && by_four) {
+            if (OUT == DENSE_STORE && !out.y_f32) {
+              *reinterpret_cast<bf16x4_t*>(reinterpret_cast<bf16_t*>(out.y) + at) =
+                  bf16x4_t{(bf16_t)v[0], (bf16_t)v[1], (bf16_t)v[2], (bf16_t)v[3]};
+              continue;
+            }
+            if (OUT == DENSE_F32 && out.act == DENSE_SOFTCAP) {
 #pragma unroll
-          for (int j = 0; j < 4; ++j) v[j] = acc[b][t][4 * g + j];
-          *reinterpret_cast<f32x4_t*>(a.workspace + ((int64_t)cut * a.M + tok) * row_tiles * 256 + rt * 256 + wave * 64 + 32 * b +
-                                      8 * g + 4 * kh) = v;
-          continue;
-        }
-        const int row = rt * 256 + wave * 64 + 32 * b + 8 * g + 4 * kh - s.row0;
-        const int64_t at = tok * s.ldy + row;
-        if (row + 3 < s.rows && (s.ldy & 3) == 0) {
-          if constexpr (OUT == DENSE_STORE) {
-            bf16x4_t v;
-#pragma unroll
-            for (int j = 0; j < 4; ++j) v[j] = (bf16_t)activate<false>(s, row + j, acc[b][t][4 * g + j]);
-            *reinterpret_cast<bf16x4_t*>(reinterpret_cast<bf16_t*>(s.y) + at) = v;
-          } else {
-            f32x4_t v;
-#pragma unroll
-            for (int j = 0; j < 4; ++j) v[j] = acc[b][t][4 * g + j];
-            f32x4_t* y = reinterpret_cast<f32x4_t*>(reinterpret_cast<float*>(s.y) + at);
+              for (int j = 0; j < 4; ++j) v[j] = softcap(out, v[j]);
+            }
+            f32x4_t* y = reinterpret_cast<f32x4_t*>(reinterpret_cast<float*>(out.y) + at);
             if constexpr (OUT == DENSE_RESIDUAL) {
               v = *y + v;
               if (a.addend) v = v + *reinterpret_cast<const f32x4_t*>(a.addend + at);
             }
             *y = v;
-          }
-        } else {
+          } else {
 #pragma unroll
-          for (int j = 0; j < 4; ++j)
-            if (row + j < s.rows) finish_one<bf16_t, OUT>(a, s, tok, row + j, acc[b][t][4 * g + j]);
+            for (int j = 0; j < 4; ++j) {
+              if (row + j >= n_rows) continue;
+              if constexpr (OUT == DENSE_STORE) store_one<bf16_t>(out, y0, tok, row + j, v[j]);
+              else finish_one<bf16_t, OUT>(a, out, tok, row + j, v[j]);
+            }
+          }
         }
       }
+    }
   }
 }
 
@@ -302,6 +395,18 @@ __global__ __launch_bounds__(256) void dense_parts_kernel(DenseArgs a, int rows,
   const int64_t stride = a.M * rows / 4;
   f32x4_t sum = p[0];
   for (int c = 1; c < cuts; ++c) sum = sum + p[c * stride];
+  if constexpr (OUT == DENSE_STORE) {
+    if (s.act == DENSE_GLU) {
+      if (local & 8) return;
+      f32x4_t up = p[2];
+      for (int c = 1; c < cuts; ++c) up = up + p[c * stride + 2];
+      const int r0 = (local >> 4) * 8 + (local & 7);
+#pragma unroll
+      for (int j = 0; j < 4; ++j)
+        if (r0 + j < s.glu_rows) store_one<bf16_t>(s, 0, tok, r0 + j, glu<false>(sum[j], up[j]));
+      return;
+    }
+  }
 #pragma unroll
   for (int j = 0; j < 4; ++j)
     if (local + j < s.rows) finish_one<bf16_t, OUT>(a, s, tok, local + j, sum[j]);
@@ -316,37 +421,77 @@ __global__ __launch_bounds__(256) void dense_one_f32_kernel(DenseArgs a) {
   const DenseSegment& s = segment_of(a, row);
   const int local = row - s.row0;
   if (local >= s.rows) return;
-  const f32x4_t* w = reinterpret_cast<const f32x4_t*>(reinterpret_cast<const float*>(a.w) + (int64_t)row * a.k);
-  const f32x4_t* x = reinterpret_cast<const f32x4_t*>(s.x);
-  float acc = 0.0f;
-  for (int i = lane; i < (int)(a.k >> 2); i += 64) {
-    const f32x4_t wv = w[i], xv = x[i];
-#pragma unroll
-    for (int j = 0; j < 4; ++j) acc = __builtin_fmaf(wv[j], xv[j], acc);
+  int group = blockIdx.y;
+  if (a.ids) {
+    group = a.ids[blockIdx.y];
+    if (group >= a.n_groups) return;
   }
+  const float* x = reinterpret_cast<const float*>(s.x) + blockIdx.y * a.x_batch;
+  auto product = [&](int r) {
+    const f32x4_t* w = reinterpret_cast<const f32x4_t*>(reinterpret_cast<const float*>(a.w) + group * a.w_batch + (int64_t)r * a.k);
+    float acc = 0.0f;
+    for (int i = lane; i < (int)(a.k >> 2); i += 64) {
+      const f32x4_t wv = w[i];
 #pragma unroll
-  for (int off = 32; off > 0; off >>= 1) acc += __shfl_xor(acc, off, 64);
+      for (int j = 0; j < 4; ++j) acc = __builtin_fmaf(wv[j], x[4 * i + j], acc);
+    }
+#pragma unroll
+    for (int off = 32; off > 0; off >>= 1) acc += __shfl_xor(acc, off, 64);
+    return acc;
+  };
+  const int64_t y0 = blockIdx.y * a.y_batch;
+  if constexpr (OUT == DENSE_STORE) {
+    if (s.act == DENSE_GLU) {
+      const int r = (local >> 4) * 8 + (local & 7);
+      if ((local & 8) || r >= s.glu_rows) return;
+      const float gate = product(row), up = product(row + 8);
+      if (lane == 0) store_one<float>(s, y0, 0, r, glu<true>(gate, up));
+      return;
+    }
+  }
+  float acc = product(row);
   if (lane != 0) return;
-  finish_one<float, OUT>(a, s, 0, local, acc);
-  if constexpr (OUT == DENSE_ARGMAX) atomicMax(a.best, awq_pack_candidate(f32_key(acc), (uint32_t)local));
+  finish_one<float, OUT>(a, s, 0, local, acc, y0);
+  if constexpr (OUT == DENSE_ARGMAX) {
+    if (s.act == DENSE_SOFTCAP) acc = softcap(s, acc);
+    atomicMax(a.best, awq_pack_candidate(f32_key(acc), (uint32_t)local));
+  }
 }
 
-// 64 rows x 64 tokens per workgroup, 4 x 4 per thread, through LDS
-template <int OUT>
+// 64 rows x 64 tokens per workgroup, 4 x 4 per thread, through LDS.  A thread's rows are two of an eight and the same two of
+// the eight behind it: a gate and its up row meet.
+template <int OUT, bool LISTED = false>
 __global__ __launch_bounds__(256) void dense_many_f32_kernel(DenseArgs a) {
   __shared__ float ws[16][68], xs[16][68];
   const int tid = threadIdx.x;
   const int row0 = blockIdx.x * 64;
-  const int64_t tok0 = (int64_t)blockIdx.y * 64;
+  const int64_t tok0 = LISTED ? 0 : (int64_t)blockIdx.y * 64;
   const DenseSegment& s = segment_of(a, row0);
-  if (row0 - s.row0 >= s.rows) return;
+  if (row0 >= a.seg[a.n_seg - 1].row0 + a.seg[a.n_seg - 1].rows) return;
+  int64_t group = blockIdx.z, n_tok = a.M;
+  const int32_t* list = nullptr;
+  if constexpr (LISTED) {
+    const DenseTile run = a.tiles[blockIdx.y];
+    if (run.count == 0) return;
+    group = run.group;
+    n_tok = run.count;
+    list = a.list + run.first;
+  }
   const int lr = tid >> 2, lk = (tid & 3) * 4;
-  const float* w = reinterpret_cast<const float*>(a.w) + (int64_t)(row0 + lr) * a.k + lk;
-  const float* x = reinterpret_cast<const float*>(s.x) + min(tok0 + lr, a.M - 1) * s.ldx + lk;
-  const int tr = (tid & 15) * 4, tc = (tid >> 4) * 4;
+  const float* w = reinterpret_cast<const float*>(a.w) + group * a.w_batch + (int64_t)(row0 + lr) * a.k + lk;
+  int64_t tok = min(tok0 + lr, n_tok - 1);
+  if constexpr (LISTED) tok = list[tok] / a.list_div;
+  const float* x = reinterpret_cast<const float*>(s.x) + blockIdx.z * a.x_batch + tok * s.ldx + lk;
+  const int tc = (tid >> 4) * 4;
+  int tr[4];
+#pragma unroll
+  for (int i = 0; i < 4; ++i) tr[i] = 16 * ((tid & 15) >> 2) + 2 * (tid & 3) + (i & 1) + 8 * (i >> 1);
   float acc[4][4] = {};
   for (int k0 = 0; k0 < (int)a.k; k0 += 16) {
-    const f32x4_t wv = *reinterpret_cast<const f32x4_t*>(w + k0), xv = *reinterpret_cast<const f32x4_t*>(x + k0);
+    const f32x4_t wv = *reinterpret_cast<const f32x4_t*>(w + k0);
+    f32x4_t xv;
+#pragma unroll
+    for (int j = 0; j < 4; ++j) xv[j] = x[k0 + j];
     __syncthreads();
 #pragma unroll
     for (int j = 0; j < 4; ++j) ws[lk + j][lr] = wv[j], xs[lk + j][lr] = xv[j];
@@ -356,24 +501,46 @@ __global__ __launch_bounds__(256) void dense_many_f32_kernel(DenseArgs a) {
 #pragma unroll
       for (int i = 0; i < 4; ++i)
 #pragma unroll
-        for (int j = 0; j < 4; ++j) acc[i][j] = __builtin_fmaf(ws[k][tr + i], xs[k][tc + j], acc[i][j]);
+        for (int j = 0; j < 4; ++j) acc[i][j] = __builtin_fmaf(ws[k][tr[i]], xs[k][tc + j], acc[i][j]);
   }
+  const int64_t y0 = blockIdx.z * a.y_batch;
 #pragma unroll
-  for (int j = 0; j < 4; ++j)
-    if (tok0 + tc + j < a.M)
+  for (int j = 0; j < 4; ++j) {
+    if (tok0 + tc + j >= n_tok) continue;
+    int64_t t = tok0 + tc + j;
+    if constexpr (LISTED) t = list[t];
 #pragma unroll
-      for (int i = 0; i < 4; ++i) {
-        const int row = row0 + tr + i - s.row0;
-        if (row < s.rows) finish_one<float, OUT>(a, s, tok0 + tc + j, row, acc[i][j]);
+    for (int i = 0; i < 4; ++i) {
+      const DenseSegment& out = segment_of(a, row0 + tr[i]);
+      const int row = row0 + tr[i] - out.row0;
+      if (row >= out.rows) continue;
+      if constexpr (OUT == DENSE_STORE) {
+        if (out.act == DENSE_GLU) {
+          const int r = (row >> 4) * 8 + (row & 7);
+          if (i < 2 && r < out.glu_rows) store_one<float>(out, y0, t, r, glu<true>(acc[i][j], acc[i | 2][j]));
+          continue;
+        }
       }
+      finish_one<float, OUT>(a, out, t, row, acc[i][j], y0);
+    }
+  }
 }
 
 template <typename S>
 __global__ __launch_bounds__(256) void dense_pack_kernel(const S* __restrict__ src, int64_t rows, int64_t cols, void* w,
-                                                         int64_t k, int64_t row0, int64_t col0, int f32) {
+                                                         int64_t k, int64_t row0, int64_t col0, int f32, int form) {
   const int64_t n = rows * cols;
   for (int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x; i < n; i += (int64_t)gridDim.x * 256) {
-    const int64_t r = row0 + i / cols, c = col0 + i % cols;
+    int64_t r = i / cols, c = i % cols;
+    if (form == PACK_TRANSPOSED) {
+      const int64_t was = r;
+      r = c;
+      c = was;
+    } else if (form != PACK_PLAIN) {
+      r = (r >> 3) * 16 + (r & 7) + (form == PACK_UP ? 8 : 0);
+    }
+    r += row0;
+    c += col0;
     if (f32)
       reinterpret_cast<float*>(w)[r * k + c] = (float)src[i];
     else
@@ -385,9 +552,9 @@ __global__ __launch_bounds__(256) void dense_pack_kernel(const S* __restrict__ s
 template <int OUT>
 int launch_one(const DenseArgs& a, bool f32, int64_t rows, hipStream_t st) {
   if (f32) {
-    hipLaunchKernelGGL(dense_one_f32_kernel<OUT>, dim3((unsigned)(rows / 4)), dim3(256), 0, st, a);
+    hipLaunchKernelGGL(dense_one_f32_kernel<OUT>, dim3((unsigned)(rows / 4), (unsigned)a.batch), dim3(256), 0, st, a);
   } else {
-    const dim3 g((unsigned)(rows / 16));
+    const dim3 g((unsigned)(rows / 16), (unsigned)a.batch);
     if constexpr (OUT == DENSE_RESIDUAL) {
       if (a.gate_o) {
         const size_t lds = (size_t)a.gate_k * 2;
@@ -409,8 +576,8 @@ int launch_one(const DenseArgs& a, bool f32, int64_t rows, hipStream_t st) {
 template <int OUT>
 int launch_many(const DenseArgs& a, bool f32, int64_t rows, hipStream_t st) {
   if (f32) {
-    hipLaunchKernelGGL(dense_many_f32_kernel<OUT>, dim3((unsigned)(rows / 64), (unsigned)((a.M + 63) / 64)), dim3(256), 0,
-                       st, a);
+    hipLaunchKernelGGL(dense_many_f32_kernel<OUT>, dim3((unsigned)(rows / 64), (unsigned)((a.M + 63) / 64), (unsigned)a.batch),
+                       dim3(256), 0, st, a);
   } else {
     const int row_tiles = (int)(rows / 256);
     const bool wide = a.M > 64;
@@ -418,24 +585,39 @@ int launch_many(const DenseArgs& a, bool f32, int64_t rows, hipStream_t st) {
     const int64_t tiles = row_tiles * tok_tiles;
     // two workgroups per compute unit, at least eight steps each
     int64_t cuts = 1;
-    if (a.workspace && a.M <= 65535 && tiles < 384) {
+    if (a.workspace && a.batch == 1 && a.M <= 65535 && tiles < 384) {
       cuts = std::min<int64_t>((512 + tiles / 2) / tiles, (a.k >> 6) / 8);
       cuts = std::max<int64_t>(1, std::min<int64_t>(cuts, a.workspace_floats / (a.M * rows)));
     }
-    const unsigned grid = (unsigned)((tiles * cuts + 7) / 8 * 8);
+    const dim3 grid((unsigned)((tiles * cuts + 7) / 8 * 8), (unsigned)a.batch);
     if (cuts > 1) {
       if (wide)
-        hipLaunchKernelGGL((dense_many_kernel<4, DENSE_PART>), dim3(grid), dim3(256), 0, st, a, row_tiles, (int)tok_tiles, (int)cuts);
+        hipLaunchKernelGGL((dense_many_kernel<4, DENSE_PART>), grid, dim3(256), 0, st, a, row_tiles, (int)tok_tiles, (int)cuts);
       else
-        hipLaunchKernelGGL((dense_many_kernel<2, DENSE_PART>), dim3(grid), dim3(256), 0, st, a, row_tiles, (int)tok_tiles, (int)cuts);
+        hipLaunchKernelGGL((dense_many_kernel<2, DENSE_PART>), grid, dim3(256), 0, st, a, row_tiles, (int)tok_tiles, (int)cuts);
       AWQ_HIP_TRY(hipGetLastError());
       hipLaunchKernelGGL(dense_parts_kernel<OUT>, dim3((unsigned)((rows / 4 + 255) / 256), (unsigned)a.M), dim3(256), 0, st, a,
                          (int)rows, (int)cuts);
     } else if (wide) {
-      hipLaunchKernelGGL((dense_many_kernel<4, OUT>), dim3(grid), dim3(256), 0, st, a, row_tiles, (int)tok_tiles, 1);
+      hipLaunchKernelGGL((dense_many_kernel<4, OUT>), grid, dim3(256), 0, st, a, row_tiles, (int)tok_tiles, 1);
     } else {
-      hipLaunchKernelGGL((dense_many_kernel<2, OUT>), dim3(grid), dim3(256), 0, st, a, row_tiles, (int)tok_tiles, 1);
+      hipLaunchKernelGGL((dense_many_kernel<2, OUT>), grid, dim3(256), 0, st, a, row_tiles, (int)tok_tiles, 1);
     }
+  }
+  AWQ_HIP_TRY(hipGetLastError());
+  return AWQ_OK;
+}
+
+// tokens with weight blocks of their own
+int launch_listed(const DenseArgs& a, bool f32, int64_t rows, hipStream_t st) {
+  if (f32) {
+    hipLaunchKernelGGL((dense_many_f32_kernel<DENSE_STORE, true>), dim3((unsigned)(rows / 64), (unsigned)a.max_tiles), dim3(256), 0,
+                       st, a);
+  } else {
+    const int row_tiles = (int)(rows / 256);
+    const unsigned grid = (unsigned)(((int64_t)row_tiles * a.max_tiles + 7) / 8 * 8);
+    hipLaunchKernelGGL((dense_many_kernel<kDenseTileTokens / 32, DENSE_STORE, true>), dim3(grid), dim3(256), 0, st, a, row_tiles,
+                       a.max_tiles, 1);
   }
   AWQ_HIP_TRY(hipGetLastError());
   return AWQ_OK;
@@ -450,32 +632,50 @@ bool dense_gate_fused(int64_t n, int64_t k_padded, int64_t M, bool f32) {
 int64_t dense_weight_bytes(int64_t rows_padded, int64_t k_padded, bool f32) { return rows_padded * k_padded * (f32 ? 4 : 2); }
 
 int launch_dense_pack(const void* src, bool src_f32, int64_t rows, int64_t cols, void* w, int64_t k_padded, int64_t row0,
-                      int64_t col0, bool f32, hipStream_t st) {
-  AWQ_REQUIRE(rows > 0 && cols > 0 && k_padded % kDenseKAlign == 0 && col0 % 8 == 0 && col0 + cols <= k_padded, "bad block");
+                      int64_t col0, bool f32, hipStream_t st, int form) {
+  AWQ_REQUIRE(rows > 0 && cols > 0 && k_padded % kDenseKAlign == 0 && col0 % 8 == 0 &&
+                  col0 + (form == PACK_TRANSPOSED ? rows : cols) <= k_padded,
+              "bad block");
   const unsigned grid = (unsigned)std::min<int64_t>((rows * cols + 255) / 256, 65536);
   if (src_f32)
     hipLaunchKernelGGL(dense_pack_kernel<float>, dim3(grid), dim3(256), 0, st, (const float*)src, rows, cols, w, k_padded,
-                       row0, col0, f32 ? 1 : 0);
+                       row0, col0, f32 ? 1 : 0, form);
   else
     hipLaunchKernelGGL(dense_pack_kernel<bf16_t>, dim3(grid), dim3(256), 0, st, (const bf16_t*)src, rows, cols, w, k_padded,
-                       row0, col0, f32 ? 1 : 0);
+                       row0, col0, f32 ? 1 : 0, form);
   AWQ_HIP_TRY(hipGetLastError());
   return AWQ_OK;
 }
 
-int launch_dense(const DenseArgs& a, bool f32, hipStream_t st) {
+int launch_dense(const DenseArgs& args, bool f32, hipStream_t st) {
+  DenseArgs a = args;
   AWQ_REQUIRE(a.w && a.M >= 1 && a.k > 0 && a.k % kDenseKAlign == 0, "bad product");
-  AWQ_REQUIRE(a.n_seg == 1 || a.n_seg == 2, "one or two segments");
-  for (int i = 0; i < a.n_seg; ++i)
-    AWQ_REQUIRE(a.seg[i].x && a.seg[i].y && a.seg[i].rows > 0 && a.seg[i].row0 % kDenseRowAlign == 0 && a.seg[i].ldx % 8 == 0,
+  AWQ_REQUIRE(a.n_seg >= 1 && a.n_seg <= kDenseSegments, "too few or too many segments");
+  for (int i = 0; i < a.n_seg; ++i) {
+    const DenseSegment& s = a.seg[i];
+    const bool shares = i > 0 && s.x == a.seg[i - 1].x;
+    AWQ_REQUIRE(s.x && s.y && s.rows > 0 && s.row0 % (shares ? kDenseSharedAlign : kDenseRowAlign) == 0 && s.ldx % 8 == 0,
                 "bad segment");
-  AWQ_REQUIRE(a.n_seg == 1 || a.seg[1].row0 >= a.seg[0].row0 + a.seg[0].rows, "segments overlap");
+    AWQ_REQUIRE(i == 0 || s.row0 >= a.seg[i - 1].row0 + a.seg[i - 1].rows, "segments overlap");
+    AWQ_REQUIRE(s.act != DENSE_GLU || (a.out == DENSE_STORE && s.glu_rows > 0 && s.rows == dense_glu_rows(s.glu_rows)), "bad gated segment");
+    AWQ_REQUIRE((s.act != DENSE_SIGMOID && s.act != DENSE_LOG_DECAY && s.act != DENSE_FORGET) || s.bias, "a segment lacks its bias");
+    AWQ_REQUIRE(s.act != DENSE_FORGET || s.lower, "a segment lacks its lower bound");
+    a.start[i] = s.row0;
+  }
   AWQ_REQUIRE(!a.gate_o || (a.out == DENSE_RESIDUAL && a.n_seg == 1 && dense_gate_fused(a.gate_n, a.gate_k, a.M, f32) && a.gate_g &&
                             a.gate_w && a.gate_k <= a.k),
               "the gated norm cannot be part of this product");
   const DenseSegment& last = a.seg[a.n_seg - 1];
   const int64_t rows = round_up(last.row0 + last.rows, kDenseRowAlign);
   AWQ_REQUIRE(rows < (1ll << 30) && a.M < (1ll << 30), "too large");
+  AWQ_REQUIRE(a.batch >= 1 && a.batch <= 65535 && (a.batch == 1 || (a.out == DENSE_STORE && a.w_batch % 8 == 0 && a.x_batch % 8 == 0)),
+              "bad batch");
+  AWQ_REQUIRE(!a.ids || (a.M == 1 && a.n_groups >= 0), "weight blocks by number take one token");
+  if (a.tiles) {
+    AWQ_REQUIRE(a.out == DENSE_STORE && a.list && a.list_div >= 1 && a.batch == 1 && a.max_tiles >= 1 && a.max_tiles <= 65535,
+                "bad list of tokens");
+    return launch_listed(a, f32, rows, st);
+  }
   switch (a.out) {
     case DENSE_STORE: return a.M == 1 ? launch_one<DENSE_STORE>(a, f32, rows, st) : launch_many<DENSE_STORE>(a, f32, rows, st);
     case DENSE_RESIDUAL:

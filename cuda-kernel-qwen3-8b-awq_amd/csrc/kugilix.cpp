@@ -9,16 +9,9 @@
 //   one product             q, k, v (and the gate) of h, and act(W_up n): two segments of one weight block
 //   the mixer               -> ctx
 //   one product             x += [W_o | W_down] [ctx, mid], both halves in one block along k
-#include "engine.hpp"
+#include "config_model.hpp"
 
 #include <math.h>
-#include <string.h>
-
-#include <chrono>
-#include <memory>
-
-#include "checkpoint.hpp"
-#include "layers.hpp"
 
 namespace {
 
@@ -43,35 +36,6 @@ struct Spec {
 };
 
 // --- config.json -------------------------------------------------------------------------------------------
-int bad_config(const std::string& why) {
-  awq_set_error("config.json: " + why);
-  return AWQ_ERR_ARG;
-}
-
-int get_number(const Json& j, const std::string& at, const char* key, double* out) {
-  const Json* v = j.find(key);
-  if (!v || !v->is(Json::Number)) return bad_config(at + key + " is missing or no number");
-  *out = v->number;
-  return AWQ_OK;
-}
-int get_int(const Json& j, const std::string& at, const char* key, double lo, double hi, int32_t* out) {
-  double d;
-  if (int rc = get_number(j, at, key, &d)) return rc;
-  if (!(d >= lo && d <= hi) || d != floor(d)) return bad_config(at + key + " is out of range");
-  *out = (int32_t)d;
-  return AWQ_OK;
-}
-int get_float(const Json& j, const std::string& at, const char* key, float* out) {
-  double d;
-  if (int rc = get_number(j, at, key, &d)) return rc;
-  *out = (float)d;
-  return AWQ_OK;
-}
-const Json* section(const Json& j, const char* key) {
-  const Json* v = j.find(key);
-  return v && v->is(Json::Object) ? v : nullptr;
-}
-
 int read_layer(const Json& j, const std::string& at, LayerSpec* s) {
   const Json *type = j.find("type"), *m = section(j, "mixer");
   if (!type || !type->is(Json::String) || !m) return bad_config(at + "type or mixer is missing");
@@ -140,9 +104,9 @@ int read_spec(const std::string& dir, Spec* s) {
 }
 
 // every tensor of the model and its shape
-std::vector<std::pair<std::string, std::vector<int64_t>>> expected_tensors(const Spec& c) {
+TensorTable expected_tensors(const Spec& c) {
   const int64_t W = c.width;
-  std::vector<std::pair<std::string, std::vector<int64_t>>> v = {{"embed", {c.vocab, W}}, {"final.norm", {W}}, {"head", {c.vocab, W}}};
+  TensorTable v = {{"embed", {c.vocab, W}}, {"final.norm", {W}}, {"head", {c.vocab, W}}};
   for (size_t i = 0; i < c.layers.size(); ++i) {
     const LayerSpec& s = c.layers[i];
     const std::string p = "l" + std::to_string(i) + ".", m = p + "mix.";
@@ -165,21 +129,6 @@ std::vector<std::pair<std::string, std::vector<int64_t>>> expected_tensors(const
     }
   }
   return v;
-}
-
-int check_tensors(const Spec& c, const Safetensors& file) {
-  for (const auto& want : expected_tensors(c)) {
-    const Tensor* t = file.find(want.first);
-    if (!t) {
-      awq_set_error("model.safetensors has no tensor " + want.first);
-      return AWQ_ERR_IO;
-    }
-    if (t->shape != want.second || (t->dtype != "BF16" && t->dtype != "F32")) {
-      awq_set_error("tensor " + want.first + " has another shape or type than config.json says");
-      return AWQ_ERR_IO;
-    }
-  }
-  return AWQ_OK;
 }
 
 // --- the model ---------------------------------------------------------------------------------------------
@@ -212,118 +161,23 @@ struct Buffers {
   std::vector<void*> cat;  // [ctx, mid] per layer (layers of one shape share)
 };
 
-constexpr int64_t kPassTokens = 2048;   // prompt positions per pass
-constexpr int64_t kLogitRows = 128;     // rows whose logits are formed at once
-constexpr int64_t kDefaultPositions = 8192;
-constexpr int64_t kDenseWorkspace = 32ll << 20;  // floats, for products that are cut along k
-
-struct KugilixEngine final : awq_engine {
+struct KugilixEngine final : ConfigModel {
   Spec spec;
-  bool f32 = false;
-  int64_t max_pos = 0, pass_tokens = 0;
-  int64_t ld = 0;  // a normalised token vector, padded
-  void *embed = nullptr, *head = nullptr;
-  const float* final_norm = nullptr;
   const double* freq = nullptr;
   std::vector<LayerDev> layers;
   std::vector<LayerRun> runs;
   Buffers step, pass;
-  int32_t* tokens = nullptr;
-  int32_t* rows = nullptr;  // which rows' logits are asked for
-  void* head_in = nullptr;  // [kLogitRows][ld]
-  float* logits = nullptr;  // [kLogitRows][vocab]
-  unsigned long long* best = nullptr;
   float* attn_parts = nullptr;
-  float* dense_ws = nullptr;
-  int64_t dense_ws_floats = 0;
-  std::vector<int64_t> bounds;
-  bool tap_on = false, tap_saved_graphs = true;
-  float* tap = nullptr;
-  int64_t tap_tokens = 0;
 
   const char* architecture() const override { return "Kugilix"; }
-  int64_t vocab_size() const override { return spec.vocab; }
-  int64_t hidden_size() const override { return spec.width; }
-  int64_t max_positions() const override { return max_pos; }
-  // nothing to clear: a run at position 0 reads neither convolution inputs nor recurrent state, and attention sees
-  // only rows of the running sequence
-  int begin_sequence() override { return AWQ_OK; }
-  const std::vector<int64_t>& length_bounds() const override { return bounds; }
-  int32_t epoch_step() const override { return 1; }
-  bool refeeds_hidden() const override { return false; }
-  int enqueue_step(StepKind kind, int64_t len_bound) override;
-  int64_t prompt_pass_tokens(int64_t done, int64_t rest) const override;
-  int enqueue_prompt_pass(const int32_t* ids, int64_t pos0, int64_t M) override;
-  int read_rows_logits(bool batched, const int32_t* which, int32_t n, float* host_dst) override;
-  int read_logits_f32(float* host_dst) override;
-  int read_hidden_f32(float* host_dst) override;
-  int set_layer_tap(int on) override;
-  int64_t read_layer_tap(float* host_dst, int64_t capacity) override;
+  int load_layers(Loader& ldr) override;
+  int make_buffers() override;
+  int64_t layer_runs() const override { return (int64_t)runs.size(); }
+  float* stream_of(bool one) override { return one ? step.x : pass.x; }
+  int run_pass(bool one, const int32_t* ids, int64_t M, PassPos pos) override;
 
-  int64_t unit() const { return f32 ? 4 : 2; }
-  int zeroed(void** p, int64_t bytes) {
-    bytes = round_up(std::max<int64_t>(bytes, 4), 4);
-    if (int rc = dev_alloc(p, bytes)) return rc;
-    return launch_fill_zero(*p, bytes, stream);
-  }
-  int load(const Safetensors& file);
-  int make_buffers(Buffers* b, int64_t n_tokens);
+  int make_activations(Buffers* b, int64_t n_tokens);
   int make_runs();
-  int run_layers(Buffers& b, int64_t M, PassPos pos);
-  int logits_of(const float* x, const int32_t* which, int64_t n, bool sample);
-};
-
-// --- weights -----------------------------------------------------------------------------------------------
-struct Loader {
-  KugilixEngine* e;
-  const Safetensors& file;
-  void* staging = nullptr;
-
-  int stage(const Tensor* t) {
-    AWQ_HIP_TRY(hipMemcpyAsync(staging, t->data, (size_t)t->bytes, hipMemcpyHostToDevice, e->stream));
-    return AWQ_OK;
-  }
-  static bool wide(const Tensor* t) { return t->dtype == "F32"; }
-  int vector(const std::string& name, const float** out) {
-    const Tensor* t = file.find(name);
-    int64_t n = 1;
-    for (int64_t d : t->shape) n *= d;
-    float* dst = nullptr;
-    if (int rc = e->dev_alloc((void**)&dst, n * 4)) return rc;
-    if (int rc = stage(t)) return rc;
-    *out = dst;
-    return launch_convert(staging, wide(t), dst, true, n, e->stream);
-  }
-  int matrix(const std::string& name, void* w, int64_t k, int64_t row0, int64_t col0) {
-    const Tensor* t = file.find(name);
-    if (int rc = stage(t)) return rc;
-    return launch_dense_pack(staging, wide(t), t->shape[0], t->shape[1], w, k, row0, col0, e->f32, e->stream);
-  }
-  int block(void** w, int64_t rows, int64_t k) { return e->zeroed(w, dense_weight_bytes(rows, k, e->f32)); }
-  int constants(const std::vector<float>& v, const float** out) {
-    float* dst = nullptr;
-    if (int rc = e->dev_alloc((void**)&dst, (int64_t)v.size() * 4)) return rc;
-    AWQ_HIP_TRY(hipMemcpy(dst, v.data(), v.size() * 4, hipMemcpyHostToDevice));
-    *out = dst;
-    return AWQ_OK;
-  }
-  void numbers(const std::string& name, std::vector<double>* out) {
-    const Tensor* t = file.find(name);
-    out->clear();
-    for (int64_t i = 0; i < t->shape[0]; ++i) {
-      uint32_t bits;
-      if (wide(t))
-        memcpy(&bits, (const char*)t->data + 4 * i, 4);
-      else {
-        uint16_t h;
-        memcpy(&h, (const char*)t->data + 2 * i, 2);
-        bits = (uint32_t)h << 16;
-      }
-      float f;
-      memcpy(&f, &bits, 4);
-      out->push_back(f);
-    }
-  }
 };
 
 double softplus(double z) { return log1p(exp(-fabs(z))) + fmax(z, 0.0); }
@@ -386,42 +240,17 @@ int load_layer(Loader& ld, KugilixEngine* e, int i) {
   return AWQ_OK;
 }
 
-int KugilixEngine::load(const Safetensors& file) {
-  const auto t0 = std::chrono::steady_clock::now();
-  Loader ldr{this, file};
-  int64_t largest = 4;
-  for (const auto& t : file.tensors()) largest = std::max(largest, t.second.bytes);
-  AWQ_HIP_TRY(hipMalloc(&ldr.staging, (size_t)largest));
-  const auto all = [&]() -> int {
-    const int64_t W = spec.width, V = spec.vocab;
-    ld = round_up(W, kDenseKAlign);
-    const Tensor* t = file.find("embed");
-    if (int rc = dev_alloc(&embed, V * W * unit())) return rc;
-    if (int rc = ldr.stage(t)) return rc;
-    if (int rc = launch_convert(ldr.staging, Loader::wide(t), embed, f32, V * W, stream)) return rc;
-    if (int rc = ldr.vector("final.norm", &final_norm)) return rc;
-    if (int rc = ldr.block(&head, round_up(V, kDenseRowAlign), ld)) return rc;
-    if (int rc = ldr.matrix("head", head, ld, 0, 0)) return rc;
-    std::vector<double> f;
-    for (int64_t i = 0; 2 * i < W; ++i) f.push_back(pow(10000.0, -2.0 * (double)i / (double)W));
-    double* fd = nullptr;
-    if (int rc = dev_alloc((void**)&fd, (int64_t)f.size() * 8)) return rc;
-    AWQ_HIP_TRY(hipMemcpy(fd, f.data(), f.size() * 8, hipMemcpyHostToDevice));
-    freq = fd;
-    for (size_t i = 0; i < spec.layers.size(); ++i)
-      if (int rc = load_layer(ldr, this, (int)i)) return rc;
-    AWQ_HIP_TRY(hipStreamSynchronize(stream));
-    return AWQ_OK;
-  };
-  const int rc = all();
-  (void)hipStreamSynchronize(stream);  // nothing may still read the staging buffer or the mapped file
-  (void)hipFree(ldr.staging);
-  if (rc == AWQ_OK) awq_note_load_seconds(std::chrono::duration<double>(std::chrono::steady_clock::now() - t0).count());
-  return rc;
+int KugilixEngine::load_layers(Loader& ldr) {
+  std::vector<double> f;
+  for (int64_t i = 0; 2 * i < width; ++i) f.push_back(pow(10000.0, -2.0 * (double)i / (double)width));
+  if (int rc = ldr.constants(f, &freq)) return rc;
+  for (size_t i = 0; i < spec.layers.size(); ++i)
+    if (int rc = load_layer(ldr, this, (int)i)) return rc;
+  return AWQ_OK;
 }
 
 // --- activations, caches and recurrent state ---------------------------------------------------------------
-int KugilixEngine::make_buffers(Buffers* b, int64_t n) {
+int KugilixEngine::make_activations(Buffers* b, int64_t n) {
   const int64_t W = spec.width;
   int64_t proj = 0, o = 0;
   b->cat.resize(layers.size());
@@ -442,6 +271,12 @@ int KugilixEngine::make_buffers(Buffers* b, int64_t n) {
   if (int rc = zeroed(&b->proj, n * proj * unit())) return rc;
   b->tokens = n;
   return AWQ_OK;
+}
+
+int KugilixEngine::make_buffers() {
+  if (int rc = make_activations(&step, 1)) return rc;
+  if (int rc = make_activations(&pass, pass_tokens)) return rc;
+  return make_runs();
 }
 
 int KugilixEngine::make_runs() {
@@ -484,8 +319,10 @@ int KugilixEngine::make_runs() {
 }
 
 // --- passes ------------------------------------------------------------------------------------------------
-int KugilixEngine::run_layers(Buffers& b, int64_t M, PassPos pos) {
+int KugilixEngine::run_pass(bool one, const int32_t* ids, int64_t M, PassPos pos) {
   const int64_t W = spec.width;
+  Buffers& b = one ? step : pass;
+  if (int rc = launch_embed_sinusoid(embed, f32, ids, d_token, pos, M, W, spec.embed_scale, freq, b.x, b.keep, stream)) return rc;
   for (size_t ri = 0; ri < runs.size(); ++ri) {
     const LayerRun& r = runs[ri];
     const LayerSpec& s = spec.layers[r.layer];
@@ -617,133 +454,12 @@ int KugilixEngine::run_layers(Buffers& b, int64_t M, PassPos pos) {
       if (int rc = launch_dense(a, f32, stream)) return rc;
     }
     if (tap_on) {
-      AWQ_HIP_TRY(hipMemcpyAsync(tap + (int64_t)ri * M * W, b.x, (size_t)(M * W) * 4, hipMemcpyDeviceToDevice, stream));
+      if (int rc = tap_layer((int64_t)ri, b.x, M)) return rc;
       if (r.add_embedding)
         if (int rc = launch_add_rows(b.x, b.keep, M * W, stream)) return rc;
     }
   }
-  if (tap_on) tap_tokens = M;
   return AWQ_OK;
-}
-
-int KugilixEngine::logits_of(const float* x, const int32_t* which, int64_t n, bool sample) {
-  NormConvArgs a;
-  a.x = x;
-  a.rows = which;
-  a.M = n;
-  a.width = spec.width;
-  a.groups = spec.groups;
-  a.eps = spec.eps;
-  a.w1 = final_norm;
-  a.out1 = head_in;
-  a.ld = ld;
-  if (int rc = launch_norm_conv(a, f32, stream)) return rc;
-  DenseArgs d;
-  d.w = head;
-  d.k = ld;
-  d.M = n;
-  d.out = sample ? DENSE_ARGMAX : DENSE_F32;
-  d.best = best;
-  d.workspace = dense_ws;
-  d.workspace_floats = dense_ws_floats;
-  d.seg[0].x = head_in;
-  d.seg[0].ldx = ld;
-  d.seg[0].y = logits;
-  d.seg[0].ldy = spec.vocab;
-  d.seg[0].rows = spec.vocab;
-  return launch_dense(d, f32, stream);
-}
-
-int KugilixEngine::enqueue_step(StepKind kind, int64_t) {
-  PassPos pos;
-  pos.dyn = d_state;
-  if (kind != STEP_SAMPLE) {
-    if (int rc = launch_embed_sinusoid(embed, f32, nullptr, d_token, pos, 1, spec.width, spec.embed_scale, freq, step.x,
-                                       step.keep, stream))
-      return rc;
-    if (int rc = run_layers(step, 1, pos)) return rc;
-  }
-  if (kind == STEP_PROMPT) return AWQ_OK;
-  if (int rc = logits_of(step.x, nullptr, 1, true)) return rc;
-  return launch_take_best(best, d_token, d_out, d_state, kind == STEP_GENERATE ? 1 : 0, stream);
-}
-
-int64_t KugilixEngine::prompt_pass_tokens(int64_t, int64_t rest) const {
-  if (rest == 1 || pass_tokens < 2) return 0;
-  // equal passes of whole tiles rather than full ones and a small rest
-  const int64_t passes = (rest + pass_tokens - 1) / pass_tokens;
-  return std::min<int64_t>(rest, std::min<int64_t>(pass_tokens, round_up((rest + passes - 1) / passes, 128)));
-}
-
-int KugilixEngine::enqueue_prompt_pass(const int32_t* ids, int64_t pos0, int64_t M) {
-  PassPos pos;
-  pos.pos0 = (int32_t)pos0;
-  pos.epoch = epoch_next;
-  epoch_next = (epoch_next + 1) & 0x3fffffff;
-  AWQ_HIP_TRY(hipMemcpyAsync(tokens, ids, (size_t)M * 4, hipMemcpyHostToDevice, stream));
-  if (int rc = launch_embed_sinusoid(embed, f32, tokens, d_token, pos, M, spec.width, spec.embed_scale, freq, pass.x,
-                                     pass.keep, stream))
-    return rc;
-  if (int rc = run_layers(pass, M, pos)) return rc;
-  // the row the first generated token is sampled from
-  AWQ_HIP_TRY(hipMemcpyAsync(step.x, pass.x + (M - 1) * spec.width, (size_t)spec.width * 4, hipMemcpyDeviceToDevice, stream));
-  return AWQ_OK;
-}
-
-int KugilixEngine::read_rows_logits(bool batched, const int32_t* which, int32_t n, float* host_dst) {
-  for (int64_t at = 0; at < n; at += kLogitRows) {
-    const int64_t k = std::min<int64_t>(kLogitRows, n - at);
-    if (batched) AWQ_HIP_TRY(hipMemcpyAsync(rows, which + at, (size_t)k * 4, hipMemcpyHostToDevice, stream));
-    if (int rc = logits_of(batched ? pass.x : step.x, batched ? rows : nullptr, k, false)) return rc;
-    AWQ_HIP_TRY(hipMemcpyAsync(host_dst + at * spec.vocab, logits, (size_t)(k * spec.vocab) * 4, hipMemcpyDeviceToHost, stream));
-    AWQ_HIP_TRY(hipStreamSynchronize(stream));
-  }
-  return AWQ_OK;
-}
-
-int KugilixEngine::read_logits_f32(float* host_dst) {
-  AWQ_HIP_TRY(hipStreamSynchronize(stream));
-  AWQ_HIP_TRY(hipMemcpy(host_dst, logits, (size_t)spec.vocab * 4, hipMemcpyDeviceToHost));
-  return AWQ_OK;
-}
-
-int KugilixEngine::read_hidden_f32(float* host_dst) {
-  AWQ_HIP_TRY(hipStreamSynchronize(stream));
-  AWQ_HIP_TRY(hipMemcpy(host_dst, step.x, (size_t)spec.width * 4, hipMemcpyDeviceToHost));
-  return AWQ_OK;
-}
-
-int KugilixEngine::set_layer_tap(int on) {
-  AWQ_HIP_TRY(hipStreamSynchronize(stream));
-  if (on && !tap)
-    if (int rc = dev_alloc((void**)&tap, (int64_t)runs.size() * pass_tokens * spec.width * 4)) return rc;
-  if ((on != 0) != tap_on) {
-    if (on) {
-      tap_saved_graphs = graph_mode;
-      graph_mode = false;
-    } else {
-      graph_mode = tap_saved_graphs;
-    }
-  }
-  tap_on = on != 0;
-  tap_tokens = 0;
-  return AWQ_OK;
-}
-
-int64_t KugilixEngine::read_layer_tap(float* host_dst, int64_t capacity) {
-  if (!tap_on || tap_tokens == 0) {
-    awq_set_error("no pass was tapped");
-    return -1;
-  }
-  const int64_t n = (int64_t)runs.size() * tap_tokens * spec.width;
-  if (host_dst) {
-    if (hipStreamSynchronize(stream) != hipSuccess ||
-        hipMemcpy(host_dst, tap, (size_t)std::min(n, capacity) * 4, hipMemcpyDeviceToHost) != hipSuccess) {
-      awq_set_error("reading the tapped layers failed");
-      return -1;
-    }
-  }
-  return n;
 }
 
 int open_kugilix(const char* dir, const awq_open_options& opt, awq_engine** out) {
@@ -752,33 +468,12 @@ int open_kugilix(const char* dir, const awq_open_options& opt, awq_engine** out)
   Safetensors file;
   if (int rc = read_spec(dir, &e->spec)) return rc;
   if (int rc = file.open(std::string(dir) + "/model.safetensors")) return rc;
-  if (int rc = check_tensors(e->spec, file)) return rc;
-  e->f32 = opt.dtype == AWQ_DTYPE_FLOAT32;
-  e->max_pos = opt.max_positions ? opt.max_positions : kDefaultPositions;
-  AWQ_REQUIRE(e->max_pos <= (1 << 24), "max_positions is too large");
-  e->pass_tokens = std::min<int64_t>(kPassTokens, e->max_pos);
-  e->bounds = {1ll << 40};
-  e->batched_prefill = true;
-  if (int rc = e->init_driver(e->max_pos)) return rc;
-  if (int rc = e->load(file)) return rc;
-  if (int rc = e->make_buffers(&e->step, 1)) return rc;
-  if (int rc = e->make_buffers(&e->pass, e->pass_tokens)) return rc;
-  if (int rc = e->make_runs()) return rc;
-  if (!e->f32) {
-    e->dense_ws_floats = std::min<int64_t>(kDenseWorkspace, 4 * e->pass_tokens * round_up(e->spec.width, kDenseRowAlign));
-    if (int rc = e->dev_alloc((void**)&e->dense_ws, e->dense_ws_floats * 4)) return rc;
-  }
-  if (int rc = e->zeroed((void**)&e->tokens, e->pass_tokens * 4)) return rc;
-  if (int rc = e->zeroed((void**)&e->rows, kLogitRows * 4)) return rc;
-  if (int rc = e->zeroed(&e->head_in, kLogitRows * e->ld * e->unit())) return rc;
-  if (int rc = e->zeroed((void**)&e->logits, kLogitRows * e->spec.vocab * 4)) return rc;
-  if (int rc = e->zeroed((void**)&e->best, 8)) return rc;
-  if (int rc = launch_fill_zero(e->d_token, 4, e->stream)) return rc;
-  AWQ_HIP_TRY(hipStreamSynchronize(e->stream));
-  e->finalized = true;
-  if (int rc = awq_reset(e.get())) return rc;
-  *out = e.release();
-  return AWQ_OK;
+  if (int rc = check_tensors(expected_tensors(e->spec), file)) return rc;
+  e->vocab = e->spec.vocab;
+  e->width = e->spec.width;
+  e->norm_groups = e->spec.groups;
+  e->eps = e->spec.eps;
+  return ConfigModel::open(std::move(e), file, opt, out);
 }
 
 ModelClass g_class("Kugilix", open_kugilix);
