@@ -14,6 +14,7 @@ Other modes (plain text output, used for the summaries under profiles/):
     --mode attention [--one-cache]   decode attention by attended length
     --mode prefill [--lengths a,b]   batched prompt pass of the 36-layer model by prompt length
     --mode traffic                   a 1 GiB copy, then the engine's w1 launches (for rocprofv3 --pmc runs)
+    --mode tudasun                   prompt and decode throughput of the Tudasun design beside the Kugilix model at equal size
     --mode kugilix                   prompt and decode throughput of the Kugilix design beside the int4 model at equal size
     --mode w4a16                     W4A16 products of config 5 (token sweep on the w1 and w2 shapes)
 """
@@ -226,6 +227,13 @@ def mode_w4a16(args):
     print(json.dumps(w4a16.measure(tokens, tuple(args.shapes.split(",")))), flush=True)
 
 
+def mode_tudasun(args):
+    bench = importlib.import_module("cuda-kernel-qwen3-8b-awq_amd.bench_tudasun")
+    widths = [int(v) for v in args.tudasun_sizes.split(",")]
+    prompts = [int(v) for v in args.tudasun_prompts.split(",")]
+    print(json.dumps(bench.measure(widths, args.tudasun_only, prompts), indent=1), flush=True)
+
+
 def mode_kugilix(args):
     bench = importlib.import_module("cuda-kernel-qwen3-8b-awq_amd.bench_kugilix")
     widths = [int(v) for v in args.kugilix_sizes.split(",")]
@@ -249,7 +257,7 @@ def main():
     ap.add_argument("--fused", type=int, default=None,
                     help="which pairs of a layer's launches run as one: 1 Wo + W1, 2 Wqkv + attention, 3 both (default: the engine's)")
     ap.add_argument("--mode", choices=["decode", "steps", "attention", "prefill", "traffic", "w4a16", "fused-timeline", "qkv-timeline",
-                                       "kugilix"], default="decode",
+                                       "kugilix", "tudasun"], default="decode",
                     help="decode: the benchmark line; steps: only the prompt and the timed decode steps (for traces)")
     ap.add_argument("--one-cache", action="store_true", help="--mode attention: every launch reads the same cache")
     ap.add_argument("--att-lengths", default="128,256,512,576,577,768,1024,1025,1536,2048,2049,4096,8192,16384,40960",
@@ -257,6 +265,9 @@ def main():
     ap.add_argument("--lengths", default="32,128,256,576,1024,1280,2040,4096,8192,30000", help="--mode prefill")
     ap.add_argument("--tokens", default="1,4,16,64,128,512,2048", help="--mode w4a16: token counts")
     ap.add_argument("--shapes", default="w1,w2", help="--mode w4a16: of w1 (12288x4096), w2 (4096x12288), wo (4096x4096)")
+    ap.add_argument("--tudasun-sizes", default="2048,4096", help="--mode tudasun: widths")
+    ap.add_argument("--tudasun-prompts", default="128,1024", help="--mode tudasun: prompt lengths")
+    ap.add_argument("--tudasun-only", action="store_true", help="--mode tudasun: without the Kugilix model")
     ap.add_argument("--kugilix-sizes", default="2048,4096", help="--mode kugilix: widths")
     ap.add_argument("--kugilix-prompts", default="128,1024", help="--mode kugilix: prompt lengths")
     ap.add_argument("--kugilix-only", action="store_true", help="--mode kugilix: without the int4 model")
@@ -277,7 +288,7 @@ def main():
     if args.mode not in ("decode", "steps"):
         return {"attention": mode_attention, "prefill": mode_prefill, "traffic": mode_traffic,
                 "fused-timeline": mode_fused_timeline, "qkv-timeline": mode_qkv_timeline,
-                "w4a16": mode_w4a16, "kugilix": mode_kugilix}[args.mode](args)
+                "w4a16": mode_w4a16, "kugilix": mode_kugilix, "tudasun": mode_tudasun}[args.mode](args)
 
     import numpy as np
     import torch

@@ -65,12 +65,12 @@ def shapes(cfg):
     return out
 
 
-def write_model(folder, cfg, seed=0):
+def write_model(folder, cfg, seed=0, shapes_of=shapes):
     """config.json and model.safetensors with random weights (one block of normal numbers, reused at offsets)"""
     import numpy as np
     rng = np.random.default_rng(seed)
     pool = rng.standard_normal(1 << 24, dtype=np.float32)
-    sh = shapes(cfg)
+    sh = shapes_of(cfg)
     header, at = {}, 0
     for name, s in sh.items():
         n = 2 * int(np.prod(s))
@@ -84,7 +84,7 @@ def write_model(folder, cfg, seed=0):
         for name, s in sh.items():
             n = int(np.prod(s))
             scale = 0.02 if name == "embed" else (s[1] ** -0.5 if len(s) == 2 else 0.1)
-            shift = 1.0 if name.endswith(("norm", "norm1", "norm2")) else 0.0
+            shift = 1.0 if name.endswith(("norm", "norm1", "norm2")) else 0.5 if name.endswith("lower") else 0.0
             while n > 0:
                 k = min(n, pool.size // 2)
                 o = int(rng.integers(0, pool.size - k))

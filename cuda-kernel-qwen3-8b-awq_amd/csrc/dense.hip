@@ -24,27 +24,33 @@ __device__ __forceinline__ float exp_minus_1_minus(float z) {
   return (expf(z) - 1.0f) - z;
 }
 
+// `bias` and `lower`: the row's entries, where the activation has them
 template <bool F32>
-__device__ __forceinline__ float activate(const DenseSegment& s, int row, float z) {
+__device__ __forceinline__ float activate_with(const DenseSegment& s, int row, float z, float bias, float lower) {
   if (s.act == DENSE_SILU) return row < s.act_rows ? z * (F32 ? sigmoid_exact(z) : sigmoid_f32(z)) : z;
   if (s.act == DENSE_XIELU) {
     const float h = 0.5f * z;
     return z > 0.0f ? __builtin_fmaf(s.act_pos * z, z, h) : __builtin_fmaf(s.act_neg, exp_minus_1_minus(z), h);
   }
-  if (s.act == DENSE_SIGMOID) {
-    z += s.bias[row];
-    return F32 ? sigmoid_exact(z) : sigmoid_f32(z);
-  }
+  if (s.act == DENSE_SIGMOID) return F32 ? sigmoid_exact(z + bias) : sigmoid_f32(z + bias);
   if (s.act == DENSE_GELU) {  // (1 + tanh u) / 2 = sigmoid(2 u)
     const float u2 = 1.5957691216057307117f * __builtin_fmaf(0.044715f * z * z, z, z);
     return z * (F32 ? sigmoid_exact(u2) : sigmoid_f32(u2));
   }
   if (s.act == DENSE_LOG_DECAY) {
-    z += s.bias[row];
-    return -s.act_pos * (log1pf(expf(-fabsf(z))) + fmaxf(-z, 0.0f));
+    z += bias;
+    if (F32) return -s.act_pos * (log1pf(expf(-fabsf(z))) + fmaxf(-z, 0.0f));
+    // (off by what one rounding of the decay itself is off)
+    const float e = __builtin_amdgcn_exp2f(-1.44269504088896340736f * fabsf(z));
+    return -s.act_pos * __builtin_fmaf(0.693147180559945309417f, __builtin_amdgcn_logf(1.0f + e), fmaxf(-z, 0.0f));
   }
-  if (s.act == DENSE_FORGET) return (1.0f - s.lower[row]) * sigmoid_exact(-(z + s.bias[row]));
+  if (s.act == DENSE_FORGET) return (1.0f - lower) * sigmoid_exact(-(z + bias));
   return z;
+}
+
+template <bool F32>
+__device__ __forceinline__ float activate(const DenseSegment& s, int row, float z) {
+  return activate_with<F32>(s, row, z, s.bias ? s.bias[row] : 0.0f, s.lower ? s.lower[row] : 0.0f);
 }
 
 __device__ __forceinline__ float softcap(const DenseSegment& s, float z) { return s.act_pos * tanhf(z / s.act_pos); }
@@ -59,6 +65,12 @@ __device__ __forceinline__ int32_t f32_key(float v) {
   const uint32_t b = __float_as_uint(v);
   if ((b & 0x7fffffffu) == 0) return 0;
   return (b & 0x80000000u) ? -(int32_t)(b & 0x7fffffffu) : (int32_t)b;
+}
+
+// the lanes' LDS writes ahead of this are seen by all lanes' reads behind it
+__device__ __forceinline__ void wave_sync() {
+  __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+  __builtin_amdgcn_wave_barrier();
 }
 
 __device__ __forceinline__ const DenseSegment& segment_of(const DenseArgs& a, int row) {
@@ -215,8 +227,8 @@ constexpr int DENSE_PART = 100;
 // LISTED: the tokens come from runs of a list, each with a weight block of its own.
 template <int TT, int OUT, bool LISTED = false>
 __global__ __launch_bounds__(256, 2) void dense_many_kernel(DenseArgs a, int row_tiles, int tok_tiles, int cuts) {
-  __shared__ __attribute__((aligned(16))) bf16_t tile0[32 * TT * 64];
-  __shared__ __attribute__((aligned(16))) bf16_t tile1[32 * TT * 64];
+  __shared__ __attribute__((aligned(16))) bf16_t tile0[2 * 32 * TT * 64];
+  bf16_t* const tile1 = tile0 + 32 * TT * 64;
   const int total = row_tiles * tok_tiles * cuts;
   // workgroups whose indices agree modulo 8 share a die: each die walks its own run of row tiles
   const int per = (total + 7) >> 3;
@@ -305,29 +317,12 @@ __global__ __launch_bounds__(256, 2) void dense_many_kernel(DenseArgs a, int row
     }
   }
   // acc[b][t][i]: row 32 b + 8 (i / 4) + 4 kh + i % 4 of the wavefront's 64, token 32 t + n
+  // A block of 32 tokens and 32 rows is turned in LDS, 4 KB of its own per wavefront, so that eight lanes hold and store the
+  // rows of a token side by side; four rows (a piece) of token n are at place piece ^ (n % 8).
   const int row_w = rt * 256 + wave * 64;
-  if constexpr (OUT == DENSE_STORE) {
-#pragma unroll
-    for (int b = 0; b < 2; ++b) {
-      const DenseSegment& out = segment_of(a, row_w + 32 * b);
-      const int local_b = row_w + 32 * b - out.row0 + 4 * kh;
-#pragma unroll
-      for (int t = 0; t < TT; ++t) {
-        if (out.act == DENSE_GLU) {
-#pragma unroll
-          for (int i = 0; i < 16; ++i)
-            if ((i & 4) == 0) acc[b][t][i] = glu<false>(acc[b][t][i], acc[b][t][i + 4]);
-        } else if (out.act != DENSE_NONE) {
-#pragma unroll
-          for (int i = 0; i < 16; ++i) {
-            const int row = local_b + 8 * (i >> 2) + (i & 3);
-            if (row < out.rows) acc[b][t][i] = activate<false>(out, row, acc[b][t][i]);
-          }
-        }
-      }
-    }
-  }
   const int64_t y0 = blockIdx.y * a.y_batch;
+  float* const turn = reinterpret_cast<float*>(tile0) + wave * 1024;
+  __syncthreads();  // the last step's readers are done
 #pragma unroll
   for (int b = 0; b < 2; ++b) {
     const DenseSegment& out = segment_of(a, row_w + 32 * b);
@@ -336,21 +331,43 @@ __global__ __launch_bounds__(256, 2) void dense_many_kernel(DenseArgs a, int row
     const int n_rows = gated ? out.glu_rows : out.rows;
     if (OUT != DENSE_PART && local_b >= out.rows) continue;  // padding
     const bool by_four = ((out.ldy | a.y_batch) & 3) == 0 && !(OUT == DENSE_STORE && out.mul);
+    // pieces of a token: 8, or 4 of a gated segment
+    const int shift = gated ? 2 : 3, piece = lane & ((1 << shift) - 1);
+    const int row = (gated ? local_b / 2 : local_b) + 4 * piece;
+    float bias[4] = {}, lower[4] = {};  // of this lane's rows
+    if (OUT == DENSE_STORE && out.bias) {
+#pragma unroll
+      for (int j = 0; j < 4; ++j) bias[j] = out.bias[min(row + j, n_rows - 1)];
+    }
+    if (OUT == DENSE_STORE && out.lower) {
+#pragma unroll
+      for (int j = 0; j < 4; ++j) lower[j] = out.lower[min(row + j, n_rows - 1)];
+    }
 #pragma unroll
     for (int t = 0; t < TT; ++t) {
-      int64_t tok = tt0 + 32 * t + n;
-      if (tok >= n_tok) continue;
-      if constexpr (LISTED) tok = list[tok];
 #pragma unroll
       for (int g = 0; g < 4; ++g) {
         if (gated && (g & 1)) continue;
         f32x4_t v;
 #pragma unroll
-        for (int j = 0; j < 4; ++j) v[j] = acc[b][t][4 * g + j];
+        for (int j = 0; j < 4; ++j) v[j] = gated ? glu<false>(acc[b][t][4 * g + j], acc[b][t][(4 * g + 4 + j) & 15]) : acc[b][t][4 * g + j];
+        const int p = gated ? g + kh : 2 * g + kh;
+        *reinterpret_cast<f32x4_t*>(turn + n * 32 + ((p ^ (n & 7)) << 2)) = v;
+      }
+      wave_sync();
+#pragma unroll 1
+      for (int token = lane >> shift; token < 32; token += 64 >> shift) {
+        f32x4_t v = *reinterpret_cast<const f32x4_t*>(turn + token * 32 + ((piece ^ (token & 7)) << 2));
+        int64_t tok = tt0 + 32 * t + token;
+        if (tok >= n_tok) continue;
+        if constexpr (LISTED) tok = list[tok];
         if constexpr (OUT == DENSE_PART) {
-          *reinterpret_cast<f32x4_t*>(a.workspace + ((int64_t)cut * a.M + tok) * row_tiles * 256 + row_w + 32 * b + 8 * g + 4 * kh) = v;
+          *reinterpret_cast<f32x4_t*>(a.workspace + ((int64_t)cut * a.M + tok) * row_tiles * 256 + row_w + 32 * b + 4 * piece) = v;
         } else {
-          const int row = gated ? local_b / 2 + 4 * g + 4 * kh : local_b + 8 * g + 4 * kh;
+          if (OUT == DENSE_STORE && !gated && out.act != DENSE_NONE) {
+#pragma unroll
+            for (int j = 0; j < 4; ++j) v[j] = activate_with<false>(out, row + j, v[j], bias[j], lower[j]);
+          }
           const int64_t at = y0 + tok * out.ldy + row;
           if (row + 3 < n_rows && by_four) {
             if (OUT == DENSE_STORE && !out.y_f32) {
@@ -378,6 +395,7 @@ __global__ __launch_bounds__(256, 2) void dense_many_kernel(DenseArgs a, int row
           }
         }
       }
+      wave_sync();
     }
   }
 }
@@ -580,13 +598,15 @@ int launch_many(const DenseArgs& a, bool f32, int64_t rows, hipStream_t st) {
                        dim3(256), 0, st, a);
   } else {
     const int row_tiles = (int)(rows / 256);
-    const bool wide = a.M > 64;
+    // few weights (few rows or a short k) are read again for less: tiles of 64 tokens where those of 128 are few
+    const bool small = (row_tiles <= 4 || a.k <= 512) && row_tiles * ((a.M + 127) / 128) <= 256;
+    const bool wide = a.M > 64 && !small;
     const int64_t tok_tiles = wide ? (a.M + 127) / 128 : (a.M + 63) / 64;
     const int64_t tiles = row_tiles * tok_tiles;
-    // two workgroups per compute unit, at least eight steps each
+    // two workgroups per compute unit, at least eight steps each (four in a small product)
     int64_t cuts = 1;
     if (a.workspace && a.batch == 1 && a.M <= 65535 && tiles < 384) {
-      cuts = std::min<int64_t>((512 + tiles / 2) / tiles, (a.k >> 6) / 8);
+      cuts = std::min<int64_t>((512 + tiles / 2) / tiles, (a.k >> 6) / (small ? 4 : 8));
       cuts = std::max<int64_t>(1, std::min<int64_t>(cuts, a.workspace_floats / (a.M * rows)));
     }
     const dim3 grid((unsigned)((tiles * cuts + 7) / 8 * 8), (unsigned)a.batch);
@@ -616,8 +636,10 @@ int launch_listed(const DenseArgs& a, bool f32, int64_t rows, hipStream_t st) {
   } else {
     const int row_tiles = (int)(rows / 256);
     const unsigned grid = (unsigned)(((int64_t)row_tiles * a.max_tiles + 7) / 8 * 8);
-    hipLaunchKernelGGL((dense_many_kernel<kDenseTileTokens / 32, DENSE_STORE, true>), dim3(grid), dim3(256), 0, st, a, row_tiles,
-                       a.max_tiles, 1);
+    if (a.tile_tokens <= 64)
+      hipLaunchKernelGGL((dense_many_kernel<2, DENSE_STORE, true>), dim3(grid), dim3(256), 0, st, a, row_tiles, a.max_tiles, 1);
+    else
+      hipLaunchKernelGGL((dense_many_kernel<4, DENSE_STORE, true>), dim3(grid), dim3(256), 0, st, a, row_tiles, a.max_tiles, 1);
   }
   AWQ_HIP_TRY(hipGetLastError());
   return AWQ_OK;
@@ -672,7 +694,8 @@ int launch_dense(const DenseArgs& args, bool f32, hipStream_t st) {
               "bad batch");
   AWQ_REQUIRE(!a.ids || (a.M == 1 && a.n_groups >= 0), "weight blocks by number take one token");
   if (a.tiles) {
-    AWQ_REQUIRE(a.out == DENSE_STORE && a.list && a.list_div >= 1 && a.batch == 1 && a.max_tiles >= 1 && a.max_tiles <= 65535,
+    AWQ_REQUIRE(a.out == DENSE_STORE && a.list && a.list_div >= 1 && a.batch == 1 && a.max_tiles >= 1 && a.max_tiles <= 65535 &&
+                    a.tile_tokens >= 1 && a.tile_tokens <= (f32 ? 64 : 128),
                 "bad list of tokens");
     return launch_listed(a, f32, rows, st);
   }

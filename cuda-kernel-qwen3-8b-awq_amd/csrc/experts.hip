@@ -110,7 +110,7 @@ __global__ __launch_bounds__(1024) void plan_kernel(RouteArgs a, int max_tiles) 
   }
   __syncthreads();
   for (int e0 = 0; e0 < E; e0 += 1024) {
-    const int e = e0 + tid, c = e < E ? counts[e] : 0, k = (c + kDenseTileTokens - 1) / kDenseTileTokens;
+    const int e = e0 + tid, c = e < E ? counts[e] : 0, k = (c + a.tile_tokens - 1) / a.tile_tokens;
     int entries = c, tiles = k;  // sums up to and with this expert
 #pragma unroll
     for (int off = 1; off < 64; off <<= 1) {
@@ -127,8 +127,8 @@ __global__ __launch_bounds__(1024) void plan_kernel(RouteArgs a, int max_tiles) 
       for (int i = 0; i < k; ++i) {
         DenseTile d;
         d.group = e;
-        d.first = at + i * kDenseTileTokens;
-        d.count = min(kDenseTileTokens, c - i * kDenseTileTokens);
+        d.first = at + i * a.tile_tokens;
+        d.count = min(a.tile_tokens, c - i * a.tile_tokens);
         a.tiles[tile + i] = d;
       }
     }
@@ -146,10 +146,12 @@ __global__ __launch_bounds__(1024) void plan_kernel(RouteArgs a, int max_tiles) 
 }  // namespace
 
 // a run of each expert may end in a tile that is not full
-int32_t route_max_tiles(int64_t M, int32_t top, int32_t experts) {
+int32_t route_max_tiles(int64_t M, int32_t top, int32_t experts, int32_t tile_tokens) {
   const int64_t pairs = M * top;
-  return (int32_t)std::max<int64_t>(1, std::min<int64_t>(pairs, pairs / kDenseTileTokens + std::min<int64_t>(experts, pairs)));
+  return (int32_t)std::max<int64_t>(1, std::min<int64_t>(pairs, pairs / tile_tokens + std::min<int64_t>(experts, pairs)));
 }
+
+int32_t route_tile_tokens(int64_t M, int32_t top, int32_t outputs, bool f32) { return !f32 && M * top >= 128ll * outputs ? 128 : 64; }
 
 int launch_route(const RouteArgs& a, hipStream_t st) {
   AWQ_REQUIRE(a.logits && a.ids && a.weights && a.M >= 1, "bad arguments");
@@ -158,7 +160,7 @@ int launch_route(const RouteArgs& a, hipStream_t st) {
   AWQ_REQUIRE(a.groups == 0 || (a.groups > 0 && a.outputs % a.groups == 0 && a.keep >= 1 && a.keep <= a.groups &&
                                 a.keep * (a.outputs / a.groups) >= a.top),
               "bad groups");
-  AWQ_REQUIRE(a.M * a.top < (1 << 30), "too many tokens");
+  AWQ_REQUIRE(a.M * a.top < (1 << 30) && a.tile_tokens >= 1, "too many tokens");
   const size_t lds = sizeof(float) * (2 * a.outputs + a.groups);
   if (a.outputs <= 1024)
     hipLaunchKernelGGL(route_kernel<4>, dim3((unsigned)((a.M + 3) / 4)), dim3(256), 4 * lds, st, a);
@@ -167,7 +169,7 @@ int launch_route(const RouteArgs& a, hipStream_t st) {
   AWQ_HIP_TRY(hipGetLastError());
   if (a.M > 1 && a.experts > 0) {
     AWQ_REQUIRE(a.tiles && a.list, "no place for the plan");
-    hipLaunchKernelGGL(plan_kernel, dim3(1), dim3(1024), sizeof(int) * 2 * a.experts, st, a, route_max_tiles(a.M, a.top, a.experts));
+    hipLaunchKernelGGL(plan_kernel, dim3(1), dim3(1024), sizeof(int) * 2 * a.experts, st, a, route_max_tiles(a.M, a.top, a.experts, a.tile_tokens));
     AWQ_HIP_TRY(hipGetLastError());
   }
   return AWQ_OK;

@@ -151,7 +151,7 @@ __global__ __launch_bounds__(256) void latent_query_kernel(LatentAttnArgs a, int
 //                                 read, slice j taking keys 16 j + 8 (e / 4) + 4 kh + e % 4; weights as two bfloat16 terms
 // A part is [maximum (binary logarithm), sum, -, -, columns].
 constexpr int kRows = 32, kKeys = 64, kScoreStride = kKeys + 4, kWeightStride = kKeys + 8;
-constexpr int kMaxParts = 128;
+constexpr int kMaxParts = 128, kMaxRow = 640;
 
 __host__ __device__ inline size_t rows_lds(int row) {
   return (size_t)(kKeys + kRows) * (row + 8) * 2 + kRows * kScoreStride * 4 + 2 * kRows * kWeightStride * 2 + kRows * 4;
@@ -166,7 +166,7 @@ __device__ __forceinline__ int tiles_per_part(int row0, int rows, int heads, int
 template <int NT>
 __global__ __launch_bounds__(256) void latent_rows_kernel(LatentAttnArgs a) {
   extern __shared__ __attribute__((aligned(16))) char raw[];
-  const int row = a.l.row(), rp = a.l.rank_padded(), KS = row + 8, pieces = row >> 3;
+  const int row = a.l.row(), rp = a.l.rank_padded(), KS = row + 8;
   bf16_t* const kt = reinterpret_cast<bf16_t*>(raw);                // [64][KS]
   bf16_t* const qt = kt + kKeys * KS;                               // [32][KS]
   float* const sc = reinterpret_cast<float*>(qt + kRows * KS);      // [32][kScoreStride]
@@ -182,10 +182,26 @@ __global__ __launch_bounds__(256) void latent_rows_kernel(LatentAttnArgs a) {
   if (first >= end) return;
   const bf16_t* const cache = reinterpret_cast<const bf16_t*>(a.cache);
   const bf16_t* const ql = reinterpret_cast<const bf16_t*>(a.ql);
-  for (int i = tid; i < kRows * pieces; i += 256) {
-    const int r = i / pieces, at = (i - r * pieces) * 8;
-    *reinterpret_cast<bf16x8_t*>(qt + r * KS + at) =
-        *reinterpret_cast<const bf16x8_t*>(ql + (int64_t)min(row0 + r, rows - 1) * row + at);
+  // four threads copy a key row, eight a query row, all loads in flight at once
+  constexpr int kPieces = kMaxRow / 32;
+  const int kr = tid >> 2, kf = (tid & 3) * 8, qr = tid >> 3, qf = (tid & 7) * 8;
+  bf16x8_t kx[kPieces];
+  auto load_keys = [&](int tile) __attribute__((always_inline)) {
+    const bf16_t* const src = cache + ((int64_t)tile * kKeys + kr) * row + kf;  // the cache is whole tiles
+#pragma unroll
+    for (int i = 0; i < kPieces; ++i)
+      if (32 * i < row) kx[i] = *reinterpret_cast<const bf16x8_t*>(src + 32 * i);
+  };
+  {
+    const bf16_t* const src = ql + (int64_t)min(row0 + qr, rows - 1) * row + qf;
+    bf16x8_t x[kPieces / 2];
+#pragma unroll
+    for (int i = 0; i < kPieces / 2; ++i)
+      if (64 * i + qf < row) x[i] = *reinterpret_cast<const bf16x8_t*>(src + 64 * i);
+    load_keys(first);
+#pragma unroll
+    for (int i = 0; i < kPieces / 2; ++i)
+      if (64 * i + qf < row) *reinterpret_cast<bf16x8_t*>(qt + qr * KS + qf + 64 * i) = x[i];
   }
   f32x16_t o[NT];
 #pragma unroll
@@ -200,11 +216,10 @@ __global__ __launch_bounds__(256) void latent_rows_kernel(LatentAttnArgs a) {
   float m_run = -INFINITY, l_run = 0.0f;
   for (int tile = first; tile < end; ++tile) {
     __syncthreads();  // the previous tile's readers are done
-    const bf16_t* const src = cache + (int64_t)tile * kKeys * row;  // the cache is whole tiles
-    for (int i = tid; i < kKeys * pieces; i += 256) {
-      const int r = i / pieces, at = (i - r * pieces) * 8;
-      *reinterpret_cast<bf16x8_t*>(kt + r * KS + at) = *reinterpret_cast<const bf16x8_t*>(src + (int64_t)r * row + at);
-    }
+#pragma unroll
+    for (int i = 0; i < kPieces; ++i)
+      if (32 * i < row) *reinterpret_cast<bf16x8_t*>(kt + kr * KS + kf + 32 * i) = kx[i];
+    if (tile + 1 < end) load_keys(tile + 1);
     __syncthreads();
     f32x4_t s0 = {0.0f, 0.0f, 0.0f, 0.0f}, s1 = s0;
     const bf16_t* const kp = kt + (16 * wave + n16) * KS + 8 * c16;
@@ -499,7 +514,7 @@ int64_t q_inputs(const LatentAttnArgs& a) { return round_up(a.dim, kDenseKAlign)
 int64_t v_inputs(const LatentAttnArgs& a) { return round_up(a.l.rank, kDenseKAlign); }
 
 // The rows kernel's shapes
-bool on_matrix_cores(const LatentAttnArgs& a, bool f32) { return !f32 && a.l.rank_padded() <= 512 && rows_lds(a.l.row()) <= 160 * 1024; }
+bool on_matrix_cores(const LatentAttnArgs& a, bool f32) { return !f32 && a.l.rank_padded() <= 512 && a.l.row() <= kMaxRow; }
 
 // Keys and values formed first: sizes the tiles have instances for, and enough queries that the products over dim and vdim
 // instead of rank (twice) pay for forming them, per key and head rank * (dim + vdim)
@@ -525,6 +540,8 @@ int launch_prepare(const LatentAttnArgs& a, hipStream_t st) {
   return AWQ_OK;
 }
 
+static_assert((size_t)(kKeys + kRows) * (kMaxRow + 8) * 2 + kRows * kScoreStride * 4 + 4 * kRows * kWeightStride + kRows * 4 <= 160 * 1024,
+              "more LDS than a compute unit has");
 template <int NT>
 int launch_rows(const LatentAttnArgs& a, int parts, hipStream_t st) {
   static bool raised = false;  // more LDS than the default limit of a launch

@@ -103,9 +103,8 @@ struct DenseArgs {
   // last) name runs of `list`; entry p of the list reads input row p / list_div and writes output row p.
   const DenseTile* tiles = nullptr;
   const int32_t* list = nullptr;
-  int32_t max_tiles = 0, list_div = 1;
+  int32_t max_tiles = 0, tile_tokens = 64, list_div = 1;
 };
-constexpr int kDenseTileTokens = 64;  // tokens of a DenseTile at most
 inline int64_t dense_glu_rows(int64_t n) { return round_up(n, 8) * 2; }
 int64_t dense_weight_bytes(int64_t rows_padded, int64_t k_padded, bool f32);
 // src [rows][cols] bfloat16 or float, row major on the device, into rows row0.., inputs col0.. of a block (col0 a
@@ -293,10 +292,13 @@ struct RouteArgs {
   float* weights = nullptr;       // [M][top], the chosen scores over their sum
   int64_t M = 0;
   // more than one token: the plan of the experts' products, token t's j-th choice is entry t * top + j
+  int32_t tile_tokens = 64;
   DenseTile* tiles = nullptr;     // [route_max_tiles]
   int32_t* list = nullptr;        // [M * top]
 };
-int32_t route_max_tiles(int64_t M, int32_t top, int32_t experts);
+// tokens of a tile: 64, or 128 where an expert has as many on average and the products have tiles of that size
+int32_t route_tile_tokens(int64_t M, int32_t top, int32_t outputs, bool f32);
+int32_t route_max_tiles(int64_t M, int32_t top, int32_t experts, int32_t tile_tokens);
 int launch_route(const RouteArgs& a, hipStream_t st);
 
 // --- around a sublayer (sublayer_ops.hip) --------------------------------------------------------------------------

@@ -45,7 +45,7 @@ __device__ __forceinline__ float group_sum(float v, float* sums) {
   return all;
 }
 
-template <typename T>
+template <typename T, int V>
 __global__ __launch_bounds__(256) void embed_tokens_kernel(const T* __restrict__ table, const T* __restrict__ side_table,
                                                            const int32_t* __restrict__ tokens, const int32_t* __restrict__ last,
                                                            PassPos pos, int64_t width, int64_t side_width, float* __restrict__ x,
@@ -58,9 +58,15 @@ __global__ __launch_bounds__(256) void embed_tokens_kernel(const T* __restrict__
   } else {
     tok = tokens[t];
   }
-  for (int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x; i < width + side_width; i += (int64_t)gridDim.x * 256) {
-    if (i < width) x[t * width + i] = (float)table[tok * width + i];
-    else side[t * side_width + i - width] = side_table[tok * side_width + i - width];
+  for (int64_t i = ((int64_t)blockIdx.x * 256 + threadIdx.x) * V; i < width + side_width; i += (int64_t)gridDim.x * 256 * V) {
+    float v[V];
+    if (i < width) {
+      read<T, V>(table + tok * width + i, v);
+      write<float, V>(x + t * width + i, v);
+    } else {
+      read<T, V>(side_table + tok * side_width + i - width, v);
+      write<T, V>(side + t * side_width + i - width, v);
+    }
   }
 }
 
@@ -190,6 +196,19 @@ __global__ __launch_bounds__(256) void head_norm_kernel(const float* __restrict_
 }
 
 template <typename T>
+void embed_tokens(const void* table, const void* side_table, const int32_t* tokens, const int32_t* last, PassPos pos, int64_t M,
+                  int64_t width, int64_t side_width, float* x, void* side, hipStream_t st) {
+  const bool quads = ((width | side_width) & 3) == 0;
+  const dim3 g((unsigned)std::min<int64_t>((width + side_width + 1023) / (quads ? 1024 : 256), 64), (unsigned)M);
+  if (quads)
+    hipLaunchKernelGGL((embed_tokens_kernel<T, 4>), g, dim3(256), 0, st, (const T*)table, (const T*)side_table, tokens, last, pos, width,
+                       side_width, x, (T*)side);
+  else
+    hipLaunchKernelGGL((embed_tokens_kernel<T, 1>), g, dim3(256), 0, st, (const T*)table, (const T*)side_table, tokens, last, pos, width,
+                       side_width, x, (T*)side);
+}
+
+template <typename T>
 int join(const JoinArgs& a, hipStream_t st) {
   const size_t lds = (size_t)a.width * 4;
   const bool quads = ((a.width | a.ldo | a.ldg | a.ldh) & 3) == 0;
@@ -218,13 +237,8 @@ int launch_embed_tokens(const void* table, const void* side_table, bool f32, con
                         PassPos pos, int64_t M, int64_t width, int64_t side_width, float* x, void* side, hipStream_t st) {
   AWQ_REQUIRE(table && x && (pos.dyn ? last != nullptr && M == 1 : tokens != nullptr), "bad arguments");
   AWQ_REQUIRE(M >= 1 && M <= 65535 && width >= 1 && side_width >= 0 && (side_width == 0 || (side_table && side)), "bad shape");
-  const dim3 g((unsigned)std::min<int64_t>((width + side_width + 255) / 256, 64), (unsigned)M);
-  if (f32)
-    hipLaunchKernelGGL(embed_tokens_kernel<float>, g, dim3(256), 0, st, (const float*)table, (const float*)side_table, tokens, last,
-                       pos, width, side_width, x, (float*)side);
-  else
-    hipLaunchKernelGGL(embed_tokens_kernel<bf16_t>, g, dim3(256), 0, st, (const bf16_t*)table, (const bf16_t*)side_table, tokens,
-                       last, pos, width, side_width, x, (bf16_t*)side);
+  if (f32) embed_tokens<float>(table, side_table, tokens, last, pos, M, width, side_width, x, side, st);
+  else embed_tokens<bf16_t>(table, side_table, tokens, last, pos, M, width, side_width, x, side, st);
   AWQ_HIP_TRY(hipGetLastError());
   return AWQ_OK;
 }

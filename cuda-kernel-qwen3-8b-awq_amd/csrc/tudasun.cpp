@@ -488,7 +488,7 @@ int TudasunEngine::make_activations(Buffers* b, int64_t n) {
       router = std::max<int64_t>(router, s.outputs());
       pairs = std::max<int64_t>(pairs, (int64_t)s.top * width);
       top = std::max<int64_t>(top, s.top);
-      tiles = std::max<int64_t>(tiles, route_max_tiles(n, s.top, s.experts));
+      tiles = std::max<int64_t>(tiles, route_max_tiles(n, s.top, s.experts, 64));
     }
   }
   // every buffer starts as zeros: what pads a product's inputs meets zero weights, and has to be finite
@@ -686,6 +686,7 @@ int TudasunEngine::routed_feed_forward(int i, Buffers& b, int64_t M, JoinArgs* e
     }
     if (int rc = launch_dense(a, f32, stream)) return rc;
   }
+  const int32_t tile_tokens = route_tile_tokens(M, s.top, s.outputs(), f32);
   {
     RouteArgs r;
     r.logits = b.router;
@@ -699,6 +700,7 @@ int TudasunEngine::routed_feed_forward(int i, Buffers& b, int64_t M, JoinArgs* e
     r.ids = b.ids;
     r.weights = b.weights;
     r.M = M;
+    r.tile_tokens = tile_tokens;
     r.tiles = b.tiles;
     r.list = b.list;
     if (int rc = launch_route(r, stream)) return rc;
@@ -716,7 +718,8 @@ int TudasunEngine::routed_feed_forward(int i, Buffers& b, int64_t M, JoinArgs* e
       } else {
         a->tiles = b.tiles;
         a->list = b.list;
-        a->max_tiles = route_max_tiles(M, s.top, s.experts);
+        a->max_tiles = route_max_tiles(M, s.top, s.experts, tile_tokens);
+        a->tile_tokens = tile_tokens;
         a->list_div = reads_token ? s.top : 1;
       }
     };
