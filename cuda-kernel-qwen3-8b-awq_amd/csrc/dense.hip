@@ -48,6 +48,26 @@ __device__ __forceinline__ float activate_with(const DenseSegment& s, int row, f
   return z;
 }
 
+// the same for four rows, with one look at which it is
+__device__ __forceinline__ void activate_four(const DenseSegment& s, int row, f32x4_t& v, const float (&bias)[4], const float (&lower)[4]) {
+  switch (s.act) {
+#define AWQ_ACTIVATE(ACT)                                                                      \
+  case ACT:                                                                                    \
+    _Pragma("unroll") for (int j = 0; j < 4; ++j) {                                            \
+      __builtin_assume(s.act == ACT);                                                          \
+      v[j] = activate_with<false>(s, row + j, v[j], bias[j], lower[j]);                        \
+    }                                                                                          \
+    break;
+    AWQ_ACTIVATE(DENSE_SILU)
+    AWQ_ACTIVATE(DENSE_XIELU)
+    AWQ_ACTIVATE(DENSE_SIGMOID)
+    AWQ_ACTIVATE(DENSE_GELU)
+    AWQ_ACTIVATE(DENSE_LOG_DECAY)
+    AWQ_ACTIVATE(DENSE_FORGET)
+#undef AWQ_ACTIVATE
+  }
+}
+
 template <bool F32>
 __device__ __forceinline__ float activate(const DenseSegment& s, int row, float z) {
   return activate_with<F32>(s, row, z, s.bias ? s.bias[row] : 0.0f, s.lower ? s.lower[row] : 0.0f);
@@ -325,7 +345,7 @@ __global__ __launch_bounds__(256, 2) void dense_many_kernel(DenseArgs a, int row
   __syncthreads();  // the last step's readers are done
 #pragma unroll
   for (int b = 0; b < 2; ++b) {
-    const DenseSegment& out = segment_of(a, row_w + 32 * b);
+    const DenseSegment out = segment_of(a, row_w + 32 * b);
     const int local_b = row_w + 32 * b - out.row0;
     const bool gated = OUT == DENSE_STORE && out.act == DENSE_GLU;
     const int n_rows = gated ? out.glu_rows : out.rows;
@@ -364,10 +384,7 @@ __global__ __launch_bounds__(256, 2) void dense_many_kernel(DenseArgs a, int row
         if constexpr (OUT == DENSE_PART) {
           *reinterpret_cast<f32x4_t*>(a.workspace + ((int64_t)cut * a.M + tok) * row_tiles * 256 + row_w + 32 * b + 4 * piece) = v;
         } else {
-          if (OUT == DENSE_STORE && !gated && out.act != DENSE_NONE) {
-#pragma unroll
-            for (int j = 0; j < 4; ++j) v[j] = activate_with<false>(out, row + j, v[j], bias[j], lower[j]);
-          }
+          if (OUT == DENSE_STORE && !gated) activate_four(out, row, v, bias, lower);
           const int64_t at = y0 + tok * out.ldy + row;
           if (row + 3 < n_rows && by_four) {
             if (OUT == DENSE_STORE && !out.y_f32) {
