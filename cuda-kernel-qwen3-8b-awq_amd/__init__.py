@@ -142,13 +142,16 @@ SIGNATURES["awq_gemv_fused"] = (ctypes.c_int, [ctypes.POINTER(AwqLinearArgs), _v
 class AwqDenseSegment(ctypes.Structure):
     """struct awq_dense_segment"""
     _fields_ = [("x", _vp), ("y", _vp), ("ldx", _i64), ("ldy", _i64), ("row0", _i32), ("rows", _i32), ("act", _i32),
-                ("act_rows", _i32), ("act_pos", _f32), ("act_neg", _f32)]
+                ("act_rows", _i32), ("act_pos", _f32), ("act_neg", _f32), ("y_f32", _i32), ("glu_rows", _i32), ("bias", _vp),
+                ("lower", _vp), ("mul", _vp), ("ldmul", _i64)]
 
 
 class AwqDenseArgs(ctypes.Structure):
     """struct awq_dense_args"""
     _fields_ = [("w", _vp), ("k", _i64), ("tokens", _i64), ("n_segments", _i32), ("out", _i32),
-                ("segment", AwqDenseSegment * 2), ("addend", _vp), ("workspace", _vp), ("workspace_floats", _i64)]
+                ("segment", AwqDenseSegment * 8), ("addend", _vp), ("workspace", _vp), ("workspace_floats", _i64),
+                ("w_batch", _i64), ("x_batch", _i64), ("y_batch", _i64), ("ids", _vp), ("batch", _i32), ("n_groups", _i32),
+                ("tiles", _vp), ("list", _vp), ("max_tiles", _i32), ("tile_tokens", _i32), ("list_div", _i32), ("reserved", _i32)]
 
 
 class AwqWindowArgs(ctypes.Structure):
@@ -159,7 +162,36 @@ class AwqWindowArgs(ctypes.Structure):
                 ("ldc", _i64), ("n_tokens", _i64), ("pos0", _i64), ("max_pos", _i64), ("workspace", _vp)]
 
 
-ACT_NONE, ACT_SILU, ACT_XIELU = range(3)
+class AwqGatedStateArgs(ctypes.Structure):
+    """struct awq_gated_state_args"""
+    _fields_ = [("q", _vp), ("k", _vp), ("v", _vp), ("g", _vp), ("ldp", _i64), ("ldg", _i64), ("heads", _i32), ("dim", _i32),
+                ("vdim", _i32), ("q_scale", _f32), ("state", _vp), ("o", _vp), ("n_tokens", _i64), ("pos0", _i64), ("norm", _vp),
+                ("gate", _vp), ("ctx", _vp), ("eps", _f32), ("reserved", _f32)]
+
+
+class AwqLatentArgs(ctypes.Structure):
+    """struct awq_latent_args"""
+    _fields_ = [("q", _vp), ("ldq", _i64), ("down", _vp), ("ldd", _i64), ("norm", _vp), ("freq", _vp), ("sink", _vp),
+                ("heads", _i32), ("dim", _i32), ("vdim", _i32), ("rank", _i32), ("rot", _i32), ("scale", _f32), ("eps", _f32),
+                ("reserved", _i32), ("cache", _vp), ("w_uk", _vp), ("w_uv", _vp), ("w_kv", _vp), ("ctx", _vp), ("ldc", _i64),
+                ("n_tokens", _i64), ("pos0", _i64), ("max_pos", _i64), ("qa", _vp), ("ql", _vp), ("ol", _vp), ("kv", _vp),
+                ("parts", _vp)]
+
+
+class AwqLatentBytes(ctypes.Structure):
+    """struct awq_latent_bytes"""
+    _fields_ = [(n, _i64) for n in ("w_uk", "w_uv", "w_kv", "qa", "ql", "ol", "kv", "parts")]
+
+
+class AwqJoinArgs(ctypes.Structure):
+    """struct awq_join_args"""
+    _fields_ = [("x", _vp), ("n_tokens", _i64), ("width", _i64), ("eps", _f32), ("top", _i32), ("experts", _i32), ("reserved", _i32),
+                ("y", _vp), ("y_gate", _vp), ("pairs", _vp), ("ids", _vp), ("weights", _vp), ("h", _vp), ("ldh", _i64), ("gate", _vp),
+                ("ldg", _i64), ("w_post", _vp), ("w_next", _vp), ("out", _vp), ("ldo", _i64)]
+
+
+(ACT_NONE, ACT_SILU, ACT_XIELU, ACT_SIGMOID, ACT_GELU, ACT_GLU, ACT_SOFTCAP, ACT_LOG_DECAY, ACT_FORGET) = range(9)
+PACK_PLAIN, PACK_GATE, PACK_UP, PACK_TRANSPOSED = range(4)
 DENSE_STORE, DENSE_RESIDUAL, DENSE_F32 = range(3)
 SIGNATURES.update({
     "awq_dense_weight_bytes": (_i64, [_i64, _i64, _i32]),
@@ -172,6 +204,17 @@ SIGNATURES.update({
     "awq_window_row": (_i32, [_i32]),
     "awq_window_workspace_floats": (_i64, [_i32, _i32, _i64, _i64]),
     "awq_window_attention": (ctypes.c_int, [ctypes.POINTER(AwqWindowArgs), _i32, _vp]),
+    "awq_dense_pack_form": (ctypes.c_int, [_vp, _i32, _i64, _i64, _vp, _i64, _i64, _i64, _i32, _i32, _vp]),
+    "awq_gated_state": (ctypes.c_int, [ctypes.POINTER(AwqGatedStateArgs), _i32, _vp]),
+    "awq_head_norm": (ctypes.c_int, [_vp, _vp, _i64, _vp, _vp, _i64, _i32, _i32, _i64, _f32, _i32, _vp]),
+    "awq_latent_row": (_i32, [_i32, _i32]),
+    "awq_latent_sizes": (ctypes.c_int, [ctypes.POINTER(AwqLatentArgs), _i64, _i32, ctypes.POINTER(AwqLatentBytes)]),
+    "awq_latent_pack": (ctypes.c_int, [ctypes.POINTER(AwqLatentArgs), _vp, _vp, _i32, _vp]),
+    "awq_latent_attention": (ctypes.c_int, [ctypes.POINTER(AwqLatentArgs), _i32, _vp]),
+    "awq_route_max_tiles": (_i32, [_i64, _i32, _i32, _i32]),
+    "awq_route": (ctypes.c_int, [_vp, _i64, _vp, _i32, _i32, _i32, _i32, _i32, _i64, _vp, _vp, _i32, _vp, _vp, _vp]),
+    "awq_join": (ctypes.c_int, [ctypes.POINTER(AwqJoinArgs), _i32, _vp]),
+    "awq_polynorm": (ctypes.c_int, [_vp, _i64, _i64, _i64, _vp, _f32, _i32, _vp]),
     "awq_linear_attention": (ctypes.c_int, [_vp, _i64, _i32, _i32, _i32, _vp, _vp, _vp, _vp, _i64, _i64, _i32, _vp]),
 })
 

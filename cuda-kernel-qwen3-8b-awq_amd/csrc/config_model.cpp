@@ -90,13 +90,9 @@ int Loader::table(const std::string& name, void** out) {
   return launch_convert(staging, wide(t), *out, e->f32, n, e->stream);
 }
 int Loader::matrix(const std::string& name, void* w, int64_t k, int64_t row0, int64_t col0, int form) {
-  return matrix_rows(name, 0, file.find(name)->shape[0], w, k, row0, col0, form);
-}
-int Loader::matrix_rows(const std::string& name, int64_t first, int64_t n, void* w, int64_t k, int64_t row0, int64_t col0, int form) {
   const Tensor* t = file.find(name);
   if (int rc = stage(t)) return rc;
-  const char* src = (const char*)staging + first * t->shape[1] * (wide(t) ? 4 : 2);
-  return launch_dense_pack(src, wide(t), n, t->shape[1], w, k, row0, col0, e->f32, e->stream, form);
+  return launch_dense_pack(staging, wide(t), t->shape[0], t->shape[1], w, k, row0, col0, e->f32, e->stream, form);
 }
 int Loader::block(void** w, int64_t n, int64_t k) { return e->zeroed(w, dense_weight_bytes(n, k, e->f32)); }
 int Loader::constants(const std::vector<float>& v, const float** out) {

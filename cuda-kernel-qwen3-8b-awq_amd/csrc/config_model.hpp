@@ -31,9 +31,6 @@ struct Loader {
   int table(const std::string& name, void** out);                             // in the activations' type
   // into rows row0.., inputs col0.. of a block of padded inputs k
   int matrix(const std::string& name, void* w, int64_t k, int64_t row0, int64_t col0, int form = PACK_PLAIN);
-  // rows first .. first + rows - 1 of the matrix
-  int matrix_rows(const std::string& name, int64_t first, int64_t rows, void* w, int64_t k, int64_t row0, int64_t col0,
-                  int form = PACK_PLAIN);
   int block(void** w, int64_t rows, int64_t k);  // zeroed
   int constants(const std::vector<float>& v, const float** out);
   int constants(const std::vector<double>& v, const double** out);

@@ -596,6 +596,26 @@ LatentScratch latent_scratch(const LatentAttnArgs& a, int64_t max_tokens, bool f
   return s;
 }
 
+int launch_latent_pack(const LatentAttnArgs& a, const void* uk, const void* uv, bool src_f32, void* w_uk, void* w_uv, void* w_kv,
+                       bool f32, hipStream_t st) {
+  const int64_t qk = q_inputs(a), vk = v_inputs(a), unit = src_f32 ? 4 : 2, keys = (int64_t)a.heads * a.dim;
+  const int64_t uk_rows = latent_uk_block(a) / qk, uv_rows = latent_uv_block(a) / vk;
+  for (int64_t h = 0; h < a.heads; ++h) {
+    if (uk)
+      if (int rc = launch_dense_pack((const char*)uk + h * a.dim * a.l.rank * unit, src_f32, a.dim, a.l.rank, w_uk, qk, h * uk_rows, 0,
+                                     f32, st, PACK_TRANSPOSED))
+        return rc;
+    if (uv)
+      if (int rc = launch_dense_pack((const char*)uv + h * a.vdim * a.l.rank * unit, src_f32, a.vdim, a.l.rank, w_uv, vk, h * uv_rows, 0,
+                                     f32, st))
+        return rc;
+  }
+  if (w_kv && uk)
+    if (int rc = launch_dense_pack(uk, src_f32, keys, a.l.rank, w_kv, vk, 0, 0, f32, st)) return rc;
+  if (w_kv && uv) return launch_dense_pack(uv, src_f32, (int64_t)a.heads * a.vdim, a.l.rank, w_kv, vk, keys, 0, f32, st);
+  return AWQ_OK;
+}
+
 int launch_latent_attention(const LatentAttnArgs& a, bool f32, hipStream_t st) {
   AWQ_REQUIRE(a.q && a.freq && a.cache && a.w_uk && a.w_uv && a.ctx && a.qa && a.ql && a.ol && (!a.down || a.norm), "bad arguments");
   AWQ_REQUIRE(a.heads >= 1 && a.heads <= 65535 && a.dim >= 1 && a.vdim >= 1 && a.l.rank >= 1 && a.l.rank <= 256 * kMaxColsPerThread &&
@@ -604,7 +624,8 @@ int launch_latent_attention(const LatentAttnArgs& a, bool f32, hipStream_t st) {
   AWQ_REQUIRE(a.M >= 1 && a.M <= 65535 && a.M * a.heads < (1ll << 30) && a.ldq >= (int64_t)a.heads * (a.dim + a.l.rot) &&
                   (a.pos.dyn ? a.M == 1 : a.pos.pos0 + a.M <= a.max_pos),
               "bad tokens");
-  if (can_form(a, f32) && a.w_kv && a.kv && !a.pos.dyn && a.M >= form_from(a) && ((a.ldq | a.ldc) & 7) == 0) {
+  if (can_form(a, f32) && !a.pos.dyn && a.M >= form_from(a)) {
+    AWQ_REQUIRE(a.w_kv && a.kv && ((a.ldq | a.ldc) & 7) == 0, "a pass of this many tokens forms keys and values: w_kv, kv, rows of 8");
     if (int rc = launch_prepare<bf16_t, false>(a, st)) return rc;
     DenseArgs d;
     d.w = a.w_kv;

@@ -279,6 +279,10 @@ LatentScratch latent_scratch(const LatentAttnArgs& a, int64_t max_tokens, bool f
 int64_t latent_uk_block(const LatentAttnArgs& a);  // elements between heads of w_uk
 int64_t latent_uv_block(const LatentAttnArgs& a);  // ... of w_uv
 int64_t latent_kv_rows(const LatentAttnArgs& a);   // padded rows of w_kv
+// W_uk [heads * dim][rank] and W_uv [heads * vdim][rank] on the device into the zeroed blocks (either source may be null: it
+// is left out; w_kv may be null)
+int launch_latent_pack(const LatentAttnArgs& a, const void* uk, const void* uv, bool src_f32, void* w_uk, void* w_uv, void* w_kv,
+                       bool f32, hipStream_t st);
 int launch_latent_attention(const LatentAttnArgs& a, bool f32, hipStream_t st);
 
 // --- routed feed-forward (experts.hip) ---------------------------------------------------------------------------

@@ -379,17 +379,17 @@ int TudasunEngine::load_layer(Loader& ldr, int i) {
   if (s.type == MIX_LATENT) {
     LatentAttnArgs a = latent_args(i);
     const int64_t qk = round_up(s.dim, kDenseKAlign), vk = round_up(s.rank, kDenseKAlign);
-    const int64_t uk_rows = latent_uk_block(a) / qk, uv_rows = latent_uv_block(a) / vk;
-    if (int rc = ldr.block(&L.w_uk, s.heads * uk_rows, qk)) return rc;
-    if (int rc = ldr.block(&L.w_uv, s.heads * uv_rows, vk)) return rc;
-    for (int h = 0; h < s.heads; ++h) {
-      if (int rc = ldr.matrix_rows(m + "uk", (int64_t)h * s.dim, s.dim, L.w_uk, qk, h * uk_rows, 0, PACK_TRANSPOSED)) return rc;
-      if (int rc = ldr.matrix_rows(m + "uv", (int64_t)h * s.vdim, s.vdim, L.w_uv, vk, h * uv_rows, 0)) return rc;
-    }
-    if (latent_forms_keys(a, pass_tokens, f32)) {
+    if (int rc = ldr.block(&L.w_uk, s.heads * latent_uk_block(a) / qk, qk)) return rc;
+    if (int rc = ldr.block(&L.w_uv, s.heads * latent_uv_block(a) / vk, vk)) return rc;
+    if (latent_forms_keys(a, pass_tokens, f32))
       if (int rc = ldr.block(&L.w_kv, latent_kv_rows(a), vk)) return rc;
-      if (int rc = ldr.matrix(m + "uk", L.w_kv, vk, 0, 0)) return rc;
-      if (int rc = ldr.matrix(m + "uv", L.w_kv, vk, keys, 0)) return rc;
+    for (const char* name : {"uk", "uv"}) {
+      const Tensor* t = ldr.file.find(m + name);
+      if (int rc = ldr.stage(t)) return rc;
+      const bool k = name[1] == 'k';
+      if (int rc = launch_latent_pack(a, k ? ldr.staging : nullptr, k ? nullptr : ldr.staging, Loader::wide(t), L.w_uk, L.w_uv, L.w_kv,
+                                      f32, stream))
+        return rc;
     }
     if (int rc = ldr.vector(m + "sink", &L.sink)) return rc;
     std::vector<double> freq;

@@ -451,13 +451,25 @@ int awq_embed_gather(const void* packed, const void* scale, const void* zp, int6
  * ------------------------------------------------------------------------- */
 
 /* Dense products y[t][r] = act(sum_k w[r][k] x[t][k]) of one weight block whose
- * rows form one or two segments, each with its own input and output.  A block
- * has rows padded to a multiple of 256 per segment and k padded with zeros to a
- * multiple of 64 (both chosen by the caller, who zero-fills the block, then
- * packs each matrix [rows][cols] into it with awq_dense_pack). */
+ * rows form segments, each with its own output.  A block has a multiple of 256
+ * rows and k padded with zeros to a multiple of 64 (both chosen by the caller,
+ * who zero-fills the block, then packs each matrix [rows][cols] into it with
+ * awq_dense_pack); a segment starts at a multiple of 256 rows, or of 32 where it
+ * has the input of the segment ahead of it. */
 #define AWQ_ACT_NONE 0
 #define AWQ_ACT_SILU 1  /* z * sigmoid(z) on the first act_rows rows of the segment */
 #define AWQ_ACT_XIELU 2 /* z > 0: act_pos z^2 + z/2; z <= 0: act_neg (exp(z) - 1 - z) + z/2 */
+#define AWQ_ACT_SIGMOID 3   /* sigmoid(z + bias) */
+#define AWQ_ACT_GELU 4      /* z/2 (1 + tanh(sqrt(2/pi) (z + 0.044715 z^3))), times mul[token][row] if mul is set */
+#define AWQ_ACT_GLU 5       /* silu(gate) * up: glu_rows outputs, packed by AWQ_PACK_GATE and AWQ_PACK_UP, rows = 2 * (glu_rows padded to 8) */
+#define AWQ_ACT_SOFTCAP 6   /* act_pos * tanh(z / act_pos) (AWQ_DENSE_F32) */
+#define AWQ_ACT_LOG_DECAY 7 /* act_pos * ln(sigmoid(z + bias)) */
+#define AWQ_ACT_FORGET 8    /* (1 - lower) * (1 - sigmoid(z + bias)) */
+#define AWQ_PACK_PLAIN 0
+#define AWQ_PACK_GATE 1
+#define AWQ_PACK_UP 2
+#define AWQ_PACK_TRANSPOSED 3 /* rows and columns exchanged */
+#define AWQ_DENSE_SEGMENTS 8
 #define AWQ_DENSE_STORE 0    /* y in the activations' type */
 #define AWQ_DENSE_RESIDUAL 1 /* y is float: y = (y + sum) + addend (may be NULL) */
 #define AWQ_DENSE_F32 2      /* y is float */
@@ -468,19 +480,41 @@ typedef struct awq_dense_segment {
   int32_t row0, rows; /* row0 a multiple of 256 */
   int32_t act, act_rows;
   float act_pos, act_neg;
+  int32_t y_f32; /* AWQ_DENSE_STORE: y is float */
+  int32_t glu_rows;
+  const float* bias;
+  const float* lower;
+  const void* mul; /* [tokens][ldmul] in the activations' type */
+  int64_t ldmul;
 } awq_dense_segment;
+/* a run of a token list that one weight block is applied to: entries first .. first + count - 1 */
+typedef struct awq_dense_tile {
+  int32_t group, first, count;
+} awq_dense_tile;
 typedef struct awq_dense_args {
   const void* w;
   int64_t k, tokens;
   int32_t n_segments, out;
-  awq_dense_segment segment[2];
+  awq_dense_segment segment[AWQ_DENSE_SEGMENTS];
   const float* addend;
   float* workspace; /* NULL, or workspace_floats of scratch for products that are cut along k */
   int64_t workspace_floats;
+  /* AWQ_DENSE_STORE: `batch` products (0 counts as 1), weight block, input and output w_batch, x_batch and y_batch elements
+   * apart; one token: product b takes block ids[b] (device) and is left out where that is not below n_groups (ids NULL: b) */
+  int64_t w_batch, x_batch, y_batch;
+  const int32_t* ids;
+  int32_t batch, n_groups;
+  /* AWQ_DENSE_STORE, many tokens: max_tiles runs (device; count 0: none) of at most tile_tokens entries of `list` (device);
+   * entry p reads input row p / list_div and writes output row p, with weight block `group` */
+  const awq_dense_tile* tiles;
+  const int32_t* list;
+  int32_t max_tiles, tile_tokens, list_div, reserved;
 } awq_dense_args;
 int64_t awq_dense_weight_bytes(int64_t rows_padded, int64_t k_padded, int32_t f32);
 int awq_dense_pack(const void* src, int32_t src_f32, int64_t rows, int64_t cols, void* w, int64_t k_padded, int64_t row0,
                    int64_t col0, int32_t f32, void* stream);
+int awq_dense_pack_form(const void* src, int32_t src_f32, int64_t rows, int64_t cols, void* w, int64_t k_padded, int64_t row0,
+                        int64_t col0, int32_t form, int32_t f32, void* stream);
 int awq_dense(const awq_dense_args* args, int32_t f32, void* stream);
 
 /* x[t][i] = table[tokens[t]][i] * scale + (i even: sin, odd: cos)(position *
@@ -536,6 +570,103 @@ int awq_window_attention(const awq_window_args* args, int32_t f32, void* stream)
 int awq_linear_attention(const void* proj, int64_t ldp, int32_t heads, int32_t dim, int32_t vdim, const float* decay,
                          const float* log2_decay, float* state, float* o, int64_t n_tokens, int64_t pos0, int32_t f32,
                          void* stream);
+
+/* Linear attention whose state decays per channel: per head
+ * S <- diag(decay) S + k v^T, o = S^T (q_scale q); state as above.  q, v
+ * [n_tokens][ldp]; g [n_tokens][ldg] float: with k the binary logarithms of the
+ * decays, with k NULL the numbers 1 - decay, which are the keys then.  One token
+ * with ctx != NULL: ctx instead of o, the norm of awq_head_norm in the same launch. */
+typedef struct awq_gated_state_args {
+  const void *q, *k, *v;
+  const float* g;
+  int64_t ldp, ldg;
+  int32_t heads, dim, vdim;
+  float q_scale;
+  float* state;
+  float* o;
+  int64_t n_tokens, pos0;
+  const float* norm;
+  const void* gate;
+  void* ctx;
+  float eps, reserved;
+} awq_gated_state_args;
+int awq_gated_state(const awq_gated_state_args* args, int32_t f32, void* stream);
+/* ctx[t][h][c] = RMS norm over each head's vdim values of o, times w [vdim], times silu(gate) (gate NULL: 1) */
+int awq_head_norm(const float* o, const void* gate, int64_t ldg, const float* w, void* ctx, int64_t ldc, int32_t heads,
+                  int32_t vdim, int64_t n_tokens, float eps, int32_t f32, void* stream);
+
+/* Attention over a shared latent for n_tokens new positions pos0..: the score of
+ * query head h with a position is (q . W_uk[h] c + q_rot . k_rot) * scale, the
+ * value W_uv[h] c, softmax with exp(sink[h]) in the denominator (sink NULL: not).
+ * q [n_tokens][ldq]: heads of dim unrotated, then rot rotated values (pairs 2 i, 2 i + 1
+ * by position * freq[i], freq binary64; changed in place by passes of many tokens).  down [n_tokens][ldd] float:
+ * latent (normalised with `norm` before it is cached) and key part; NULL: the cache
+ * already has these positions.  cache: rows of awq_latent_row(rank, rot) elements, max_pos
+ * of them rounded up to 64.  Weights packed by awq_latent_pack into the three blocks of
+ * awq_latent_sizes; scratch as awq_latent_sizes says. */
+typedef struct awq_latent_args {
+  void* q;
+  int64_t ldq;
+  const float* down;
+  int64_t ldd;
+  const float* norm;
+  const double* freq;
+  const float* sink;
+  int32_t heads, dim, vdim, rank, rot;
+  float scale, eps;
+  int32_t reserved;
+  void* cache;
+  const void *w_uk, *w_uv, *w_kv;
+  void* ctx;
+  int64_t ldc, n_tokens, pos0, max_pos;
+  void *qa, *ql, *ol, *kv;
+  float* parts;
+} awq_latent_args;
+/* bytes of w_uk, w_uv, w_kv and of the scratch qa, ql, ol, kv, parts for passes of up to max_tokens tokens (w_kv and kv 0:
+ * no such pass forms keys and values) */
+typedef struct awq_latent_bytes {
+  int64_t w_uk, w_uv, w_kv, qa, ql, ol, kv, parts;
+} awq_latent_bytes;
+int32_t awq_latent_row(int32_t rank, int32_t rot);
+int awq_latent_sizes(const awq_latent_args* args, int64_t max_tokens, int32_t f32, awq_latent_bytes* out);
+/* W_uk [heads * dim][rank], W_uv [heads * vdim][rank], bfloat16 on the device, into the zero-filled blocks */
+int awq_latent_pack(const awq_latent_args* args, const void* uk, const void* uv, int32_t f32, void* stream);
+int awq_latent_attention(const awq_latent_args* args, int32_t f32, void* stream);
+
+/* Router: softmax of a token's `outputs` logits, choice of `top` by score + correction among the outputs of the `keep` of
+ * `groups` equal groups with the largest choice score (groups 0: all), weights = chosen scores over their sum.  Outputs from
+ * `experts` on have no weights of their own.  More than one token: tiles [awq_route_max_tiles] and list [n_tokens * top]
+ * receive the plan of the experts' products (awq_dense_args), entry t * top + j being token t's j-th choice. */
+int32_t awq_route_max_tiles(int64_t n_tokens, int32_t top, int32_t experts, int32_t tile_tokens);
+int awq_route(const float* logits, int64_t ld, const float* correction, int32_t outputs, int32_t experts, int32_t top,
+              int32_t groups, int32_t keep, int64_t n_tokens, int32_t* ids, float* weights, int32_t tile_tokens,
+              awq_dense_tile* tiles, int32_t* list, void* stream);
+
+/* The end of a sublayer, x += RMS norm(s * gate) * w_post with s = y * sigmoid(y_gate) + the weighted experts' outputs
+ * (pairs, or h for outputs from `experts` on); out = RMS norm(x) * w_next, or x (w_next NULL).  Anything may be NULL but x,
+ * w_post and one of y and pairs. */
+typedef struct awq_join_args {
+  float* x;
+  int64_t n_tokens, width;
+  float eps;
+  int32_t top, experts, reserved;
+  const float* y;
+  const float* y_gate;
+  const float* pairs;
+  const int32_t* ids;
+  const float* weights;
+  const void* h;
+  int64_t ldh;
+  const void* gate;
+  int64_t ldg;
+  const float* w_post;
+  const float* w_next;
+  void* out;
+  int64_t ldo;
+} awq_join_args;
+int awq_join(const awq_join_args* args, int32_t f32, void* stream);
+/* z <- a N(z) + b N(z^2) + c N(z^3) + e in place, N the division of a token's n values by their root mean square */
+int awq_polynorm(void* z, int64_t ld, int64_t n, int64_t n_tokens, const float* abce, float eps, int32_t f32, void* stream);
 
 #ifdef __cplusplus
 }
