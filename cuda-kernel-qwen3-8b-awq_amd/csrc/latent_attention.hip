@@ -16,53 +16,43 @@ __device__ __forceinline__ float wave_sum(float v) {
 }
 
 // --- queries and cache rows ----------------------------------------------------------------------------------
-// blockIdx.x: token, blockIdx.y: kPrepareHeads heads, and behind the last heads the token's cache row.  Angles are brought
-// into [-pi, pi] in binary64.  INTO: the unrotated parts go to qa, padded to `kq` inputs a head, the rotated ones to their
-// place in ql; otherwise the rotated parts are rotated in place.
-constexpr int kPrepareHeads = 4;
-
-template <typename T, bool INTO>
-__global__ __launch_bounds__(256) void latent_prepare_kernel(LatentAttnArgs a, int kq) {
-  extern __shared__ float turn[];  // [rot / 2][2]: cosine, sine
-  __shared__ float sums[4];
-  const int tid = threadIdx.x, t = blockIdx.x, pos = a.pos.position() + t;
-  const int rot = a.l.rot, rank = a.l.rank, rp = a.l.rank_padded(), row = a.l.row();
-  for (int i = tid; 2 * i < rot; i += 256) {
+// turn[rot / 2][2]: cosine and sine of the position's angles, brought into [-pi, pi] in binary64
+__device__ __forceinline__ void turns_of(const LatentAttnArgs& a, int pos, float* turn) {
+  for (int i = threadIdx.x; 2 * i < a.l.rot; i += 256) {
     const double turns = (double)pos * a.freq[i] * 0.15915494309189533577;  // 1 / 2 pi
     const float x = (float)((turns - rint(turns)) * 6.28318530717958647693);
     turn[2 * i] = cosf(x);
     turn[2 * i + 1] = sinf(x);
   }
   __syncthreads();
-  const int h0 = blockIdx.y * kPrepareHeads;
-  if (h0 < a.heads) {
-    const int nh = min(kPrepareHeads, a.heads - h0);
-    T* const q = reinterpret_cast<T*>(a.q) + t * a.ldq + (int64_t)h0 * (a.dim + rot);
-    if constexpr (INTO) {
-      T* const qa = reinterpret_cast<T*>(a.qa) + ((int64_t)t * a.heads + h0) * kq;
-      for (int i = tid; i < nh * kq; i += 256) {
-        const int h = i / kq, d = i - h * kq;
-        qa[i] = d < a.dim ? q[(int64_t)h * (a.dim + rot) + d] : (T)0.0f;
-      }
+}
+
+// `nh` heads' rotated parts, the first head's values at q.  INTO: to their place behind the latent entries of the queries
+// ql, with zeros around them (entries rank .. row - 1); otherwise in place.
+template <typename T, bool INTO>
+__device__ __forceinline__ void rotate_queries(const LatentAttnArgs& a, T* q, T* ql, int nh, const float* turn) {
+  const int rot = a.l.rot, rank = a.l.rank, rp = a.l.rank_padded(), row = a.l.row();
+  const int tail = INTO ? row - rank : rot, skip = INTO ? rp - rank : 0;
+  for (int i = threadIdx.x; i < nh * tail; i += 256) {
+    const int h = i / tail, e = i - h * tail - skip;
+    T* const src = q + (int64_t)h * (a.dim + rot) + a.dim;
+    T* const dst = ql + (int64_t)h * row + rp;
+    if (e >= 0 && e < rot) {
+      if (e & 1) continue;
+      const float u = (float)src[e], v = (float)src[e + 1], c = turn[e], s = turn[e + 1];
+      T* const out = INTO ? dst : src;
+      out[e] = (T)(u * c - v * s);
+      out[e + 1] = (T)(v * c + u * s);
+    } else if constexpr (INTO) {
+      dst[e] = (T)0.0f;
     }
-    // entries rank .. row - 1 of a query in the latent space: zeros, the rotated pairs, zeros
-    const int tail = INTO ? row - rank : rot, skip = INTO ? rp - rank : 0;
-    for (int i = tid; i < nh * tail; i += 256) {
-      const int h = i / tail, e = i - h * tail - skip;
-      T* const src = q + (int64_t)h * (a.dim + rot) + a.dim;
-      T* const dst = reinterpret_cast<T*>(a.ql) + ((int64_t)t * a.heads + h0 + h) * row + rp;
-      if (e >= 0 && e < rot) {
-        if (e & 1) continue;
-        const float u = (float)src[e], v = (float)src[e + 1], c = turn[e], s = turn[e + 1];
-        T* const out = INTO ? dst : src;
-        out[e] = (T)(u * c - v * s);
-        out[e + 1] = (T)(v * c + u * s);
-      } else if constexpr (INTO) {
-        dst[e] = (T)0.0f;
-      }
-    }
-    return;
   }
+}
+
+// the cache row of token t of the pass
+template <typename T>
+__device__ __forceinline__ void append_row(const LatentAttnArgs& a, int t, int pos, const float* turn, float (&sums)[4]) {
+  const int tid = threadIdx.x, rot = a.l.rot, rank = a.l.rank, rp = a.l.rank_padded(), row = a.l.row();
   const float* const d = a.down + t * a.ldd;
   float sq = 0.0f;
   for (int i = tid; i < rank; i += 256) sq = __builtin_fmaf(d[i], d[i], sq);
@@ -81,6 +71,77 @@ __global__ __launch_bounds__(256) void latent_prepare_kernel(LatentAttnArgs a, i
       v = e & 1 ? x * cs + other * sn : x * cs - other * sn;
     }
     c[i] = (T)v;
+  }
+}
+
+// blockIdx.x: token, blockIdx.y: kPrepareHeads heads, and behind the last heads the token's cache row.  INTO: the
+// unrotated parts go to qa, padded to `kq` inputs a head, the rotated ones to their place in ql; otherwise the rotated parts
+// are rotated in place.
+constexpr int kPrepareHeads = 4;
+
+template <typename T, bool INTO>
+__global__ __launch_bounds__(256) void latent_prepare_kernel(LatentAttnArgs a, int kq) {
+  extern __shared__ float turn[];
+  __shared__ float sums[4];
+  const int t = blockIdx.x, pos = a.pos.position() + t;
+  turns_of(a, pos, turn);
+  const int h0 = blockIdx.y * kPrepareHeads;
+  if (h0 >= a.heads) {
+    append_row<T>(a, t, pos, turn, sums);
+    return;
+  }
+  const int nh = min(kPrepareHeads, a.heads - h0);
+  T* const q = reinterpret_cast<T*>(a.q) + t * a.ldq + (int64_t)h0 * (a.dim + a.l.rot);
+  if constexpr (INTO) {
+    T* const qa = reinterpret_cast<T*>(a.qa) + ((int64_t)t * a.heads + h0) * kq;
+    for (int i = threadIdx.x; i < nh * kq; i += 256) {
+      const int h = i / kq, d = i - h * kq;
+      qa[i] = d < a.dim ? q[(int64_t)h * (a.dim + a.l.rot) + d] : (T)0.0f;
+    }
+  }
+  rotate_queries<T, INTO>(a, q, reinterpret_cast<T*>(a.ql) + ((int64_t)t * a.heads + h0) * a.l.row(), nh, turn);
+}
+
+// One token: the same and the product with W_uk in one launch.  blockIdx.x: head, blockIdx.y: 64 of its latent entries, 16 a
+// wavefront (the first such workgroup of a head rotates, one more of the first head appends the cache row);
+// v_mfma_f32_16x16x32_bf16 with the query in every column.
+__global__ __launch_bounds__(256) void latent_query_one_kernel(LatentAttnArgs a, int64_t w_block, int chunks) {
+  extern __shared__ float turn[];
+  __shared__ float sums[4];
+  const int h = blockIdx.x, part = blockIdx.y, pos = a.pos.position();
+  if (part == chunks) {
+    if (h != 0) return;
+    turns_of(a, pos, turn);
+    append_row<bf16_t>(a, 0, pos, turn, sums);
+    return;
+  }
+  const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), r = lane & 15, c = lane >> 4;
+  const int row0 = part * 64 + wave * 16, rank = a.l.rank;
+  bf16_t* const q = reinterpret_cast<bf16_t*>(a.q) + (int64_t)h * (a.dim + a.l.rot);
+  bf16_t* const ql = reinterpret_cast<bf16_t*>(a.ql) + (int64_t)h * a.l.row();
+  if (row0 < rank) {
+    const bf16x8_t* w = reinterpret_cast<const bf16x8_t*>(reinterpret_cast<const bf16_t*>(a.w_uk) + h * w_block) +
+                        ((int64_t)(row0 >> 5) * (a.dim >> 4) + (c >> 1)) * 64 + 32 * (c & 1) + (row0 & 16) + r;
+    const bf16x8_t* x = reinterpret_cast<const bf16x8_t*>(q) + c;
+    f32x4_t acc = {0.0f, 0.0f, 0.0f, 0.0f};
+    constexpr int U = 8;
+    const int steps = a.dim >> 5;
+    bf16x8_t wv[U], xv[U];
+#pragma unroll
+    for (int i = 0; i < U; ++i)
+      if (i < steps) wv[i] = w[(int64_t)i * 128], xv[i] = x[i * 4];
+#pragma unroll
+    for (int i = 0; i < U; ++i)
+      if (i < steps) acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wv[i], xv[i], acc, 0, 0, 0);
+    for (int i = U; i < steps; ++i) acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(w[(int64_t)i * 128], x[i * 4], acc, 0, 0, 0);
+    if (r == 0)
+#pragma unroll
+      for (int j = 0; j < 4; ++j)
+        if (row0 + 4 * c + j < rank) ql[row0 + 4 * c + j] = (bf16_t)acc[j];
+  }
+  if (part == 0) {
+    turns_of(a, pos, turn);
+    rotate_queries<bf16_t, true>(a, q, ql, 1, turn);
   }
 }
 
@@ -315,36 +376,86 @@ __global__ __launch_bounds__(256) void latent_rows_kernel(LatentAttnArgs a) {
   }
 }
 
-// a workgroup per query row: the parts and the sink
-__global__ __launch_bounds__(256) void latent_combine_kernel(LatentAttnArgs a, int parts, int kv_in) {
-  __shared__ float scale[kMaxParts];
-  const int r = blockIdx.x, tid = threadIdx.x, lane = tid & 63;
-  const int ps = a.l.rank_padded() + 4, rank = a.l.rank;
+// The parts of query row r and the sink: `scale` receives every part's factor; returns what the weighted parts are divided by
+__device__ __forceinline__ float combine_factors(const LatentAttnArgs& a, int r, int parts, float* scale, int* used_parts) {
+  const int tid = threadIdx.x, lane = tid & 63, ps = a.l.rank_padded() + 4;
   int tiles;
   const int per = tiles_per_part(r / kRows * kRows, (int)a.M * a.heads, a.heads, a.pos.position(), parts, &tiles);
   const int used = (tiles + per - 1) / per;
   const float* const p = a.parts + (int64_t)r * parts * ps;
   const float sink = a.sink ? a.sink[r % a.heads] * kLog2e : -INFINITY;
-  float m = sink, l = 0.0f;
-  for (int s = lane; s < used; s += 64) m = fmaxf(m, p[(int64_t)s * ps]);
+  float pm[kMaxParts / 64], pl[kMaxParts / 64], m = sink, l = 0.0f;
+#pragma unroll
+  for (int i = 0; i < kMaxParts / 64; ++i) {
+    const int s = lane + 64 * i;
+    pm[i] = s < used ? p[(int64_t)s * ps] : -INFINITY;
+    pl[i] = s < used ? p[(int64_t)s * ps + 1] : 0.0f;
+    m = fmaxf(m, pm[i]);
+  }
 #pragma unroll
   for (int off = 32; off > 0; off >>= 1) m = fmaxf(m, __shfl_xor(m, off, 64));
-  for (int s = lane; s < used; s += 64) {
-    const float e = exp2f(p[(int64_t)s * ps] - m);
-    l = __builtin_fmaf(e, p[(int64_t)s * ps + 1], l);
-    if (tid < 64) scale[s] = e;
+#pragma unroll
+  for (int i = 0; i < kMaxParts / 64; ++i) {
+    const float e = exp2f(pm[i] - m);
+    l = __builtin_fmaf(e, pl[i], l);
+    if (tid < 64) scale[lane + 64 * i] = e;
   }
   l = wave_sum(l) + exp2f(sink - m);
   __syncthreads();
-  const float inv = 1.0f / l;
-  bf16_t* const out = reinterpret_cast<bf16_t*>(a.ol) + (int64_t)r * kv_in;
-  for (int c = tid; c < kv_in; c += 256) {
-    float v = 0.0f;
-    if (c < rank)
+  *used_parts = used;
+  return l;
+}
+__device__ __forceinline__ float combine_column(const LatentAttnArgs& a, int r, int parts, const float* scale, int used, int c) {
+  const int ps = a.l.rank_padded() + 4;
+  const float* const p = a.parts + (int64_t)r * parts * ps + 4 + c;
+  float v = 0.0f;
 #pragma unroll 8
-      for (int s = 0; s < used; ++s) v = __builtin_fmaf(scale[s], p[(int64_t)s * ps + 4 + c], v);
-    out[c] = (bf16_t)(v * inv);
-  }
+  for (int s = 0; s < used; ++s) v = __builtin_fmaf(scale[s], p[(int64_t)s * ps], v);
+  return v;
+}
+
+// a workgroup per query row
+__global__ __launch_bounds__(256) void latent_combine_kernel(LatentAttnArgs a, int parts, int kv_in) {
+  __shared__ float scale[kMaxParts];
+  const int r = blockIdx.x;
+  int used;
+  const float inv = 1.0f / combine_factors(a, r, parts, scale, &used);
+  bf16_t* const out = reinterpret_cast<bf16_t*>(a.ol) + (int64_t)r * kv_in;
+  for (int c = threadIdx.x; c < kv_in; c += 256) out[c] = (bf16_t)(c < a.l.rank ? combine_column(a, r, parts, scale, used, c) * inv : 0.0f);
+}
+
+// One token: the same and the product with W_uv in one launch.  blockIdx.x: head, blockIdx.y: 64 of its values, 16 a
+// wavefront; every workgroup combines for itself while its weights are on their way.
+__global__ __launch_bounds__(256) void latent_value_one_kernel(LatentAttnArgs a, int parts, int kv_in, int64_t w_block) {
+  extern __shared__ __attribute__((aligned(16))) bf16_t ol[];  // [kv_in]
+  __shared__ float scale[kMaxParts];
+  constexpr int U = 16;
+  const int h = blockIdx.x, tid = threadIdx.x;
+  const int lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), r = lane & 15, c = lane >> 4;
+  const int row0 = blockIdx.y * 64 + wave * 16, steps = kv_in >> 5;
+  const bool mine = row0 < a.vdim;
+  const bf16x8_t* w = reinterpret_cast<const bf16x8_t*>(reinterpret_cast<const bf16_t*>(a.w_uv) + h * w_block) +
+                      ((int64_t)(row0 >> 5) * (kv_in >> 4) + (c >> 1)) * 64 + 32 * (c & 1) + (row0 & 16) + r;
+  bf16x8_t wv[U];
+#pragma unroll
+  for (int i = 0; i < U; ++i)
+    if (mine && i < steps) wv[i] = w[(int64_t)i * 128];
+  int used;
+  const float inv = 1.0f / combine_factors(a, h, parts, scale, &used);
+  for (int col = tid; col < kv_in; col += 256) ol[col] = (bf16_t)(col < a.l.rank ? combine_column(a, h, parts, scale, used, col) * inv : 0.0f);
+  __syncthreads();
+  if (!mine) return;
+  const bf16x8_t* x = reinterpret_cast<const bf16x8_t*>(ol) + c;
+  f32x4_t acc = {0.0f, 0.0f, 0.0f, 0.0f};
+#pragma unroll
+  for (int i = 0; i < U; ++i)
+    if (i < steps) acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wv[i], x[i * 4], acc, 0, 0, 0);
+  for (int i = U; i < steps; ++i) acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(w[(int64_t)i * 128], x[i * 4], acc, 0, 0, 0);
+  if (r != 0) return;
+  bf16_t* const out = reinterpret_cast<bf16_t*>(a.ctx) + (int64_t)h * a.vdim + row0;
+#pragma unroll
+  for (int j = 0; j < 4; ++j)
+    if (row0 + 4 * c + j < a.vdim) out[4 * c + j] = (bf16_t)acc[j];
 }
 
 // --- with keys and values formed first -------------------------------------------------------------------------
@@ -647,16 +758,30 @@ int launch_latent_attention(const LatentAttnArgs& a, bool f32, hipStream_t st) {
     AWQ_HIP_TRY(hipGetLastError());
     return AWQ_OK;
   }
-  if (int rc = f32 ? launch_prepare<float, true>(a, st) : launch_prepare<bf16_t, true>(a, st)) return rc;
-  if (int rc = heads_product(a, a.w_uk, latent_uk_block(a), q_inputs(a), a.qa, a.ql, (int64_t)a.heads * a.l.row(), a.l.row(),
-                             a.l.rank, f32, st))
-    return rc;
-  if (on_matrix_cores(a, f32)) {
+  const bool cores = on_matrix_cores(a, f32);
+  if (a.M == 1 && cores && a.dim % kDenseKAlign == 0 && ((a.dim + a.l.rot) & 7) == 0 && ((uintptr_t)a.q & 15) == 0) {
+    const int chunks = (a.l.rank + 63) / 64;
+    hipLaunchKernelGGL(latent_query_one_kernel, dim3((unsigned)a.heads, (unsigned)(chunks + (a.down ? 1 : 0))), dim3(256),
+                       (size_t)(a.l.rot + 2) * 4, st, a, latent_uk_block(a), chunks);
+    AWQ_HIP_TRY(hipGetLastError());
+  } else {
+    if (int rc = f32 ? launch_prepare<float, true>(a, st) : launch_prepare<bf16_t, true>(a, st)) return rc;
+    if (int rc = heads_product(a, a.w_uk, latent_uk_block(a), q_inputs(a), a.qa, a.ql, (int64_t)a.heads * a.l.row(), a.l.row(),
+                               a.l.rank, f32, st))
+      return rc;
+  }
+  if (cores) {
     AWQ_REQUIRE(a.parts, "no scratch for the parts");
     const int parts = parts_of(a, a.M, a.pos.dyn ? a.max_pos : a.pos.pos0 + a.M);
     const int rp = a.l.rank_padded();
     if (int rc = rp <= 128 ? launch_rows<1>(a, parts, st) : rp <= 256 ? launch_rows<2>(a, parts, st) : launch_rows<4>(a, parts, st))
       return rc;
+    if (a.M == 1) {
+      hipLaunchKernelGGL(latent_value_one_kernel, dim3((unsigned)a.heads, (unsigned)((a.vdim + 63) / 64)), dim3(256),
+                         (size_t)v_inputs(a) * 2, st, a, parts, (int)v_inputs(a), latent_uv_block(a));
+      AWQ_HIP_TRY(hipGetLastError());
+      return AWQ_OK;
+    }
     hipLaunchKernelGGL(latent_combine_kernel, dim3((unsigned)(a.M * a.heads)), dim3(256), 0, st, a, parts, (int)v_inputs(a));
   } else {
     const size_t lds = (size_t)(a.l.row() + 256 + 4) * 4;

@@ -110,7 +110,7 @@ def test_the_test_models_tell_mistakes_apart(name, monkeypatch):
     assert moved(patch=("gated_state", forget)) > 0.1
     assert moved(patch=("norm", lambda x, g, eps: plain.rms(x, eps) * g)) > 0.1
     assert moved(patch=("rotate", lambda x, p, base: x)) > 0.1
-    assert moved(mixers("gla", lambda l: l["mixer"].update(tau=2 * l["mixer"]["tau"]))) > 0.1
+    assert moved(mixers("gla", lambda l: l["mixer"].update(tau=0.25 * l["mixer"]["tau"]))) > 0.1
     assert moved(change_w=without("lower")) > 0.1
     assert moved(change_w=without("f.b", "a2.b")) > 0.1
     assert moved(change_w=without("correction")) > 0.1
