@@ -4,8 +4,8 @@ framework's closest one) at equal width, heads, vocabulary and number of layers.
 
 Random weights, written once as a model folder and opened the way a user's folder is.  Four layers take every mechanism:
 gated linear attention with a dense feed-forward, latent attention, latent attention on the latents of the layer ahead,
-and HGRN2, the last three with routed experts.  A token meets as many feed-forward weights in an expert layer as five
-quarters of the dense one has (four experts and the shared one, each with three matrices of 3/4 width: 11.25 width^2; dense 6).
+and HGRN2, the last three with routed experts.  A token meets up to 11.25 width^2
+feed-forward weights in an expert layer (four experts and the shared one, each three matrices of 3/4 width), 6 in the dense one.
 
 Run on the GPU box: python bench.py --mode tudasun [--tudasun-sizes 2048,4096] [--tudasun-only]
 """

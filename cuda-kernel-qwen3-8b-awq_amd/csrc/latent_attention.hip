@@ -74,23 +74,21 @@ __device__ __forceinline__ void append_row(const LatentAttnArgs& a, int t, int p
   }
 }
 
-// blockIdx.x: token, blockIdx.y: kPrepareHeads heads, and behind the last heads the token's cache row.  INTO: the
+// blockIdx.x: token, blockIdx.y: `per` heads, and behind the last heads the token's cache row.  INTO: the
 // unrotated parts go to qa, padded to `kq` inputs a head, the rotated ones to their place in ql; otherwise the rotated parts
 // are rotated in place.
-constexpr int kPrepareHeads = 4;
-
 template <typename T, bool INTO>
-__global__ __launch_bounds__(256) void latent_prepare_kernel(LatentAttnArgs a, int kq) {
+__global__ __launch_bounds__(256) void latent_prepare_kernel(LatentAttnArgs a, int kq, int per) {
   extern __shared__ float turn[];
   __shared__ float sums[4];
   const int t = blockIdx.x, pos = a.pos.position() + t;
   turns_of(a, pos, turn);
-  const int h0 = blockIdx.y * kPrepareHeads;
+  const int h0 = blockIdx.y * per;
   if (h0 >= a.heads) {
     append_row<T>(a, t, pos, turn, sums);
     return;
   }
-  const int nh = min(kPrepareHeads, a.heads - h0);
+  const int nh = min(per, a.heads - h0);
   T* const q = reinterpret_cast<T*>(a.q) + t * a.ldq + (int64_t)h0 * (a.dim + a.l.rot);
   if constexpr (INTO) {
     T* const qa = reinterpret_cast<T*>(a.qa) + ((int64_t)t * a.heads + h0) * kq;
@@ -645,8 +643,9 @@ int parts_of(const LatentAttnArgs& a, int64_t M, int64_t keys) {
 
 template <typename T, bool INTO>
 int launch_prepare(const LatentAttnArgs& a, hipStream_t st) {
-  const dim3 g((unsigned)a.M, (unsigned)((a.heads + kPrepareHeads - 1) / kPrepareHeads + (a.down ? 1 : 0)));
-  hipLaunchKernelGGL((latent_prepare_kernel<T, INTO>), g, dim3(256), (size_t)(a.l.rot + 2) * 4, st, a, (int)q_inputs(a));
+  const int per = a.M >= 256 ? 32 : 4;  // heads of a workgroup: each forms the angles again
+  const dim3 g((unsigned)a.M, (unsigned)((a.heads + per - 1) / per + (a.down ? 1 : 0)));
+  hipLaunchKernelGGL((latent_prepare_kernel<T, INTO>), g, dim3(256), (size_t)(a.l.rot + 2) * 4, st, a, (int)q_inputs(a), per);
   AWQ_HIP_TRY(hipGetLastError());
   return AWQ_OK;
 }

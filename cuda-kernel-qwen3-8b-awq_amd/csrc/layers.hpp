@@ -1,6 +1,7 @@
 // Building blocks of decoder layers in bfloat16 or binary32, shared by the models that are described by a
 // config.json: dense products, grouped RMS norms with a causal convolution over time, attention over a sliding
-// window with a distance bias, linear attention with a decaying state, greedy sampling from binary32 logits.
+// window with a distance bias, attention over a shared latent, linear attention with a decaying state (a decay per head or
+// per channel), routed experts, gated and normalised sums into the residual stream, greedy sampling from binary32 logits.
 // Every size and constant is an argument.  `f32` selects the binary32 form of a launch: weights and activations
 // are then float, and no product runs at less than binary32; otherwise they are bfloat16 with binary32 sums.
 // What is stated as float here is float in both forms.

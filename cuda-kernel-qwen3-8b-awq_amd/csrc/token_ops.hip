@@ -221,7 +221,8 @@ bool launch_norm4(const NormConvArgs& a, hipStream_t st) {
   const int64_t part = a.width / a.groups;
   const int taps = a.conv ? a.taps : 0;
   if (part % 4 || a.ld % 4 || taps > 8) return false;
-  const int tokens = a.M == 1 ? 1 : a.M >= 512 ? 8 : a.M >= 64 ? 4 : 2;
+  // (without a convolution nothing is shared between the tokens of a workgroup but the weights)
+  const int tokens = a.M == 1 ? 1 : a.M >= 512 && taps > 0 ? 8 : a.M >= 64 ? 4 : 2;
   const dim3 g((unsigned)((a.M + tokens - 1) / tokens), (unsigned)a.groups);
   const dim3 b((unsigned)std::min<int64_t>(256, round_up(part / 4, 64)));
   switch (taps) {
